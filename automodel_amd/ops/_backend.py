@@ -17,11 +17,17 @@ import os
 import torch
 
 _SO_NAME = "libamd_ops.so"
+_DECODE_SO_NAME = "libamd_ops_decode.so"    # inference subset (ops/build.py --decode)
 _loaded: bool | None = None
 
 
 def so_path() -> str:
-    return os.path.join(os.path.dirname(os.path.abspath(__file__)), _SO_NAME)
+    """The full library if it is built, else the inference subset if that is,
+    else where the full library belongs."""
+    here = os.path.dirname(os.path.abspath(__file__))
+    full = os.path.join(here, _SO_NAME)
+    subset = os.path.join(here, _DECODE_SO_NAME)
+    return subset if os.path.exists(subset) and not os.path.exists(full) else full
 
 
 def ops_available() -> bool:

@@ -4,7 +4,11 @@ Compiles every ``csrc/*.hip`` + ``csrc/bind.cpp`` with hipcc in parallel and
 links ``automodel_amd/ops/libamd_ops.so``. No JIT cache: the .so lives in the
 package so it travels with the repo snapshot to GPU boxes.
 
-Usage: ``python -m automodel_amd.ops.build [--force]``
+``--decode`` links only the inference kernels (attention forward, latent
+attention, residual norms, decode GEMV) into ``libamd_ops_decode.so``: what a
+checkout with nothing built needs to generate, in a fraction of the time.
+
+Usage: ``python -m automodel_amd.ops.build [--force] [--decode]``
 """
 
 from __future__ import annotations
@@ -20,6 +24,9 @@ PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(PKG_DIR, "csrc")
 BUILD_DIR = os.path.join(PKG_DIR, "_build")
 SO_PATH = os.path.join(PKG_DIR, "libamd_ops.so")
+DECODE_SO_PATH = os.path.join(PKG_DIR, "libamd_ops_decode.so")
+DECODE_SOURCES = ("bind_decode.cpp", "flash_attn.hip", "gemv.hip",
+                  "latent_attn.hip", "latent_decode.hip", "residual_norm.hip")
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 
@@ -30,12 +37,16 @@ def _torch_paths() -> tuple[str, str]:
     return os.path.join(base, "include"), os.path.join(base, "lib")
 
 
-def _sources() -> list[str]:
+def _sources(decode_only: bool = False) -> list[str]:
     out = []
     for f in sorted(os.listdir(CSRC)):
-        if f.endswith((".hip", ".cpp")):
+        if f.endswith((".hip", ".cpp")) and (not decode_only or f in DECODE_SOURCES):
             out.append(os.path.join(CSRC, f))
     return out
+
+
+def _jobs() -> int:
+    return max(1, min(16, int(os.environ.get("MAX_JOBS") or os.cpu_count() or 8)))
 
 
 def _hash_inputs(srcs: list[str]) -> str:
@@ -48,17 +59,18 @@ def _hash_inputs(srcs: list[str]) -> str:
     return h.hexdigest()
 
 
-def build(force: bool = False, verbose: bool = True) -> str:
+def build(force: bool = False, verbose: bool = True, decode_only: bool = False) -> str:
     inc, lib = _torch_paths()
-    srcs = _sources()
-    stamp_path = os.path.join(BUILD_DIR, "stamp.json")
+    srcs = _sources(decode_only)
+    so_path = DECODE_SO_PATH if decode_only else SO_PATH
+    stamp_path = os.path.join(BUILD_DIR, os.path.basename(so_path) + ".stamp.json")
     digest = _hash_inputs(srcs)
-    if not force and os.path.exists(SO_PATH) and os.path.exists(stamp_path):
+    if not force and os.path.exists(so_path) and os.path.exists(stamp_path):
         try:
             if json.load(open(stamp_path)).get("digest") == digest:
                 if verbose:
-                    print(f"[amd_ops] up to date: {SO_PATH}")
-                return SO_PATH
+                    print(f"[amd_ops] up to date: {so_path}")
+                return so_path
         except Exception:
             pass
 
@@ -68,6 +80,9 @@ def build(force: bool = False, verbose: bool = True) -> str:
         f"-I{inc}", f"-I{os.path.join(inc, 'torch/csrc/api/include')}",
         "-D_GLIBCXX_USE_CXX11_ABI=1", "-DUSE_ROCM", "-D__HIP_PLATFORM_AMD__",
         "-Wno-unused-result",
+        # no v_pk_{add,mul,fma}_f32: some packed-f32 forms have returned wrong
+        # results on this hardware (the host pass warns about the feature name)
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     ]
 
     def compile_one(src: str) -> str:
@@ -80,24 +95,27 @@ def build(force: bool = False, verbose: bool = True) -> str:
             raise RuntimeError(f"hipcc failed for {src}:\n{r.stdout}\n{r.stderr}")
         return obj
 
-    with concurrent.futures.ThreadPoolExecutor(max_workers=min(8, len(srcs))) as ex:
+    with concurrent.futures.ThreadPoolExecutor(max_workers=min(_jobs(), len(srcs))) as ex:
         objs = list(ex.map(compile_one, srcs))
 
+    tmp_so = f"{so_path}.{os.getpid()}.tmp"    # a reader never sees half a library
     link = [
         "hipcc", f"--offload-arch={ARCH}", "-shared", "-fPIC", *objs,
         f"-L{lib}", "-ltorch", "-ltorch_hip", "-ltorch_cpu", "-lc10", "-lc10_hip",
-        "-lamdhip64", f"-Wl,-rpath,{lib}", "-o", SO_PATH,
+        "-lamdhip64", f"-Wl,-rpath,{lib}", "-o", tmp_so,
     ]
     if verbose:
-        print("[amd_ops] linking libamd_ops.so")
+        print(f"[amd_ops] linking {os.path.basename(so_path)}")
     r = subprocess.run(link, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
-    json.dump({"digest": digest}, open(stamp_path, "w"))
+    os.replace(tmp_so, so_path)
+    with open(stamp_path, "w") as f:
+        json.dump({"digest": digest}, f)
     if verbose:
-        print(f"[amd_ops] built {SO_PATH}")
-    return SO_PATH
+        print(f"[amd_ops] built {so_path}")
+    return so_path
 
 
 if __name__ == "__main__":
-    build(force="--force" in sys.argv)
+    build(force="--force" in sys.argv, decode_only="--decode" in sys.argv)

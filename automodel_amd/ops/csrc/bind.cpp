@@ -1,5 +1,7 @@
 // TORCH_LIBRARY registration for the amd_ops namespace.
 // Loaded from python via torch.ops.load_library (automodel_amd/ops/_backend.py).
+// The inference ops register in bind_decode.cpp, so that they can also be
+// linked into a library of their own (ops/build.py --decode).
 
 #include <torch/library.h>
 
@@ -29,10 +31,6 @@ TORCH_LIBRARY(amd_ops, m) {
       "float weight_decay) -> ()");
   m.impl("adamw_step", &amd_ops::adamw_step);
 
-  m.def(
-      "flash_attn_fwd(Tensor q, Tensor k, Tensor v, float scale, bool causal, "
-      "int q_start=0, Tensor? doc_start=None) -> (Tensor, Tensor)");
-  m.impl("flash_attn_fwd", &amd_ops::flash_attn_fwd);
   m.def(
       "flash_attn_bwd(Tensor dout, Tensor q, Tensor k, Tensor v, Tensor o, Tensor lse, "
       "float scale, bool causal, int q_start=0, Tensor? doc_start=None, "
@@ -69,9 +67,6 @@ TORCH_LIBRARY(amd_ops, m) {
   m.impl("lora_fused_fwd", &amd_ops::lora_fused_fwd);
   m.def("sgmv_fused_fwd(Tensor x, Tensor A, Tensor B, Tensor scales, Tensor offs, Tensor tile_map, Tensor? n_tiles=None) -> Tensor");
   m.impl("sgmv_fused_fwd", &amd_ops::sgmv_fused_fwd);
-
-  m.def("gemv_bf16(Tensor x, Tensor w, Tensor? bias) -> Tensor");
-  m.impl("gemv_bf16", &amd_ops::gemv_bf16);
 
   m.def("build_group_plan(Tensor counts, int M, int bm=128) -> (Tensor, Tensor, Tensor)");
   m.impl("build_group_plan", &amd_ops::build_group_plan);
