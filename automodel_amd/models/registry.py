@@ -388,6 +388,13 @@ def _ensure_builtin() -> None:
     except ImportError:
         pass
     try:
+        from automodel_amd.models.rezadra.model import RezadraForCausalLM
+
+        for name in RezadraForCausalLM.hf_architectures:
+            _REGISTRY[name] = RezadraForCausalLM
+    except ImportError:
+        pass
+    try:
         from automodel_amd.models.vlm.model import VLMForConditionalGeneration
 
         for name in VLMForConditionalGeneration.hf_architectures:
@@ -414,7 +421,9 @@ def build_model(
     if pretrained_path:
         with open(os.path.join(pretrained_path, "config.json")) as f:
             hf_cfg = json.load(f)
-        architecture = architecture or hf_cfg.get("architectures", ["LlamaForCausalLM"])[0]
+        # most configs list ``architectures``; some designs name one ``architecture``
+        architecture = architecture or hf_cfg.get(
+            "architectures", [hf_cfg.get("architecture", "LlamaForCausalLM")])[0]
         try:
             cls = get_model_class(architecture)
         except KeyError:
@@ -463,3 +472,14 @@ def build_model(
             model = model.to(device)
     model = model.to(dtype=torch_dtype)
     return model
+
+
+def load_pretrained(path: str, dtype: str = "bfloat16", device: str = "cuda",
+                    backend: dict | None = None) -> torch.nn.Module:
+    """Build the model of a local checkpoint directory and load its weights,
+    ready for inference on one device."""
+    from automodel_amd.checkpoint.hf_loader import load_hf_weights
+
+    model = build_model(pretrained_path=path, dtype=dtype, backend=backend)
+    load_hf_weights(model, path, device=device)
+    return model.to(device).eval()

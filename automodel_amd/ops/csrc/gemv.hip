@@ -9,7 +9,9 @@
 //     fully coalesced);
 //   * batch columns (B) accumulate in registers in the same pass, so W
 //     traffic is independent of B;
-//   * fp32 dot accumulation + wave reduce, lane 0 stores.
+//   * fp32 dot accumulation + wave reduce, lane 0 stores;
+//   * the epilogue can apply max(y, 0)^2 and can store f32 (residual inputs,
+//     logits) instead of bf16.
 // Grid = N/4 workgroups of 4 waves: N=4096 -> 1024 blocks >> 256 CUs.
 
 #include <torch/library.h>
@@ -26,7 +28,8 @@ namespace amd_ops {
 template <int B>
 __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
     const bf16* __restrict__ W, const bf16* __restrict__ x,
-    const bf16* __restrict__ bias, bf16* __restrict__ y, int N, int K) {
+    const bf16* __restrict__ bias, bf16* __restrict__ y, float* __restrict__ yf, bool relu2,
+    int N, int K) {
   const int lane = threadIdx.x & (WAVE_SIZE - 1);
   const int wid = blockIdx.x * (blockDim.x / WAVE_SIZE) + (threadIdx.x / WAVE_SIZE);
   const int row0 = 2 * wid;
@@ -59,15 +62,23 @@ __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
     const float t0 = wave_reduce_sum(acc0[b]);
     const float t1 = wave_reduce_sum(acc1[b]);
     if (lane == 0) {
-      y[(long)b * N + row0] = f2bf(t0 + (bias ? bf2f(bias[row0]) : 0.f));
-      if (two)
-        y[(long)b * N + row0 + 1] = f2bf(t1 + (bias ? bf2f(bias[row0 + 1]) : 0.f));
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        if (i && !two) break;
+        float t = (i ? t1 : t0) + (bias ? bf2f(bias[row0 + i]) : 0.f);
+        if (relu2) {
+          t = fmaxf(t, 0.f);
+          t *= t;
+        }
+        if (yf) yf[(long)b * N + row0 + i] = t;
+        else y[(long)b * N + row0 + i] = f2bf(t);
+      }
     }
   }
 }
 
 at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
-                     const c10::optional<at::Tensor>& bias) {
+                     const c10::optional<at::Tensor>& bias, bool relu2, bool out_f32) {
   TORCH_CHECK(x.is_cuda() && w.is_cuda(), "gemv_bf16: GPU tensors required");
   TORCH_CHECK(x.dtype() == at::kBFloat16 && w.dtype() == at::kBFloat16,
               "gemv_bf16: bf16 only");
@@ -76,9 +87,9 @@ at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
   TORCH_CHECK(w.size(1) == K, "K mismatch");
   TORCH_CHECK(B >= 1 && B <= 16, "gemv_bf16: B in [1,16], got ", B,
               " (larger batches belong on hipBLASLt)");
-  TORCH_CHECK(K % (WAVE_SIZE * 8) == 0, "gemv_bf16: K % 512 == 0, got ", K);
+  TORCH_CHECK(K % 8 == 0, "gemv_bf16: K % 8 == 0, got ", K);
   auto xc = x.contiguous(), wc = w.contiguous();
-  auto y = at::empty({B, N}, x.options());
+  auto y = at::empty({B, N}, x.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
   const bf16* bptr = nullptr;
   if (bias.has_value()) {
     TORCH_CHECK(bias->numel() == N && bias->dtype() == at::kBFloat16, "bias [N] bf16");
@@ -92,7 +103,8 @@ at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
   gemv_bf16_kernel<BB><<<grid, dim3(waves_per_block * WAVE_SIZE), 0, stream>>>( \
       reinterpret_cast<const bf16*>(wc.data_ptr()),                            \
       reinterpret_cast<const bf16*>(xc.data_ptr()), bptr,                      \
-      reinterpret_cast<bf16*>(y.data_ptr()), N, K)
+      out_f32 ? nullptr : reinterpret_cast<bf16*>(y.data_ptr()),               \
+      out_f32 ? y.data_ptr<float>() : nullptr, relu2, N, K)
   switch (B) {
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;

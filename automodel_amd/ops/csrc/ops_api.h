@@ -69,7 +69,8 @@ at::Tensor sgmv_fused_fwd(const at::Tensor& x, const at::Tensor& A,
                           const std::optional<at::Tensor>& n_tiles = std::nullopt);
 
 at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
-                     const c10::optional<at::Tensor>& bias);
+                     const c10::optional<at::Tensor>& bias, bool relu2 = false,
+                     bool out_f32 = false);
 
 std::tuple<at::Tensor, at::Tensor, at::Tensor> build_group_plan(
     const at::Tensor& counts, int64_t M, int64_t bm = 128);
@@ -91,5 +92,38 @@ at::Tensor transpose_bf16(const at::Tensor& in);
 at::Tensor permute_gather(const at::Tensor& x, const at::Tensor& src);
 at::Tensor unpermute_combine(const at::Tensor& yp, const at::Tensor& pos,
                              const at::Tensor& probs);
+
+// --- inference: f32 residual stream (residual_norm.hip) ---
+at::Tensor embed_rms_norm(const at::Tensor& ids, const at::Tensor& table, const at::Tensor& w,
+                          double eps);
+at::Tensor residual_rms_norm(const at::Tensor& x, const at::Tensor& w, double eps);
+at::Tensor residual_add_norm(at::Tensor x, const at::Tensor& y, const at::Tensor& w_post,
+                             double mult, double eps_post,
+                             const std::optional<at::Tensor>& w_next, double eps_next);
+at::Tensor concat_cast(const at::Tensor& a, const at::Tensor& b, bool to_bf16);
+at::Tensor relu2_(at::Tensor x);
+
+// --- inference: latent attention (latent_attn.hip, latent_decode.hip) ---
+std::tuple<at::Tensor, at::Tensor, at::Tensor> latent_prep(
+    const at::Tensor& qkv, const at::Tensor& w, double eps, const at::Tensor& cos,
+    const at::Tensor& sin, const at::Tensor& pos, const std::optional<at::Tensor>& slot,
+    const std::optional<at::Tensor>& cache, int64_t heads, int64_t dn, int64_t dr,
+    int64_t head_pad, int64_t rows_pad);
+std::tuple<at::Tensor, at::Tensor> latent_assemble(const at::Tensor& kv, const at::Tensor& kr,
+                                                   int64_t heads, int64_t dn, int64_t dv,
+                                                   int64_t k_pad, int64_t v_pad, int64_t n_tok);
+at::Tensor attn_rows(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
+                     const at::Tensor& base, const at::Tensor& count, double scale, bool out_f32);
+at::Tensor latent_decode_prep(const at::Tensor& qkv, const at::Tensor& w_uk,
+                              const at::Tensor& w_norm, double eps, const at::Tensor& cos,
+                              const at::Tensor& sin, const at::Tensor& pos, const at::Tensor& slot,
+                              at::Tensor cache, int64_t heads, int64_t dn, int64_t dr);
+std::tuple<at::Tensor, at::Tensor> latent_decode_attn(const at::Tensor& q, const at::Tensor& cache,
+                                                      const at::Tensor& slot, const at::Tensor& pos,
+                                                      int64_t rank, int64_t rot, double scale,
+                                                      int64_t splits);
+at::Tensor latent_decode_combine(const at::Tensor& part_o,
+                                 const std::optional<at::Tensor>& part_ml, const at::Tensor& w_uv,
+                                 int64_t dv);
 
 }  // namespace amd_ops

@@ -20,14 +20,18 @@ def build_rope_cache(
     base: float = 10000.0,
     scaling: dict | None = None,
     device=None,
+    angle_dtype: torch.dtype = torch.float32,
 ) -> tuple[torch.Tensor, torch.Tensor]:
     """Return (cos, sin) of shape [max_seq_len, head_dim], fp32.
+
+    ``angle_dtype`` is the precision of frequencies and angles before the
+    cosine; float64 keeps far positions exact to the last fp32 bit.
 
     ``scaling`` supports HF rope_scaling dicts: llama3-style
     {rope_type: "llama3", factor, low_freq_factor, high_freq_factor,
     original_max_position_embeddings} and linear {rope_type: "linear", factor}.
     """
-    inv_freq = 1.0 / (base ** (torch.arange(0, head_dim, 2, dtype=torch.float32) / head_dim))
+    inv_freq = 1.0 / (base ** (torch.arange(0, head_dim, 2, dtype=angle_dtype) / head_dim))
     if scaling:
         rope_type = scaling.get("rope_type", scaling.get("type", "default"))
         if rope_type == "linear":
@@ -81,11 +85,11 @@ def build_rope_cache(
                     (1 - smooth) * scaled + smooth * inv_freq,
                 ),
             )
-    t = torch.arange(max_seq_len, dtype=torch.float32)
+    t = torch.arange(max_seq_len, dtype=angle_dtype)
     freqs = torch.outer(t, inv_freq)
     emb = torch.cat([freqs, freqs], dim=-1)
     scale = locals().get("attention_scaling", 1.0)
-    cos, sin = emb.cos() * scale, emb.sin() * scale
+    cos, sin = (emb.cos() * scale).float(), (emb.sin() * scale).float()
     if device is not None:
         cos, sin = cos.to(device), sin.to(device)
     return cos, sin

@@ -16,17 +16,17 @@ import torch.nn.functional as F
 _PAD_TO = {5: 8, 6: 8, 7: 8, 9: 16, 10: 16, 11: 16, 12: 16, 13: 16, 14: 16, 15: 16}
 
 
-def gemv_bf16(x2d: torch.Tensor, w: torch.Tensor,
-              bias: torch.Tensor | None = None) -> torch.Tensor:
+def gemv_bf16(x2d: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None,
+              relu2: bool = False, out_f32: bool = False) -> torch.Tensor:
     """y = x2d @ w.T via the HIP kernel; pads odd batch sizes to a
-    compiled template instance."""
+    compiled template instance. Epilogues: max(y, 0)^2, f32 output."""
     from automodel_amd.ops._backend import hip_ops
 
     B = x2d.shape[0]
     tgt = _PAD_TO.get(B, B)
     if tgt != B:
         x2d = F.pad(x2d, (0, 0, 0, tgt - B))
-    y = hip_ops().gemv_bf16(x2d, w, bias)
+    y = hip_ops().gemv_bf16(x2d, w, bias, relu2, out_f32)
     return y[:B] if tgt != B else y
 
 
@@ -39,6 +39,33 @@ def _gemv_eligible(x: torch.Tensor, w: torch.Tensor) -> bool:
     # measured on MI355X (profiles/README.md): the wave-per-row GEMV beats
     # hipBLASLt up to ~4 rows; above that the library's m-tiled path wins
     return rows <= 4 and x.shape[-1] % 512 == 0
+
+
+def project(lin: nn.Module, x: torch.Tensor, relu2: bool = False,
+            out_f32: bool = False) -> torch.Tensor:
+    """``lin(x)`` for packed rows x [T, K], optionally followed by max(y, 0)^2
+    and optionally in float32 (a residual input or logits must not be rounded
+    to bf16 on the way out of the accumulator).
+
+    Inference on the GPU: few bf16 rows take the GEMV with its fused epilogue,
+    others the library GEMM. Wrapped layers (adapters) and autograd take the
+    module itself."""
+    from automodel_amd.ops import residual_norm as rn
+
+    if type(lin) not in (nn.Linear, DecodeLinear) or lin.bias is not None or not rn.use_hip(x):
+        y = lin(x)
+        y = rn.relu2(y) if relu2 else y
+        return y.float() if out_f32 else y
+    w = lin.weight
+    if x.shape[0] == 0:
+        return x.new_empty(0, w.shape[0], dtype=torch.float32 if out_f32 else x.dtype)
+    if x.dtype == torch.bfloat16 and x.shape[0] <= 4 and x.shape[1] % 8 == 0:
+        return gemv_bf16(x, w, None, relu2, out_f32)
+    if out_f32 and x.dtype == torch.bfloat16:
+        y = torch.mm(x, w.t(), out_dtype=torch.float32)
+    else:
+        y = F.linear(x, w)
+    return rn.relu2(y) if relu2 else y
 
 
 class DecodeLinear(nn.Linear):

@@ -10,6 +10,9 @@ Used via a context so module signatures stay unchanged (same pattern as the
 varlen context in ops/attention.py): attention layers call
 ``maybe_update_kv(k, v)`` after rope; under an active cache it returns the
 full prefix k/v and records the new slots; otherwise it is a no-op.
+
+Models with another kind of cache build it in ``model.make_cache(batch,
+max_len)`` (``make_cache`` below asks for it); latent attention's is here too.
 """
 
 from __future__ import annotations
@@ -18,10 +21,14 @@ from contextlib import contextmanager
 
 import torch
 
-_ACTIVE: "KVCache | None" = None
+from automodel_amd.ops.latent_attention import LatentAttentionSpec, PackedStep
+
+_ACTIVE: "KVCache | LatentKVCache | None" = None
 
 
 class KVCache:
+    ragged = False          # one position for the whole rectangular batch
+
     def __init__(self, n_layers: int, batch: int, max_len: int,
                  n_kv_heads: int, head_dim: int, device, dtype):
         shape = (n_layers, batch, max_len, n_kv_heads, head_dim)
@@ -120,6 +127,88 @@ class StaticKVCache(KVCache):
         self.pos_dev.add_(1)
 
 
+class LatentKVCache:
+    """Cache of latent-attention models: per LAYER RUN (a looped layer counts
+    once per pass) one [slots, max_len, row] tensor whose rows hold a token's
+    normed latent and its shared rotated key.
+
+    Sequences live in slots with their own lengths, so a batch may be ragged
+    and may shrink: ``plan_prompts`` / ``plan_decode`` describe the next
+    forward as packed tokens, ``free`` gives a finished sequence's slot back.
+    A slot needs no clearing before reuse: a sequence only ever reads the rows
+    it has written itself.
+    """
+
+    ragged = True
+
+    def __init__(self, specs: list[LatentAttentionSpec], n_slots: int, max_len: int,
+                 device, dtype):
+        self.n_slots, self.max_len = n_slots, max_len
+        self.rows = [torch.zeros(n_slots, max_len, s.cache_width, device=device, dtype=dtype)
+                     for s in specs]
+        self.device = torch.device(device)
+        self.lens = [0] * n_slots
+        self._free = list(range(n_slots - 1, -1, -1))
+        self.step: PackedStep | None = None
+        self._layer = 0
+
+    # -- slots -----------------------------------------------------------------
+    def alloc(self, n: int) -> list[int]:
+        if n > len(self._free):
+            raise RuntimeError(f"latent cache: {n} slots wanted, {len(self._free)} free "
+                               f"of {self.n_slots}")
+        return [self._free.pop() for _ in range(n)]
+
+    def free(self, slots: list[int]) -> None:
+        for s in slots:
+            assert s not in self._free, f"slot {s} freed twice"
+            self.lens[s] = 0
+            self._free.append(s)
+
+    # -- steps -----------------------------------------------------------------
+    def plan_prompts(self, slots: list[int], lengths: list[int],
+                     logit_rows: list[int] | None = None) -> PackedStep:
+        """Whole prompts of ``lengths`` tokens from position 0 of ``slots``."""
+        if not lengths or min(lengths) < 1 or max(lengths) > self.max_len:
+            raise ValueError(f"prompt lengths {lengths} do not fit max_len {self.max_len}")
+        if any(self.lens[s] for s in slots):
+            raise ValueError("a prompt must start an empty slot")
+        self.step = PackedStep.for_prompts(lengths, self.device, slots, logit_rows)
+        self._pending = list(zip(slots, lengths))
+        return self.step
+
+    def plan_decode(self, slots: list[int]) -> PackedStep:
+        """One more token for each of ``slots``."""
+        pos = [self.lens[s] for s in slots]
+        if not pos or max(pos) >= self.max_len:
+            raise RuntimeError("KV cache overflow")
+        both = torch.tensor([pos, slots], dtype=torch.int32).to(self.device)
+        self.step = PackedStep(positions=both[0], slots=both[1], prompt=False)
+        self._pending = [(s, 1) for s in slots]
+        return self.step
+
+    def begin_forward(self) -> None:
+        self._layer = 0
+
+    def next_layer(self) -> torch.Tensor:
+        """Rows of the next layer run, consumed in execution order."""
+        self._layer += 1
+        return self.rows[self._layer - 1]
+
+    def advance(self) -> None:
+        """Account for the planned step after its forward."""
+        assert self._layer == len(self.rows), (
+            "model did not consult the latent cache in every layer run")
+        for s, n in self._pending:
+            self.lens[s] += n
+        self._pending = []
+
+    def advance_device(self) -> None:
+        """Move a decode plan to the next position on the device: the only
+        per-step bookkeeping of a captured decode step."""
+        self.step.positions.add_(1)
+
+
 @contextmanager
 def kv_cache_context(cache: KVCache):
     global _ACTIVE
@@ -131,7 +220,7 @@ def kv_cache_context(cache: KVCache):
         _ACTIVE = prev
 
 
-def active_kv_cache() -> KVCache | None:
+def active_kv_cache() -> KVCache | LatentKVCache | None:
     return _ACTIVE
 
 
@@ -143,3 +232,10 @@ def maybe_update_kv(k: torch.Tensor, v: torch.Tensor):
     pos = _ACTIVE.pos
     k_full, v_full = _ACTIVE.update(k, v)
     return k_full, v_full, pos
+
+
+def make_cache(model, batch: int, max_len: int, static: bool = False):
+    """The cache ``model`` decodes with: its own, or the dense K/V pair."""
+    if hasattr(model, "make_cache"):
+        return model.make_cache(batch, max_len)
+    return (StaticKVCache if static else KVCache).for_model(model, batch, max_len)
