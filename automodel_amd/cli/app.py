@@ -4,6 +4,8 @@ Reference behavior: nemo_automodel/cli/app.py:95-159 (parse YAML, resolve the
 ``recipe:`` target, dispatch to a launcher). Usage:
 
     automodel <cfg.yaml> [--nproc-per-node N] [--a.b.c=v ...]
+    automodel capabilities [ARCHITECTURE]
+    automodel generate --model DIR --prompt-ids 5,17,3 [--prompt-ids ...]
 """
 
 from __future__ import annotations
@@ -44,6 +46,54 @@ def query_capabilities(arch: str | None = None) -> None:
         print(f"{name}: {flags}")
 
 
+def generate_command(argv: list[str]) -> None:
+    """Generate from a local checkpoint: one line of JSON per prompt. Prompts
+    of any lengths run as batches through the cached decode path."""
+    import argparse
+    import json
+
+    import torch
+
+    from automodel_amd.models.registry import load_pretrained
+    from automodel_amd.utils.generation import generate_batch
+
+    ap = argparse.ArgumentParser(prog="automodel generate", description=generate_command.__doc__)
+    ap.add_argument("--model", required=True, help="folder with config.json and safetensors")
+    ap.add_argument("--prompt-ids", action="append", default=[], metavar="IDS",
+                    help="comma-separated token ids; may be given several times")
+    ap.add_argument("--prompt", action="append", default=[], metavar="TEXT",
+                    help="text, with --tokenizer")
+    ap.add_argument("--tokenizer", default=None, help="tokenizer folder")
+    ap.add_argument("--max-new-tokens", type=int, default=32)
+    ap.add_argument("--max-batch", type=int, default=16)
+    ap.add_argument("--temperature", type=float, default=0.0)
+    ap.add_argument("--eos", type=int, default=None, help="end token id")
+    ap.add_argument("--dtype", default=None, choices=["bfloat16", "float32"])
+    args = ap.parse_args(argv)
+
+    tok = None
+    if args.tokenizer:
+        from automodel_amd.models.auto_tokenizer import build_tokenizer
+
+        tok = build_tokenizer(args.tokenizer)
+    if args.prompt and tok is None:
+        ap.error("--prompt needs --tokenizer")
+    prompts = [[int(t) for t in p.split(",")] for p in args.prompt_ids]
+    prompts += [tok.encode(p) for p in args.prompt]
+    if not prompts:
+        ap.error("give --prompt-ids or --prompt")
+    device = "cuda" if torch.cuda.is_available() else "cpu"
+    dtype = args.dtype or ("bfloat16" if device == "cuda" else "float32")
+    model = load_pretrained(args.model, dtype=dtype, device=device)
+    outs = generate_batch(model, prompts, args.max_new_tokens, args.temperature, args.eos,
+                          args.max_batch)
+    for p, o in zip(prompts, outs):
+        rec = {"prompt_ids": p, "output_ids": o}
+        if tok is not None:
+            rec["text"] = tok.decode(o)
+        print(json.dumps(rec))
+
+
 def main(argv: list[str] | None = None) -> None:
     argv = argv if argv is not None else sys.argv[1:]
     if not argv or argv[0] in ("-h", "--help"):
@@ -51,6 +101,9 @@ def main(argv: list[str] | None = None) -> None:
         return
     if argv[0] == "capabilities":
         query_capabilities(argv[1] if len(argv) > 1 else None)
+        return
+    if argv[0] == "generate":
+        generate_command(argv[1:])
         return
     cfg_path = argv[0]
     rest = argv[1:]

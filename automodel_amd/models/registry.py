@@ -479,7 +479,10 @@ def load_pretrained(path: str, dtype: str = "bfloat16", device: str = "cuda",
     """Build the model of a local checkpoint directory and load its weights,
     ready for inference on one device."""
     from automodel_amd.checkpoint.hf_loader import load_hf_weights
+    from automodel_amd.models.hf_fallback import HFFallbackForCausalLM
 
-    model = build_model(pretrained_path=path, dtype=dtype, backend=backend)
-    load_hf_weights(model, path, device=device)
+    # not a meta build: tables and other buffers outside the checkpoint must exist
+    model = build_model(pretrained_path=path, dtype=dtype, backend=backend, meta_init=False)
+    if not isinstance(model, HFFallbackForCausalLM):    # which loads its own weights
+        load_hf_weights(model, path)
     return model.to(device).eval()

@@ -184,7 +184,7 @@ int row_threads(int W, int V, long rows) {
 void check_rows(const at::Tensor& x, const char* who) {
   TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.is_contiguous() && x.scalar_type() == at::kFloat,
               who, ": residual must be a contiguous f32 [T, W] GPU tensor");
-  TORCH_CHECK(x.size(1) >= 1 && x.size(1) <= 36864, who, ": width out of range");
+  TORCH_CHECK(x.size(1) >= 1 && x.size(1) <= 16384, who, ": width out of range");
 }
 void check_vec(const at::Tensor& w, int64_t n, const char* who) {
   TORCH_CHECK(w.is_cuda() && w.is_contiguous() && w.numel() == n &&

@@ -4,7 +4,8 @@ Reference behavior: nemo_automodel/components/speculative/serve_target.py
 (serve the target model for decode evaluation; production serving defers to
 vLLM/SGLang). This server wraps the in-tree KV-cached / hipGraph decode
 (utils/generation.py) behind an OpenAI-ish completion endpoint — enough for
-eval loops and demo serving; continuous batching is round-2.
+eval loops and demo serving. A request may carry several prompts of any lengths
+(``batch_prompt_ids``); they are generated together.
 
 Run:  python -m automodel_amd.serving.server --config model.yaml --port 8000
 Test: build_app(model, tokenizer) + fastapi.testclient (CPU-tested).
@@ -25,6 +26,7 @@ def build_app(model, tokenizer, use_cache: bool = True, use_graph: bool = False,
 
     from automodel_amd.utils.generation import (
         generate,
+        generate_batch,
         generate_cached,
         generate_graphed,
     )
@@ -38,6 +40,7 @@ def build_app(model, tokenizer, use_cache: bool = True, use_graph: bool = False,
     class GenRequest(BaseModel):
         prompt: str | None = None
         prompt_ids: list[int] | None = None
+        batch_prompt_ids: list[list[int]] | None = None
         max_new_tokens: int = 64
         temperature: float = 0.0
         speculative: bool = False      # greedy draft-verify (needs a proposer
@@ -51,8 +54,17 @@ def build_app(model, tokenizer, use_cache: bool = True, use_graph: bool = False,
 
     @app.post("/generate")
     def gen(req: GenRequest):
-        assert (req.prompt is None) != (req.prompt_ids is None), \
-            "give prompt XOR prompt_ids"
+        given = [req.prompt, req.prompt_ids, req.batch_prompt_ids]
+        assert sum(g is not None for g in given) == 1, \
+            "give one of prompt, prompt_ids, batch_prompt_ids"
+        if req.batch_prompt_ids is not None:
+            with gen_lock:
+                new = generate_batch(model, req.batch_prompt_ids, req.max_new_tokens,
+                                     temperature=req.temperature)
+            resp = {"prompt_len": [len(p) for p in req.batch_prompt_ids], "output_ids": new}
+            if tokenizer is not None:
+                resp["text"] = [tokenizer.decode(n) for n in new]
+            return resp
         if req.prompt_ids is not None:
             ids = req.prompt_ids
         else:
@@ -98,7 +110,7 @@ def main(argv=None):
     import uvicorn
 
     from automodel_amd.config.loader import load_yaml_config
-    from automodel_amd.models.registry import build_model
+    from automodel_amd.models.registry import build_model, load_pretrained
 
     ap = argparse.ArgumentParser()
     ap.add_argument("--config", required=True, help="model YAML (model: block)")
@@ -114,13 +126,16 @@ def main(argv=None):
 
     cfg = load_yaml_config(args.config)
     device = "cuda" if torch.cuda.is_available() else "cpu"
-    model = build_model(
-        config=cfg.model.config.to_dict(),
-        architecture=cfg.model.get("architecture"),
-        pretrained_path=cfg.model.get("pretrained_path"),
-        dtype=cfg.model.get("dtype", "bfloat16" if device == "cuda" else "float32"),
-        meta_init=False, device=device,
-    ).eval()
+    dtype = cfg.model.get("dtype", "bfloat16" if device == "cuda" else "float32")
+    pretrained = cfg.model.get("pretrained_path")
+    if pretrained:
+        model = load_pretrained(pretrained, dtype=dtype, device=device)
+    else:
+        model = build_model(
+            config=cfg.model.config.to_dict(),
+            architecture=cfg.model.get("architecture"),
+            dtype=dtype, meta_init=False, device=device,
+        ).eval()
     tokenizer = None
     tok_path = cfg.get_by_dotted("model.tokenizer_path", None)
     if tok_path:

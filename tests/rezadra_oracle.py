@@ -58,15 +58,14 @@ def latent_attention(h, w, p, mixer, eps, fault=None):
     v = (c @ w[p + "uv"].T).view(T, H, dv)
     out = torch.empty(T, H, dv, dtype=h.dtype)
     for i in range(T):
-        lo, hi = 0, i + 1
-        if fault == "first_key_lost" and i > 0:
-            lo = 1
-        if fault == "own_key_lost" and i > 0:
-            hi = i
+        seen = list(range(i + 1))
+        if isinstance(fault, tuple) and i > 0:      # ("lost", key) or ("lost", "own")
+            lost = i if fault[1] == "own" else fault[1]
+            seen = [j for j in seen if j != lost]
         for a in range(H):
-            s = (kn[lo:hi, a] @ qn[i, a] + kr[lo:hi] @ qr[i, a]) * scale
+            s = (kn[seen, a] @ qn[i, a] + kr[seen] @ qr[i, a]) * scale
             e = torch.exp(s - s.max())
-            out[i, a] = (e / e.sum()) @ v[lo:hi, a]
+            out[i, a] = (e / e.sum()) @ v[seen, a]
     return out.reshape(T, H * dv) @ w[p + "o"].T
 
 
