@@ -16,6 +16,8 @@ TORCH_LIBRARY_FRAGMENT(amd_ops, m) {
       "gemv_bf16(Tensor x, Tensor w, Tensor? bias, bool relu2=False, bool out_f32=False) "
       "-> Tensor");
   m.impl("gemv_bf16", &amd_ops::gemv_bf16);
+  m.def("gemm_skinny_bf16(Tensor x, Tensor w, bool relu2, bool out_f32) -> Tensor");
+  m.impl("gemm_skinny_bf16", &amd_ops::gemm_skinny_bf16);
 
   m.def("embed_rms_norm(Tensor ids, Tensor table, Tensor w, float eps) -> Tensor");
   m.impl("embed_rms_norm", &amd_ops::embed_rms_norm);

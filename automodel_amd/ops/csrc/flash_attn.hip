@@ -326,7 +326,10 @@ std::tuple<at::Tensor, at::Tensor> flash_attn_fwd(
 #define FA_FWD_CASE(A, C)                                                             \
   if (!done && Dqk == A && Dv == C) {                                                 \
     done = true;                                                                      \
-    if (varlen) {                                                                     \
+    if (varlen && Sq % (8 * QBLK) == 0) {                                             \
+      launch_fwd<A, C, 8, true>(q, k, v, out, lse, ds_ptr, B, Sq, Skv, Hq, Hk,        \
+                                (int)q_start, (float)scale, causal, stream);          \
+    } else if (varlen) {                                                              \
       launch_fwd<A, C, 4, true>(q, k, v, out, lse, ds_ptr, B, Sq, Skv, Hq, Hk,        \
                                 (int)q_start, (float)scale, causal, stream);          \
     } else if (Sq % (8 * QBLK) == 0) {                                                \

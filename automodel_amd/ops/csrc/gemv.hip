@@ -23,6 +23,16 @@
 
 namespace amd_ops {
 
+typedef __bf16 gemv_bf16x2 __attribute__((ext_vector_type(2)));
+typedef __bf16 gemv_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float gemv_f32x4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ float dot2(const bf16x8& a, const bf16x8& b, int j, float c) {
+  const gemv_bf16x8 av = __builtin_bit_cast(gemv_bf16x8, a), bv = __builtin_bit_cast(gemv_bf16x8, b);
+  return __builtin_amdgcn_fdot2_f32_bf16(gemv_bf16x2{av[2 * j], av[2 * j + 1]},
+                                         gemv_bf16x2{bv[2 * j], bv[2 * j + 1]}, c, false);
+}
+
 // Two rows per wave: doubles outstanding b128 loads per wave (latency
 // hiding for the short 8-iteration K sweep at K=4096).
 template <int B>
@@ -48,10 +58,9 @@ __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
       const bf16x8 xv = *reinterpret_cast<const bf16x8*>(x + (long)b * K + k);
       float d0 = 0.f, d1 = 0.f;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const float xf = bf2f(xv.v[j]);
-        d0 += bf2f(w0.v[j]) * xf;
-        d1 += bf2f(w1.v[j]) * xf;
+      for (int j = 0; j < 4; ++j) {               // v_dot2_f32_bf16: f32 accumulation
+        d0 = dot2(w0, xv, j, d0);
+        d1 = dot2(w1, xv, j, d1);
       }
       acc0[b] += d0;
       acc1[b] += d1;
@@ -114,6 +123,122 @@ at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
     case 16: LAUNCH(16); break;
     default: TORCH_CHECK(false, "gemv_bf16: pad B to one of 1,2,3,4,8,16 (python wrapper does)");
   }
+#undef LAUNCH
+  HIP_CHECK_KERNEL();
+  return y;
+}
+
+// ---------------------------------------------------------------------------
+// Skinny GEMM for decode batches of 5..64 rows: the same weight stream, with
+// the products on the matrix cores. A workgroup owns 16 rows of W; its waves
+// split K and reduce through LDS, so that even N = 4096 fills the chip. Per
+// 64-wide K chunk a lane loads 32 contiguous bytes of its W row (a full line
+// per four lanes) and the same K range of the x rows; the K order inside a
+// chunk is the same permutation for both, which the dot product does not see.
+// ---------------------------------------------------------------------------
+template <int NB, int WAVES>
+__global__ __launch_bounds__(WAVES * WAVE_SIZE) void gemm_skinny_kernel(
+    const bf16* __restrict__ W, const bf16* __restrict__ x, bf16* __restrict__ y,
+    float* __restrict__ yf, bool relu2, int B, int N, int K) {
+  constexpr int U = NB <= 2 ? 4 : 2;              // chunks in flight
+  __shared__ float red[WAVES][16][16 * NB + 1];
+  const int lane = threadIdx.x & (WAVE_SIZE - 1), wid = threadIdx.x / WAVE_SIZE;
+  const int lo16 = lane & 15, hi4 = lane >> 4;
+  const int n0 = blockIdx.x * 16;
+  const bf16* wrow = W + (long)min(n0 + lo16, N - 1) * K + hi4 * 16;
+  const bf16* xrow[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) xrow[b] = x + (long)min(b * 16 + lo16, B - 1) * K + hi4 * 16;
+  gemv_f32x4 acc[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) acc[b] = gemv_f32x4{0.f, 0.f, 0.f, 0.f};
+
+  const int full = K / 64;                        // whole chunks, split over the waves
+  const int per = (full + WAVES - 1) / WAVES;
+  int c = wid * per;
+  const int c_hi = min(c + per, full);
+  for (; c + U <= c_hi; c += U) {
+    gemv_bf16x8 w[U][2], v[U][NB][2];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const long k = (long)(c + u) * 64;
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        w[u][i] = *reinterpret_cast<const gemv_bf16x8*>(wrow + k + i * 8);
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+          v[u][b][i] = *reinterpret_cast<const gemv_bf16x8*>(xrow[b] + k + i * 8);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int b = 0; b < NB; ++b)
+          acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[u][i], v[u][b][i], acc[b], 0, 0, 0);
+  }
+  // leftover chunks, and for the last wave the K tail (8-wide pieces past K
+  // contribute zeros)
+  const int c_end = wid == WAVES - 1 ? (K + 63) / 64 : c_hi;
+  if (wid == WAVES - 1 && c > full) c = full;
+  for (; c < c_end; ++c) {
+    const long k = (long)c * 64;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const bool in = k + hi4 * 16 + i * 8 < K;   // K % 8 == 0: all 8 or none
+      gemv_bf16x8 zero = {};
+      const gemv_bf16x8 w = in ? *reinterpret_cast<const gemv_bf16x8*>(wrow + k + i * 8) : zero;
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        const gemv_bf16x8 v =
+            in ? *reinterpret_cast<const gemv_bf16x8*>(xrow[b] + k + i * 8) : zero;
+        acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, v, acc[b], 0, 0, 0);
+      }
+    }
+  }
+#pragma unroll
+  for (int b = 0; b < NB; ++b)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) red[wid][hi4 * 4 + i][b * 16 + lo16] = acc[b][i];
+  __syncthreads();
+  for (int i = threadIdx.x; i < 256 * NB; i += WAVES * WAVE_SIZE) {
+    const int row = i & 15, col = i >> 4;
+    if (n0 + row >= N || col >= B) continue;
+    float t = 0.f;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) t += red[w][row][col];
+    if (relu2) {
+      t = fmaxf(t, 0.f);
+      t *= t;
+    }
+    const long o = (long)col * N + n0 + row;
+    if (yf) yf[o] = t;
+    else y[o] = f2bf(t);
+  }
+}
+
+at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32) {
+  TORCH_CHECK(x.is_cuda() && w.is_cuda() && x.dtype() == at::kBFloat16 &&
+                  w.dtype() == at::kBFloat16 && x.dim() == 2 && w.dim() == 2,
+              "gemm_skinny_bf16: x [B,K], w [N,K] bf16 on the GPU");
+  const int B = (int)x.size(0), K = (int)x.size(1), N = (int)w.size(0);
+  TORCH_CHECK(w.size(1) == K && K % 8 == 0 && K >= 8 && N >= 1, "gemm_skinny_bf16: K % 8 == 0");
+  TORCH_CHECK(B >= 1 && B <= 64, "gemm_skinny_bf16: 1..64 rows, got ", B);
+  auto xc = x.contiguous(), wc = w.contiguous();
+  auto y = at::empty({B, N}, x.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  auto stream = c10::hip::getCurrentHIPStream();
+#define LAUNCH(NB, WAVES)                                                                    \
+  gemm_skinny_kernel<NB, WAVES>                                                              \
+      <<<dim3((N + 15) / 16), dim3(WAVES * WAVE_SIZE), 0, stream>>>(                         \
+          reinterpret_cast<const bf16*>(wc.data_ptr()),                                      \
+          reinterpret_cast<const bf16*>(xc.data_ptr()),                                      \
+          out_f32 ? nullptr : reinterpret_cast<bf16*>(y.data_ptr()),                         \
+          out_f32 ? y.data_ptr<float>() : nullptr, relu2, B, N, K)
+  const bool deep = K >= 2048;
+  if (B <= 16) { if (deep) LAUNCH(1, 8); else LAUNCH(1, 4); }
+  else if (B <= 32) { if (deep) LAUNCH(2, 8); else LAUNCH(2, 4); }
+  else { if (deep) LAUNCH(4, 8); else LAUNCH(4, 4); }
 #undef LAUNCH
   HIP_CHECK_KERNEL();
   return y;

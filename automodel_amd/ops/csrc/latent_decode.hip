@@ -136,8 +136,10 @@ __device__ __forceinline__ lat_bf16x4 lds_tr16(const char* p) {
       (lds_ptr)(__attribute__((address_space(3))) char*)const_cast<char*>(p));
 }
 
-// NCT: 16-column value tiles per wave (4 waves cover RP <= 64 * NCT)
-template <int MT, int NCT>
+// NCT: 16-column value tiles per wave (4 waves cover RP <= 64 * NCT).
+// NPM: bound on the 16-byte pieces of a key tile per thread (exactly C / 32).
+// The next tile travels through registers while the current one is used.
+template <int MT, int NCT, int NPM>
 __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ cache, const int* __restrict__ slot,
     const int* __restrict__ pos, float* __restrict__ part_o, float* __restrict__ part_ml,
@@ -163,16 +165,35 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
   const bf16* base = cache + (long)(n > 0 ? sl : 0) * max_len * C;
 
   const int vecs = C / 8;                         // 16-byte pieces per row
-  for (int i = tid; i < 16 * MT * vecs; i += 256) {
-    const int row = i / vecs, c = (i % vecs) * 8;
-    bf16x8 x;
-    if (h0 + row < H) {
-      x = *reinterpret_cast<const bf16x8*>(q + ((long)r * H + h0 + row) * C + c);
-    } else {
+  const int np = C / 32;                          // pieces of a 64-row tile per thread
+  const unsigned magic = ((1u << 20) + vecs - 1) / vecs;    // i / vecs, exact for i < 64 vecs
+  uint4 pre[NPM];
+  auto fetch = [&](int t) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) x.v[j] = f2bf(0.f);
+    for (int j = 0; j < NPM; ++j) {
+      if (j < np) {                               // uniform
+        const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+        const int key = min(t * LD_KEYS + (int)row, n - 1);   // rows past the end: masked below
+        pre[j] = *reinterpret_cast<const uint4*>(base + (long)key * C + c * 8);
+      }
     }
-    *reinterpret_cast<bf16x8*>(qt + row * KS + c * 2) = x;
+  };
+  if (t_lo < t_hi) fetch(t_lo);
+  // queries: 16 MT rows of the same width, np / (4 / MT) pieces per thread
+  for (int i0 = tid; i0 < 16 * MT * vecs; i0 += 1024) {
+    uint4 x[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+      x[j] = uint4{0u, 0u, 0u, 0u};
+      if (i < 16u * MT * vecs && h0 + (int)row < H)
+        x[j] = *reinterpret_cast<const uint4*>(q + ((long)r * H + h0 + row) * C + c * 8);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+      if (i < 16u * MT * vecs) *reinterpret_cast<uint4*>(qt + row * KS + c * 16) = x[j];
+    }
   }
 
   lat_f32x4 acc[MT][NCT];
@@ -187,13 +208,15 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
 
   for (int t = t_lo; t < t_hi; ++t) {
     const int k0 = t * LD_KEYS;
-    for (int i = tid; i < LD_KEYS * vecs; i += 256) {
-      const int row = i / vecs, c = (i % vecs) * 8;
-      const int key = min(k0 + row, n - 1);       // rows past the end are masked below
-      *reinterpret_cast<bf16x8*>(kt + row * KS + c * 2) =
-          *reinterpret_cast<const bf16x8*>(base + (long)key * C + c);
+#pragma unroll
+    for (int j = 0; j < NPM; ++j) {
+      if (j < np) {
+        const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+        *reinterpret_cast<uint4*>(kt + row * KS + c * 16) = pre[j];
+      }
     }
     __syncthreads();
+    if (t + 1 < t_hi) fetch(t + 1);
 
     // scores: D[head = 4*hi4 + i][key = lo16] of this wave's 16 keys
     lat_f32x4 s[MT];
@@ -293,12 +316,10 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
         part_ml[o * 2] = m_run[a][i];
         part_ml[o * 2 + 1] = l;
       }
-      if (t_lo < t_hi) {
 #pragma unroll
-        for (int c = 0; c < NCT; ++c) {
-          const int n0 = (wid * NCT + c) * 16;
-          if (n0 < RP) part_o[o * RP + n0 + lo16] = acc[a][c][i];
-        }
+      for (int c = 0; c < NCT; ++c) {             // an empty split stores zeros
+        const int n0 = (wid * NCT + c) * 16;
+        if (n0 < RP) part_o[o * RP + n0 + lo16] = acc[a][c][i];
       }
     }
 }
@@ -341,23 +362,44 @@ __global__ __launch_bounds__(256) void latent_decode_combine_kernel(
     }
     __syncthreads();
   }
-  for (int i = tid; i < RT * rank; i += 256) {
-    const int rr = i / rank, c = i % rank, r = r0 + rr;
-    float a = 0.f;
-    if (r < R) {
-      const float* po = part_o + ((long)r * H + h) * S * stride + c;
-      if (part_ml) {
-        for (int s = 0; s < S; ++s) {
-          const float w = wt[rr * S + s];
-          if (w != 0.f) a = fmaf(w, po[(long)s * stride], a);   // empty splits are not read
-        }
-      } else {
-        a = po[0];
+  // merge: a thread owns 4 columns of a row (1 if the rank is no multiple of
+  // 4); where that leaves threads idle, they share a column's splits
+  constexpr int M = V == 1 ? 1 : 4;
+  const int cols = rank / M, items = RT * cols;
+  const int groups = min(max(256 / items, 1), S);
+  float* half = wt + RT * S;                      // [groups][items][M], groups > 1 only
+  for (int i0 = tid; i0 < items * groups; i0 += 256) {
+    const int i = i0 % items, g = i0 / items;
+    const int rr = i / cols, c = (i % cols) * M, r = min(r0 + rr, R - 1);
+    const float* po = part_o + ((long)r * H + h) * S * stride + c;
+    float a[M];
+#pragma unroll
+    for (int j = 0; j < M; ++j) a[j] = 0.f;
+    if (part_ml) {
+#pragma unroll 8
+      for (int s = g; s < S; s += groups) {
+        const float w = r0 + rr < R ? wt[rr * S + s] : 0.f;
+        const LatPack<float, M> x = *reinterpret_cast<const LatPack<float, M>*>(po + (long)s * stride);
+#pragma unroll
+        for (int j = 0; j < M; ++j) a[j] = fmaf(w, x.v[j], a[j]);
       }
+    } else {
+#pragma unroll
+      for (int j = 0; j < M; ++j) a[j] = po[j];
     }
-    ol[i] = a;
+    float* dst = groups > 1 ? half + ((long)g * items + i) * M : ol + rr * rank + c;
+#pragma unroll
+    for (int j = 0; j < M; ++j) dst[j] = a[j];
   }
   __syncthreads();
+  if (groups > 1) {                               // uniform
+    for (int i = tid; i < items * M; i += 256) {
+      float a = 0.f;
+      for (int g = 0; g < groups; ++g) a += half[g * items * M + i];
+      ol[i] = a;
+    }
+    __syncthreads();
+  }
   const int v_lo = blockIdx.x * LC_ROWS, v_hi = min(v_lo + LC_ROWS, dv);
   for (int v = v_lo + wid; v < v_hi; v += 4) {
     const T* w = w_uv + ((long)h * dv + v) * rank;
@@ -460,26 +502,34 @@ std::tuple<at::Tensor, at::Tensor> latent_decode_attn(const at::Tensor& q, const
   auto part_ml = at::empty({R, H, splits, 2}, part_o.options());
   if (R == 0) return {part_o, part_ml};
   auto stream = c10::hip::getCurrentHIPStream();
-#define LAUNCH(MT, NCT)                                                                          \
+  // head tiles per workgroup: both share the staged keys, but two workgroups
+  // are better where the splits alone leave CUs idle
+  const bool two = H > 16 && R * splits * ((H + 31) / 32) >= 256;
+#define LAUNCH1(MT, NCT, NPM)                                                                    \
   do {                                                                                           \
     const size_t smem = (LD_KEYS + 16 * MT) * (C * 2 + 16) + 16 * MT * (LD_PSTRIDE + 16);        \
     TORCH_CHECK(smem <= LDS_MAX, "latent_decode_attn: tile exceeds LDS");                        \
     static const hipError_t attr_ = hipFuncSetAttribute(                                         \
-        reinterpret_cast<const void*>(&latent_decode_attn_kernel<MT, NCT>),                      \
+        reinterpret_cast<const void*>(&latent_decode_attn_kernel<MT, NCT, NPM>),                 \
         hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS_MAX);                               \
     TORCH_CHECK(attr_ == hipSuccess, "latent_decode_attn: LDS attribute");                       \
-    latent_decode_attn_kernel<MT, NCT>                                                           \
+    latent_decode_attn_kernel<MT, NCT, NPM>                                                      \
         <<<dim3(splits, (H + 16 * MT - 1) / (16 * MT), R), dim3(256), smem, stream>>>(           \
             reinterpret_cast<const bf16*>(q.data_ptr()),                                         \
             reinterpret_cast<const bf16*>(cache.data_ptr()), slot.data_ptr<int>(),               \
             pos.data_ptr<int>(), part_o.data_ptr<float>(), part_ml.data_ptr<float>(),            \
             (int)cache.size(0), (int)cache.size(1), (int)H, (int)RP, (int)C, (float)scale);      \
   } while (0)
-  if (H <= 16) {
-    if (RP <= 128) LAUNCH(1, 2); else if (RP <= 256) LAUNCH(1, 4); else LAUNCH(1, 8);
-  } else {
-    if (RP <= 128) LAUNCH(2, 2); else if (RP <= 256) LAUNCH(2, 4); else LAUNCH(2, 8);
-  }
+#define LAUNCH(NCT, NPM)                                                                         \
+  do {                                                                                           \
+    if (two) LAUNCH1(2, NCT, NPM); else LAUNCH1(1, NCT, NPM);                                    \
+  } while (0)
+  TORCH_CHECK(C / 32 <= 26, "latent_decode_attn: latent and rotated key too wide");
+  if (RP <= 128 && C <= 256) LAUNCH(2, 8);
+  else if (RP <= 256 && C <= 384) LAUNCH(4, 12);
+  else if (C <= 640) LAUNCH(8, 20);
+  else LAUNCH(8, 26);
+#undef LAUNCH1
 #undef LAUNCH
   HIP_CHECK_KERNEL();
   return {part_o, part_ml};
@@ -515,7 +565,7 @@ at::Tensor latent_decode_combine(const at::Tensor& part_o,
           reinterpret_cast<TT*>(out.data_ptr()), (int)R, (int)H, (int)dv, (int)rank, (int)n,    \
           (int)S)
   ROW_TILE(R, {
-    const size_t smem = (RT * rank + RT * S) * sizeof(float);
+    const size_t smem = (RT * rank + RT * S + 1024) * sizeof(float);
     TORCH_CHECK(smem <= 64 * 1024, "latent_decode_combine: rank or splits too large");
     if (w_uv.scalar_type() == at::kBFloat16) {
       if (vec) LAUNCH(bf16, 8); else LAUNCH(bf16, 1);

@@ -71,6 +71,7 @@ at::Tensor sgmv_fused_fwd(const at::Tensor& x, const at::Tensor& A,
 at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
                      const c10::optional<at::Tensor>& bias, bool relu2 = false,
                      bool out_f32 = false);
+at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32);
 
 std::tuple<at::Tensor, at::Tensor, at::Tensor> build_group_plan(
     const at::Tensor& counts, int64_t M, int64_t bm = 128);

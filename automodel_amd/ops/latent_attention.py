@@ -20,13 +20,13 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
+import numpy as np
 import torch
 import torch.nn.functional as F
 
 from automodel_amd.ops._backend import hip_ops
 from automodel_amd.ops.attention import (
     _target_dims,
-    doc_bounds_from_cu,
     flash_attention_varlen,
 )
 from automodel_amd.ops.residual_norm import rms_f32, use_hip
@@ -34,8 +34,9 @@ from automodel_amd.ops.rope import build_rope_cache
 
 FLASH_MAX_HEAD_DIM = 256
 MFMA_MAX_RANK = 512
+MFMA_MAX_CACHE_WIDTH = 832
 _KEYS_PER_TILE = 64                 # latent_decode.hip LD_KEYS
-_TARGET_WORKGROUPS = 512            # two per CU
+_TARGET_WORKGROUPS = 256            # one per CU: a staged tile fills most of its LDS
 
 
 def pad32(n: int) -> int:
@@ -78,35 +79,29 @@ class PackedStep:
     slots: torch.Tensor | None = None
     prompt: bool = True
     cu_seqlens: torch.Tensor | None = None      # int32 [n + 1], prompt steps
-    doc_start: torch.Tensor | None = None       # int32 [rows padded to 128]
-    base: torch.Tensor | None = None            # int64 [T] first key row
-    count: torch.Tensor | None = None           # int32 [T] visible keys
+    doc_start: torch.Tensor | None = None       # int32 [rows padded to 256]
     logit_rows: torch.Tensor | None = None      # rows whose logits are wanted
     n_seqs: int = 1
 
     @classmethod
     def for_prompts(cls, lengths: list[int], device, slots: list[int] | None = None,
                     logit_rows: list[int] | None = None) -> "PackedStep":
-        lens = torch.tensor(lengths, dtype=torch.int64)
-        cu = torch.zeros(len(lengths) + 1, dtype=torch.int64)
-        cu[1:] = lens.cumsum(0)
+        lens = np.asarray(lengths, dtype=np.int32)
+        cu = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
         total = int(cu[-1])
-        ds, _ = doc_bounds_from_cu(cu, total + (-total) % 128)
-        start = ds[:total].long()
-        pos = torch.arange(total) - start
-
-        def dev(x, dtype):
-            return x.to(device=device, dtype=dtype)
-
-        return cls(
-            positions=dev(pos, torch.int32),
-            slots=None if slots is None else dev(
-                torch.repeat_interleave(torch.tensor(slots), lens), torch.int32),
-            cu_seqlens=dev(cu, torch.int32), doc_start=dev(ds, torch.int32),
-            base=dev(start, torch.int64), count=dev(pos + 1, torch.int32),
-            logit_rows=None if logit_rows is None else dev(
-                torch.tensor(logit_rows), torch.int64),
-            n_seqs=len(lengths))
+        start = np.repeat(cu[:-1], lens)
+        parts = {
+            "positions": np.arange(total, dtype=np.int32) - start,
+            # padding rows form a document of their own after the last one
+            "doc_start": np.concatenate([start, np.full((-total) % 256, total, np.int32)]),
+            "cu_seqlens": cu,
+            "slots": None if slots is None else np.repeat(np.asarray(slots, np.int32), lens),
+            "logit_rows": None if logit_rows is None else np.asarray(logit_rows, np.int32),
+        }
+        parts = {k: v for k, v in parts.items() if v is not None}
+        flat = torch.from_numpy(np.concatenate(list(parts.values())).astype(np.int32)).to(device)
+        views = dict(zip(parts, flat.split([len(v) for v in parts.values()])))
+        return cls(**views, n_seqs=len(lengths))
 
 
 def rope_half_tables(rot_dim: int, n: int, base: float, device) -> tuple[torch.Tensor, torch.Tensor]:
@@ -153,7 +148,8 @@ def latent_attention_prompt(qkv, norm_w, w_kv_b, spec: LatentAttentionSpec, rope
         flash = (qkv.dtype == torch.bfloat16 and dn + spec.rot_dim <= FLASH_MAX_HEAD_DIM
                  and dv <= FLASH_MAX_HEAD_DIM)
         kd, vd = _target_dims(dn + spec.rot_dim, dv) if flash else (dn + spec.rot_dim, dv)
-        rows = T + (-T) % 128 if flash else T
+        # rows in whole workgroups of the flash kernel: 8 waves of 32, 4 if few
+        rows = T + (-T) % (256 if T > 1024 else 128) if flash else T
         q, c, kr = ops.latent_prep(
             qkv, norm_w, spec.eps, rope[0], rope[1], step.positions,
             step.slots if cache is not None else None, cache,
@@ -164,7 +160,8 @@ def latent_attention_prompt(qkv, norm_w, w_kv_b, spec: LatentAttentionSpec, rope
             o, _ = ops.flash_attn_fwd(q[None], k[None], v[None], spec.scale, True, 0,
                                       step.doc_start if step.n_seqs > 1 else None)
             return o[0, :T, :, :dv].reshape(T, H * dv)
-        o = ops.attn_rows(q, k, v, step.base, step.count, spec.scale, False)
+        o = ops.attn_rows(q, k, v, step.doc_start[:T].long(), step.positions + 1, spec.scale,
+                          False)
         return o.view(T, H * dv)
 
     qn, qr, c, kr = _split_torch(qkv, norm_w, spec, rope, step.positions)
@@ -192,7 +189,7 @@ def decode_splits(rows: int, heads: int, max_len: int) -> int:
     than there are key tiles. Depends on capacities only, so that it is the
     same on every replay of a captured step."""
     groups = -(-heads // (16 if heads <= 16 else 32))
-    want = -(-_TARGET_WORKGROUPS // max(1, rows * groups))
+    want = _TARGET_WORKGROUPS // max(1, rows * groups)
     return max(1, min(want, -(-max_len // _KEYS_PER_TILE), 64))
 
 
@@ -207,7 +204,8 @@ def latent_attention_decode(qkv, norm_w, w_kv_b, spec: LatentAttentionSpec, rope
         ops = hip_ops()
         q = ops.latent_decode_prep(qkv, w_uk, norm_w, spec.eps, rope[0], rope[1],
                                    step.positions, step.slots, cache, H, dn, spec.rot_dim)
-        if qkv.dtype == torch.bfloat16 and rank <= MFMA_MAX_RANK:
+        if (qkv.dtype == torch.bfloat16 and rank <= MFMA_MAX_RANK
+                and spec.cache_width <= MFMA_MAX_CACHE_WIDTH):
             part, ml = ops.latent_decode_attn(
                 q, cache, step.slots, step.positions, rank, spec.rot_dim, spec.scale,
                 decode_splits(R, H, cache.shape[1]))

@@ -47,8 +47,8 @@ def project(lin: nn.Module, x: torch.Tensor, relu2: bool = False,
     and optionally in float32 (a residual input or logits must not be rounded
     to bf16 on the way out of the accumulator).
 
-    Inference on the GPU: few bf16 rows take the GEMV with its fused epilogue,
-    others the library GEMM. Wrapped layers (adapters) and autograd take the
+    Inference on the GPU: up to 4 bf16 rows take the GEMV, up to 64 the skinny
+    MFMA GEMM, both with fused epilogues; more take the library GEMM. Wrapped layers (adapters) and autograd take the
     module itself."""
     from automodel_amd.ops import residual_norm as rn
 
@@ -59,8 +59,12 @@ def project(lin: nn.Module, x: torch.Tensor, relu2: bool = False,
     w = lin.weight
     if x.shape[0] == 0:
         return x.new_empty(0, w.shape[0], dtype=torch.float32 if out_f32 else x.dtype)
-    if x.dtype == torch.bfloat16 and x.shape[0] <= 4 and x.shape[1] % 8 == 0:
-        return gemv_bf16(x, w, None, relu2, out_f32)
+    if x.dtype == torch.bfloat16 and x.shape[0] <= 64 and x.shape[1] % 8 == 0:
+        if x.shape[0] <= 4:
+            return gemv_bf16(x, w, None, relu2, out_f32)
+        from automodel_amd.ops._backend import hip_ops
+
+        return hip_ops().gemm_skinny_bf16(x, w, relu2, out_f32)
     if out_f32 and x.dtype == torch.bfloat16:
         y = torch.mm(x, w.t(), out_dtype=torch.float32)
     else:

@@ -15,6 +15,7 @@ from __future__ import annotations
 
 from collections.abc import Sequence
 
+import numpy as np
 import torch
 
 from automodel_amd.utils.kv_cache import kv_cache_context, make_cache
@@ -76,11 +77,11 @@ class DecodeSession:
             cache.begin_forward()
             if cache.ragged:
                 handles = cache.alloc(len(prompts))
-                flat = [t for p in prompts for t in p]
+                flat = np.concatenate([np.asarray(p, dtype=np.int64) for p in prompts])
                 starts = [sum(lens[:i]) for i in range(len(lens))]
                 rows = [s + j for s, w in zip(starts, want) for j in w]
                 cache.plan_prompts(handles, lens, rows)
-                logits = self.model(torch.tensor([flat], device=self.device))
+                logits = self.model(torch.from_numpy(flat).to(self.device).unsqueeze(0))
                 cache.advance()
             else:
                 if self.live or len(set(lens)) != 1:

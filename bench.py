@@ -51,6 +51,11 @@ def parse_args():
                    help="disable fused qkv/gate_up projections")
     p.add_argument("--profile-steps", type=int, default=0,
                    help="if >0, run this many steps (no JSON contract) for rocprof")
+    p.add_argument("--serving", default=None, choices=["rezadra"],
+                   help="instead of the training step, measure this design's prefill and "
+                        "decode throughput beside the closest in-tree models (one GPU)")
+    p.add_argument("--serving-part", default="all",
+                   help="all | prefill | decode | e.g. decode:rezadra:8b-layer:1")
     return p.parse_args()
 
 
@@ -113,6 +118,11 @@ ARCH_BY_MODEL = {"qwen3_moe_30b": "Qwen3MoeForCausalLM",
 
 def main():
     args = parse_args()
+    if args.serving:
+        from benchmarks.serving_bench import main as serving_main
+
+        serving_main(args.serving_part, args.steps, args.warmup)
+        return
     world = int(os.environ.get("WORLD_SIZE", 1))
     rank = int(os.environ.get("RANK", 0))
 

@@ -1,0 +1,152 @@
+"""Prefill and decode throughput of Rezadra beside the closest in-tree models.
+
+Same width, layer runs, attention heads and parameter count per layer, random
+weights, bf16, one GPU:
+
+* prefill against DeepSeek-V3 (latent attention, every layer dense), which
+  shares the flash kernel; both without logits for the inner positions;
+* decode against Llama (the family with a captured decode step), both as
+  hipGraph replays of the one-token step.
+
+Run as ``python bench.py --serving rezadra`` (``--serving-part`` picks one
+part, e.g. for a profile). One JSON line per measurement.
+"""
+
+from __future__ import annotations
+
+import json
+import time
+
+import torch
+
+SIZES = {
+    # width, heads, layer runs, feed-forward of the squared-ReLU MLP (two
+    # matrices) and of the gated MLP (three), equal in parameters
+    "2b-layer": dict(width=2048, heads=16, runs=12, ff=9216, gated=6144, kv_heads=4),
+    "8b-layer": dict(width=4096, heads=32, runs=12, ff=21504, gated=14336, kv_heads=8),
+}
+VOCAB = 32768
+MLA = dict(kv_lora_rank=512, qk_nope_head_dim=128, qk_rope_head_dim=64, v_head_dim=128)
+
+
+def _build(architecture: str, config: dict, linears_for_decode: bool = False):
+    from automodel_amd.models.registry import build_model
+
+    model = build_model(config=config, architecture=architecture, dtype="bfloat16",
+                        meta_init=True)
+    model.init_weights(device="cuda")
+    model = model.to(torch.bfloat16).eval()
+    if linears_for_decode:
+        from automodel_amd.serving import swap_linears_for_decode
+
+        swap_linears_for_decode(model)
+    return model
+
+
+def rezadra(size: dict):
+    layers, loop = size["runs"] - 4, {"start": 2, "stop": 6, "times": 2}
+    return _build("Rezadra", dict(
+        vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=layers, loop=loop,
+        num_attention_heads=size["heads"], intermediate_size=size["ff"],
+        residual_multiplier=0.5, **MLA))
+
+
+def deepseek(size: dict):
+    return _build("DeepseekV3ForCausalLM", dict(
+        vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=size["runs"],
+        num_attention_heads=size["heads"], intermediate_size=size["gated"], q_lora_rank=0,
+        first_k_dense_replace=size["runs"], max_position_embeddings=8192, **MLA))
+
+
+def llama(size: dict, batch: int):
+    return _build("LlamaForCausalLM", dict(
+        vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=size["runs"],
+        num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=128,
+        intermediate_size=size["gated"], max_position_embeddings=8192), batch <= 4)
+
+
+def _timed(fn, steps: int, warmup: int) -> float:
+    for _ in range(warmup):
+        fn()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / steps
+
+
+def _say(**rec) -> None:
+    print(json.dumps(rec), flush=True)
+
+
+@torch.no_grad()
+def prefill(name: str, which: str, batch: int, seq: int, steps: int, warmup: int) -> None:
+    from automodel_amd.utils.generation import DecodeSession
+
+    size = SIZES[name]
+    torch.manual_seed(0)
+    ids = torch.randint(0, VOCAB, (batch, seq))
+    if which == "rezadra":
+        session = DecodeSession(rezadra(size), batch, seq)
+        prompts = ids.tolist()
+
+        def run():
+            session.release(session.prefill(prompts)[0])
+    else:
+        model, dev_ids = deepseek(size), ids.cuda()
+
+        def run():
+            hidden = model(dev_ids, return_hidden=True)
+            return model.lm_head(hidden[:, -1])
+    dt = _timed(run, steps, warmup)
+    _say(part="prefill", model=which, size=name, batch=batch, seq=seq,
+         ms=round(dt * 1e3, 2), tokens_per_s=round(batch * seq / dt))
+
+
+@torch.no_grad()
+def decode(name: str, which: str, batch: int, context: int, steps: int, warmup: int) -> None:
+    from automodel_amd.utils.generation import DecodeSession, _GraphStep
+    from automodel_amd.utils.kv_cache import kv_cache_context
+
+    size = SIZES[name]
+    torch.manual_seed(0)
+    model = rezadra(size) if which == "rezadra" else llama(size, batch)
+    session = DecodeSession(model, batch, context + steps + warmup + 8, static=True)
+    handles, logits = session.prefill(torch.randint(0, VOCAB, (batch, context)).tolist())
+    with kv_cache_context(session.cache):
+        step = _GraphStep(session, handles, logits.argmax(-1, keepdim=True))
+        del logits
+        s = torch.cuda.Stream()
+        s.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(s):
+            step()
+        torch.cuda.current_stream().wait_stream(s)
+        graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(graph):
+            step()
+        dt = _timed(graph.replay, steps, warmup)
+    _say(part="decode", model=which, size=name, batch=batch, context=context,
+         ms_per_step=round(dt * 1e3, 3), tokens_per_s=round(batch / dt, 1))
+
+
+PREFILL = [("2b-layer", 1, 4096), ("2b-layer", 8, 1024), ("8b-layer", 1, 4096),
+           ("8b-layer", 4, 2048)]
+DECODE = [("2b-layer", 1, 2048), ("2b-layer", 16, 2048), ("8b-layer", 1, 4096),
+          ("8b-layer", 4, 4096), ("8b-layer", 32, 4096)]
+
+
+def main(part: str = "all", steps: int = 10, warmup: int = 3) -> None:
+    assert torch.cuda.is_available(), "the serving bench needs a GPU"
+    for kind, fn, cases, peer in (("prefill", prefill, PREFILL, "deepseek-v3-dense"),
+                                  ("decode", decode, DECODE, "llama")):
+        if part not in ("all", kind) and not part.startswith(kind + ":"):
+            continue
+        only = part.split(":")[1:]                    # e.g. decode:rezadra:8b-layer:1
+        n = steps if kind == "prefill" else 10 * steps
+        for name, batch, length in cases:
+            for which in ("rezadra", peer):
+                tag = [which, name, str(batch)]
+                if tag[:len(only)] == only:
+                    fn(name, which, batch, length, n, warmup)
+                    torch.cuda.empty_cache()

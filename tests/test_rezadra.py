@@ -236,6 +236,7 @@ MIXERS = {
     "plain": make_layer(heads=3, dim=16, rot_dim=8, vdim=24, kv_rank=32)["mixer"],
     "odd": make_layer(heads=2, dim=9, rot_dim=6, vdim=5, kv_rank=19, base=50.0)["mixer"],
     "large": make_layer(heads=17, dim=128, rot_dim=64, vdim=128, kv_rank=512)["mixer"],
+    "rotation-wider": make_layer(heads=3, dim=16, rot_dim=160, vdim=16, kv_rank=512)["mixer"],
     "value-wider": make_layer(heads=2, dim=8, rot_dim=56, vdim=120, kv_rank=200)["mixer"],
 }
 
@@ -308,6 +309,60 @@ def test_faults_would_show():
     for fault in (("lost", 0), ("lost", "own"), "latent_not_normed", "key_not_rotated"):
         bad = oracle.forward(ids, weights("mixed"), ALL["mixed"], fault=fault)
         assert rel(bad, want_logits("mixed", ids)) > 5 * TOL["bfloat16"], fault
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("splits", [1, 2, 3, 7, 33, 64])
+@pytest.mark.parametrize("heads,rank,rot", [(5, 64, 32), (16, 200, 6), (33, 512, 64), (70, 96, 96)])
+@torch.no_grad()
+def test_decode_attention_splits(splits, heads, rank, rot):
+    """Any number of splits, many tiles per split, empty splits, rows of
+    different lengths in scattered slots; rows beyond a length are poison."""
+    from automodel_amd.ops._backend import hip_ops
+
+    g = torch.Generator().manual_seed(splits)
+    lens, slots, n_slots, max_len = [1, 63, 64, 65, 500, 640, 321], [6, 0, 3, 8, 2, 7, 1], 9, 640
+    RP, C = la.pad32(rank), la.pad32(rank) + la.pad32(rot)
+    cache = torch.full((n_slots, max_len, C), 1e4).bfloat16()
+    q = torch.zeros(len(lens), heads, C).bfloat16()
+    q[:, :, :rank] = torch.randn(len(lens), heads, rank, generator=g).bfloat16()
+    q[:, :, RP:RP + rot] = torch.randn(len(lens), heads, rot, generator=g).bfloat16()
+    for s, n in zip(slots, lens):
+        cache[s, :n] = torch.randn(n, C, generator=g).bfloat16()
+    scale = 1.5 * (rank + rot) ** -0.5
+    w_uv = torch.randn(heads * 12, rank, generator=g).bfloat16() / rank ** 0.5
+    pos = torch.tensor(lens, dtype=torch.int32, device="cuda") - 1
+    slot = torch.tensor(slots, dtype=torch.int32, device="cuda")
+    part, ml = hip_ops().latent_decode_attn(q.cuda(), cache.cuda(), slot, pos, rank, rot, scale,
+                                            splits)
+    got = hip_ops().latent_decode_combine(part, ml, w_uv.cuda(), 12)
+    want = []
+    for r, (s, n) in enumerate(zip(slots, lens)):
+        k = cache[s, :n].double()
+        p = torch.softmax(q[r].double() @ k.T * scale, -1)
+        o = p @ k[:, :rank]
+        want.append(torch.einsum("hr,hvr->hv", o, w_uv.double().view(heads, 12, rank)).reshape(-1))
+    close(got, torch.stack(want), "bfloat16")
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("rows", [1, 3, 4, 5, 16, 17, 32, 33, 64])
+@pytest.mark.parametrize("n,k", [(16, 8), (50, 72), (1000, 192), (129, 2048), (257, 4168)])
+@pytest.mark.parametrize("relu2,f32", [(False, False), (True, False), (False, True)])
+@torch.no_grad()
+def test_decode_projection(rows, n, k, relu2, f32):
+    from automodel_amd.serving.decode_linear import project
+
+    g = torch.Generator().manual_seed(rows + n)
+    lin = torch.nn.Linear(k, n, bias=False)
+    lin.weight.data = torch.randn(n, k, generator=g) / k ** 0.5
+    lin = lin.bfloat16()
+    x = torch.randn(rows, k, generator=g).bfloat16()
+    want = x.double() @ lin.weight.double().T
+    want = oracle.relu_squared(want) if relu2 else want
+    got = project(lin.cuda(), x.cuda(), relu2, f32)
+    assert got.dtype == (torch.float32 if f32 else torch.bfloat16)
+    assert rel(got, want) < (1e-5 if f32 else 6e-3)
 
 
 @on_each
