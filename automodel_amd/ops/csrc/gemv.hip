@@ -131,83 +131,90 @@ at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
 // ---------------------------------------------------------------------------
 // Skinny GEMM for decode batches of 5..64 rows: the same weight stream, with
 // the products on the matrix cores. A workgroup owns 16 rows of W; its waves
-// split K and reduce through LDS, so that even N = 4096 fills the chip. Per
-// 64-wide K chunk a lane loads 32 contiguous bytes of its W row (a full line
-// per four lanes) and the same K range of the x rows; the K order inside a
-// chunk is the same permutation for both, which the dot product does not see.
+// split K and reduce through LDS at the end, so that even N = 4096 fills the
+// chip. Matrix fragments want one row per lane, memory wants consecutive lanes
+// on consecutive bytes: each wave moves its 16 x 128 tile of W (and the x rows
+// of the same K range) with coalesced loads into LDS of its own, the next
+// tile's loads in flight meanwhile. No workgroup barrier in the loop.
 // ---------------------------------------------------------------------------
+constexpr int SK_KC = 128;                        // K per tile
+constexpr int SK_STRIDE = SK_KC * 2 + 16;         // LDS bytes per row
+
 template <int NB, int WAVES>
 __global__ __launch_bounds__(WAVES * WAVE_SIZE) void gemm_skinny_kernel(
     const bf16* __restrict__ W, const bf16* __restrict__ x, bf16* __restrict__ y,
     float* __restrict__ yf, bool relu2, int B, int N, int K) {
-  constexpr int U = NB <= 2 ? 4 : 2;              // chunks in flight
-  __shared__ float red[WAVES][16][16 * NB + 1];
+  constexpr int RED = WAVES * 16 * (16 * NB + 1) * 4;
+  constexpr int TILE = 16 * (1 + NB) * SK_STRIDE;
+  __shared__ __attribute__((aligned(16))) char lds[WAVES * TILE > RED ? WAVES * TILE : RED];
   const int lane = threadIdx.x & (WAVE_SIZE - 1), wid = threadIdx.x / WAVE_SIZE;
   const int lo16 = lane & 15, hi4 = lane >> 4;
   const int n0 = blockIdx.x * 16;
-  const bf16* wrow = W + (long)min(n0 + lo16, N - 1) * K + hi4 * 16;
-  const bf16* xrow[NB];
-#pragma unroll
-  for (int b = 0; b < NB; ++b) xrow[b] = x + (long)min(b * 16 + lo16, B - 1) * K + hi4 * 16;
+  char* wl = lds + wid * TILE;                    // [16][SK_STRIDE]
+  char* xl = wl + 16 * SK_STRIDE;                 // [16 NB][SK_STRIDE]
+
   gemv_f32x4 acc[NB];
 #pragma unroll
   for (int b = 0; b < NB; ++b) acc[b] = gemv_f32x4{0.f, 0.f, 0.f, 0.f};
+  const int tiles = (K + SK_KC - 1) / SK_KC;
+  const int per = (tiles + WAVES - 1) / WAVES;
+  const int t_lo = wid * per, t_hi = min(t_lo + per, tiles);
 
-  const int full = K / 64;                        // whole chunks, split over the waves
-  const int per = (full + WAVES - 1) / WAVES;
-  int c = wid * per;
-  const int c_hi = min(c + per, full);
-  for (; c + U <= c_hi; c += U) {
-    gemv_bf16x8 w[U][2], v[U][NB][2];
+  // load j covers rows 4j + hi4, 16 bytes per lane at column 8 lo16
+  gemv_bf16x8 wr[4], xr[4 * NB];
+  auto fetch = [&](int t) {
+    const int k = t * SK_KC + lo16 * 8;
+    const bool in = k < K;                        // K % 8 == 0: all 8 or none
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const long k = (long)(c + u) * 64;
-#pragma unroll
-      for (int i = 0; i < 2; ++i) {
-        w[u][i] = *reinterpret_cast<const gemv_bf16x8*>(wrow + k + i * 8);
-#pragma unroll
-        for (int b = 0; b < NB; ++b)
-          v[u][b][i] = *reinterpret_cast<const gemv_bf16x8*>(xrow[b] + k + i * 8);
-      }
+    for (int j = 0; j < 4; ++j) {
+      wr[j] = gemv_bf16x8{};
+      if (in)
+        wr[j] = *reinterpret_cast<const gemv_bf16x8*>(
+            W + (long)min(n0 + 4 * j + hi4, N - 1) * K + k);
     }
 #pragma unroll
-    for (int u = 0; u < U; ++u)
+    for (int j = 0; j < 4 * NB; ++j) {
+      xr[j] = gemv_bf16x8{};
+      if (in)
+        xr[j] = *reinterpret_cast<const gemv_bf16x8*>(x + (long)min(4 * j + hi4, B - 1) * K + k);
+    }
+  };
+  if (t_lo < t_hi) fetch(t_lo);
+  for (int t = t_lo; t < t_hi; ++t) {
 #pragma unroll
-      for (int i = 0; i < 2; ++i)
+    for (int j = 0; j < 4; ++j)
+      *reinterpret_cast<gemv_bf16x8*>(wl + (4 * j + hi4) * SK_STRIDE + lo16 * 16) = wr[j];
 #pragma unroll
-        for (int b = 0; b < NB; ++b)
-          acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[u][i], v[u][b][i], acc[b], 0, 0, 0);
-  }
-  // leftover chunks, and for the last wave the K tail (8-wide pieces past K
-  // contribute zeros)
-  const int c_end = wid == WAVES - 1 ? (K + 63) / 64 : c_hi;
-  if (wid == WAVES - 1 && c > full) c = full;
-  for (; c < c_end; ++c) {
-    const long k = (long)c * 64;
+    for (int j = 0; j < 4 * NB; ++j)
+      *reinterpret_cast<gemv_bf16x8*>(xl + (4 * j + hi4) * SK_STRIDE + lo16 * 16) = xr[j];
+    __builtin_amdgcn_wave_barrier();
+    if (t + 1 < t_hi) fetch(t + 1);
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const bool in = k + hi4 * 16 + i * 8 < K;   // K % 8 == 0: all 8 or none
-      gemv_bf16x8 zero = {};
-      const gemv_bf16x8 w = in ? *reinterpret_cast<const gemv_bf16x8*>(wrow + k + i * 8) : zero;
+    for (int kk = 0; kk < SK_KC / 32; ++kk) {
+      const int off = lo16 * SK_STRIDE + kk * 64 + hi4 * 16;
+      const gemv_bf16x8 w = *reinterpret_cast<const gemv_bf16x8*>(wl + off);
 #pragma unroll
       for (int b = 0; b < NB; ++b) {
-        const gemv_bf16x8 v =
-            in ? *reinterpret_cast<const gemv_bf16x8*>(xrow[b] + k + i * 8) : zero;
+        const gemv_bf16x8 v = *reinterpret_cast<const gemv_bf16x8*>(xl + b * 16 * SK_STRIDE + off);
         acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, v, acc[b], 0, 0, 0);
       }
     }
+    __builtin_amdgcn_wave_barrier();              // the tile is overwritten next
   }
+  __syncthreads();                                // tiles become the reduction buffer
+  float* red = reinterpret_cast<float*>(lds);
+  constexpr int RS = 16 * NB + 1;
 #pragma unroll
   for (int b = 0; b < NB; ++b)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) red[wid][hi4 * 4 + i][b * 16 + lo16] = acc[b][i];
+    for (int i = 0; i < 4; ++i) red[(wid * 16 + hi4 * 4 + i) * RS + b * 16 + lo16] = acc[b][i];
   __syncthreads();
   for (int i = threadIdx.x; i < 256 * NB; i += WAVES * WAVE_SIZE) {
     const int row = i & 15, col = i >> 4;
     if (n0 + row >= N || col >= B) continue;
     float t = 0.f;
 #pragma unroll
-    for (int w = 0; w < WAVES; ++w) t += red[w][row][col];
+    for (int w = 0; w < WAVES; ++w) t += red[(w * 16 + row) * RS + col];
     if (relu2) {
       t = fmaxf(t, 0.f);
       t *= t;
@@ -235,10 +242,12 @@ at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2
           reinterpret_cast<const bf16*>(xc.data_ptr()),                                      \
           out_f32 ? nullptr : reinterpret_cast<bf16*>(y.data_ptr()),                         \
           out_f32 ? y.data_ptr<float>() : nullptr, relu2, B, N, K)
+  // waves per workgroup: enough of them across the chip, each with K left to
+  // stream; LDS grows with the x rows
   const bool deep = K >= 2048;
   if (B <= 16) { if (deep) LAUNCH(1, 8); else LAUNCH(1, 4); }
-  else if (B <= 32) { if (deep) LAUNCH(2, 8); else LAUNCH(2, 4); }
-  else { if (deep) LAUNCH(4, 8); else LAUNCH(4, 4); }
+  else if (B <= 32) { LAUNCH(2, 4); }
+  else { LAUNCH(4, 2); }
 #undef LAUNCH
   HIP_CHECK_KERNEL();
   return y;

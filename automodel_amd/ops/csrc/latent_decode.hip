@@ -7,7 +7,7 @@
 //   latent_decode_attn     split-KV attention of all heads over the cache:
 //                          the heads are the M dimension of 16x16x32 MFMAs, so
 //                          one staged key tile serves them all
-//   latent_decode_combine  merges the splits and applies W_uv per head
+//   latent_decode_combine  merges the splits, then applies W_uv per head
 //
 // Lengths and slots are device tensors: a captured step replays for every
 // position. Keys are split evenly over the row's own length.
@@ -124,6 +124,7 @@ __global__ __launch_bounds__(256) void latent_decode_prep_kernel(
 typedef __bf16 lat_bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 lat_bf16x4 __attribute__((ext_vector_type(4)));
 typedef float lat_f32x4 __attribute__((ext_vector_type(4)));
+typedef unsigned lat_u32x4 __attribute__((ext_vector_type(4)));    // 16 bytes in flight
 
 constexpr int LD_KEYS = 64;           // keys per tile: 4 waves x 16
 constexpr int LD_PSTRIDE = LD_KEYS * 2 + 16;
@@ -167,32 +168,32 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
   const int vecs = C / 8;                         // 16-byte pieces per row
   const int np = C / 32;                          // pieces of a 64-row tile per thread
   const unsigned magic = ((1u << 20) + vecs - 1) / vecs;    // i / vecs, exact for i < 64 vecs
-  uint4 pre[NPM];
+  lat_u32x4 pre[NPM];
   auto fetch = [&](int t) {
 #pragma unroll
     for (int j = 0; j < NPM; ++j) {
       if (j < np) {                               // uniform
         const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
         const int key = min(t * LD_KEYS + (int)row, n - 1);   // rows past the end: masked below
-        pre[j] = *reinterpret_cast<const uint4*>(base + (long)key * C + c * 8);
+        pre[j] = *reinterpret_cast<const lat_u32x4*>(base + (long)key * C + c * 8);
       }
     }
   };
   if (t_lo < t_hi) fetch(t_lo);
   // queries: 16 MT rows of the same width, np / (4 / MT) pieces per thread
   for (int i0 = tid; i0 < 16 * MT * vecs; i0 += 1024) {
-    uint4 x[4];
+    lat_u32x4 x[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
-      x[j] = uint4{0u, 0u, 0u, 0u};
+      x[j] = lat_u32x4{0u, 0u, 0u, 0u};
       if (i < 16u * MT * vecs && h0 + (int)row < H)
-        x[j] = *reinterpret_cast<const uint4*>(q + ((long)r * H + h0 + row) * C + c * 8);
+        x[j] = *reinterpret_cast<const lat_u32x4*>(q + ((long)r * H + h0 + row) * C + c * 8);
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
-      if (i < 16u * MT * vecs) *reinterpret_cast<uint4*>(qt + row * KS + c * 16) = x[j];
+      if (i < 16u * MT * vecs) *reinterpret_cast<lat_u32x4*>(qt + row * KS + c * 16) = x[j];
     }
   }
 
@@ -212,7 +213,7 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
     for (int j = 0; j < NPM; ++j) {
       if (j < np) {
         const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
-        *reinterpret_cast<uint4*>(kt + row * KS + c * 16) = pre[j];
+        *reinterpret_cast<lat_u32x4*>(kt + row * KS + c * 16) = pre[j];
       }
     }
     __syncthreads();
@@ -325,100 +326,95 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// combine: grid (value chunks of 32, H, row groups). Merges the splits into the
-// normalised latent output (LDS, f32), then one wave per value row takes the
-// dot product with W_uv. part_ml == null: part_o is already normalised.
+// merge: grid (column chunks of 128, H, R). Splits -> normalised latent output
+// in f32; 32 threads cover the columns, 8 groups of them share the splits.
+// ---------------------------------------------------------------------------
+constexpr int LM_COLS = 128;
+__global__ __launch_bounds__(256) void latent_decode_merge_kernel(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml, float* __restrict__ o,
+    int H, int RP, int S) {
+  extern __shared__ float sm[];
+  float* wt = sm;                                 // [S]
+  lat_f32x4* half = reinterpret_cast<lat_f32x4*>(sm + (S + 3) / 4 * 4);    // [8][32]
+  const int tid = threadIdx.x, lane = tid & 63;
+  const long rh = (long)blockIdx.z * H + blockIdx.y;
+  const float* ml = part_ml + rh * S * 2;
+  if (tid < 64) {                                 // one wave weighs the splits
+    float m = -1e30f;
+    for (int s = lane; s < S; s += 64) m = fmaxf(m, ml[2 * s]);
+    m = wave_reduce_max(m);
+    float l = 0.f;
+    for (int s = lane; s < S; s += 64) l += __expf(ml[2 * s] - m) * ml[2 * s + 1];
+    l = wave_reduce_sum(l);
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    for (int s = lane; s < S; s += 64) wt[s] = __expf(ml[2 * s] - m) * inv;
+  }
+  __syncthreads();
+  const int col = blockIdx.x * LM_COLS + (tid & 31) * 4, g = tid >> 5;
+  lat_f32x4 a = {0.f, 0.f, 0.f, 0.f};
+  if (col < RP) {                                 // RP % 32 == 0
+    const float* po = part_o + rh * S * RP + col;
+#pragma unroll 8
+    for (int s = g; s < S; s += 8)
+      a += wt[s] * *reinterpret_cast<const lat_f32x4*>(po + (long)s * RP);
+  }
+  half[g * 32 + (tid & 31)] = a;
+  __syncthreads();
+  if (g == 0 && col < RP) {
+#pragma unroll
+    for (int i = 1; i < 8; ++i) a += half[i * 32 + tid];
+    *reinterpret_cast<lat_f32x4*>(o + rh * RP + col) = a;
+  }
+}
+
+// ---------------------------------------------------------------------------
+// value up-projection: grid (value chunks of 32, H, row groups of RT). A wave
+// takes 8 rows of W_uv[h] at once against the latent outputs in LDS.
 // ---------------------------------------------------------------------------
 constexpr int LC_ROWS = 32;
 template <typename T, int V, int RT>
-__global__ __launch_bounds__(256) void latent_decode_combine_kernel(
-    const float* __restrict__ part_o, const float* __restrict__ part_ml,
-    const T* __restrict__ w_uv, T* __restrict__ out, int R, int H, int dv, int rank, int stride,
-    int S) {
-  extern __shared__ float sm[];
-  float* ol = sm;                                 // [RT][rank]
-  float* wt = sm + RT * rank;                     // [RT][S]
+__global__ __launch_bounds__(256) void latent_decode_value_kernel(
+    const float* __restrict__ o_lat, const T* __restrict__ w_uv, T* __restrict__ out, int R, int H,
+    int dv, int rank, int stride) {
+  extern __shared__ float sm[];                   // [RT][rank]
+  constexpr int NV = LC_ROWS / 4;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int h = blockIdx.y, r0 = blockIdx.z * RT;
-  if (part_ml) {
-    if (wid < RT) {                               // a wave per row (looping over rows)
-      for (int rr = wid; rr < RT; rr += 4) {
-        const int r = r0 + rr;
-        if (r >= R) break;
-        const float* ml = part_ml + ((long)r * H + h) * S * 2;
-        float m = -1e30f;
-        for (int s = lane; s < S; s += 64) m = fmaxf(m, ml[2 * s + 1] > 0.f ? ml[2 * s] : -1e30f);
-        m = wave_reduce_max(m);
-        float l = 0.f;
-        for (int s = lane; s < S; s += 64) {
-          const float w = ml[2 * s + 1] > 0.f ? __expf(ml[2 * s] - m) : 0.f;
-          wt[rr * S + s] = w;
-          l += w * ml[2 * s + 1];
-        }
-        l = wave_reduce_sum(l);
-        const float inv = l > 0.f ? 1.f / l : 0.f;
-        for (int s = lane; s < S; s += 64) wt[rr * S + s] *= inv;
-      }
-    }
-    __syncthreads();
+  for (int i = tid; i < RT * rank; i += 256) {
+    const int r = min(r0 + i / rank, R - 1);
+    sm[i] = o_lat[((long)r * H + h) * stride + i % rank];
   }
-  // merge: a thread owns 4 columns of a row (1 if the rank is no multiple of
-  // 4); where that leaves threads idle, they share a column's splits
-  constexpr int M = V == 1 ? 1 : 4;
-  const int cols = rank / M, items = RT * cols;
-  const int groups = min(max(256 / items, 1), S);
-  float* half = wt + RT * S;                      // [groups][items][M], groups > 1 only
-  for (int i0 = tid; i0 < items * groups; i0 += 256) {
-    const int i = i0 % items, g = i0 / items;
-    const int rr = i / cols, c = (i % cols) * M, r = min(r0 + rr, R - 1);
-    const float* po = part_o + ((long)r * H + h) * S * stride + c;
-    float a[M];
+  const int v0 = blockIdx.x * LC_ROWS + wid * NV;
+  const T* w[NV];
 #pragma unroll
-    for (int j = 0; j < M; ++j) a[j] = 0.f;
-    if (part_ml) {
-#pragma unroll 8
-      for (int s = g; s < S; s += groups) {
-        const float w = r0 + rr < R ? wt[rr * S + s] : 0.f;
-        const LatPack<float, M> x = *reinterpret_cast<const LatPack<float, M>*>(po + (long)s * stride);
+  for (int v = 0; v < NV; ++v) w[v] = w_uv + ((long)h * dv + min(v0 + v, dv - 1)) * rank;
+  float acc[NV][RT];
 #pragma unroll
-        for (int j = 0; j < M; ++j) a[j] = fmaf(w, x.v[j], a[j]);
-      }
-    } else {
+  for (int v = 0; v < NV; ++v)
 #pragma unroll
-      for (int j = 0; j < M; ++j) a[j] = po[j];
-    }
-    float* dst = groups > 1 ? half + ((long)g * items + i) * M : ol + rr * rank + c;
-#pragma unroll
-    for (int j = 0; j < M; ++j) dst[j] = a[j];
-  }
+    for (int rr = 0; rr < RT; ++rr) acc[v][rr] = 0.f;
   __syncthreads();
-  if (groups > 1) {                               // uniform
-    for (int i = tid; i < items * M; i += 256) {
-      float a = 0.f;
-      for (int g = 0; g < groups; ++g) a += half[g * items * M + i];
-      ol[i] = a;
-    }
-    __syncthreads();
+  for (int c = lane * V; c < rank; c += 64 * V) {
+    LatPack<T, V> x[NV];
+#pragma unroll
+    for (int v = 0; v < NV; ++v) x[v] = *reinterpret_cast<const LatPack<T, V>*>(w[v] + c);
+#pragma unroll
+    for (int rr = 0; rr < RT; ++rr)
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float o = sm[rr * rank + c + j];
+#pragma unroll
+        for (int v = 0; v < NV; ++v) acc[v][rr] = fmaf(lat_f(x[v].v[j]), o, acc[v][rr]);
+      }
   }
-  const int v_lo = blockIdx.x * LC_ROWS, v_hi = min(v_lo + LC_ROWS, dv);
-  for (int v = v_lo + wid; v < v_hi; v += 4) {
-    const T* w = w_uv + ((long)h * dv + v) * rank;
-    float acc[RT];
 #pragma unroll
-    for (int rr = 0; rr < RT; ++rr) acc[rr] = 0.f;
-    for (int c = lane * V; c < rank; c += 64 * V) {
-      const LatPack<T, V> x = *reinterpret_cast<const LatPack<T, V>*>(w + c);
-#pragma unroll
-      for (int rr = 0; rr < RT; ++rr)
-#pragma unroll
-        for (int j = 0; j < V; ++j) acc[rr] = fmaf(lat_f(x.v[j]), ol[rr * rank + c + j], acc[rr]);
-    }
+  for (int v = 0; v < NV; ++v)
 #pragma unroll
     for (int rr = 0; rr < RT; ++rr) {
-      const float a = wave_reduce_sum(acc[rr]);
-      if (lane == 0 && r0 + rr < R) out[((long)(r0 + rr) * H + h) * dv + v] = lat_t<T>(a);
+      const float a = wave_reduce_sum(acc[v][rr]);
+      if (lane == 0 && v0 + v < dv && r0 + rr < R)
+        out[((long)(r0 + rr) * H + h) * dv + v0 + v] = lat_t<T>(a);
     }
-  }
 }
 
 // ---------------------------------------------------------------------------
@@ -557,16 +553,24 @@ at::Tensor latent_decode_combine(const at::Tensor& part_o,
   if (R == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
   const bool vec = rank % 8 == 0;
-  const float* ml = part_ml ? part_ml->data_ptr<float>() : nullptr;
+  at::Tensor o_lat = part_o;
+  if (part_ml) {
+    TORCH_CHECK(n % 32 == 0 && S <= 1024, "latent_decode_combine: padded rank, splits <= 1024");
+    o_lat = at::empty({R, H, n}, part_o.options());
+    latent_decode_merge_kernel<<<dim3((n + LM_COLS - 1) / LM_COLS, H, R), dim3(256),
+                                 ((S + 3) / 4 * 4 + 1024) * sizeof(float), stream>>>(
+        part_o.data_ptr<float>(), part_ml->data_ptr<float>(), o_lat.data_ptr<float>(), (int)H,
+        (int)n, (int)S);
+    HIP_CHECK_KERNEL();
+  }
 #define LAUNCH(TT, VV)                                                                          \
-  latent_decode_combine_kernel<TT, VV, RT>                                                      \
+  latent_decode_value_kernel<TT, VV, RT>                                                        \
       <<<dim3((dv + LC_ROWS - 1) / LC_ROWS, H, (R + RT - 1) / RT), dim3(256), smem, stream>>>(  \
-          part_o.data_ptr<float>(), ml, reinterpret_cast<const TT*>(w_uv.data_ptr()),           \
-          reinterpret_cast<TT*>(out.data_ptr()), (int)R, (int)H, (int)dv, (int)rank, (int)n,    \
-          (int)S)
+          o_lat.data_ptr<float>(), reinterpret_cast<const TT*>(w_uv.data_ptr()),                \
+          reinterpret_cast<TT*>(out.data_ptr()), (int)R, (int)H, (int)dv, (int)rank, (int)n)
   ROW_TILE(R, {
-    const size_t smem = (RT * rank + RT * S + 1024) * sizeof(float);
-    TORCH_CHECK(smem <= 64 * 1024, "latent_decode_combine: rank or splits too large");
+    const size_t smem = RT * rank * sizeof(float);
+    TORCH_CHECK(smem <= 64 * 1024, "latent_decode_combine: rank too large");
     if (w_uv.scalar_type() == at::kBFloat16) {
       if (vec) LAUNCH(bf16, 8); else LAUNCH(bf16, 1);
     } else {
