@@ -119,7 +119,7 @@ __global__ __launch_bounds__(256) void latent_decode_prep_kernel(
 }
 
 // ---------------------------------------------------------------------------
-// attention over the cache. grid (splits, head groups of 16*MT, rows)
+// attention over the cache. grid (splits, head groups of 16*HT, rows)
 // ---------------------------------------------------------------------------
 typedef __bf16 lat_bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 lat_bf16x4 __attribute__((ext_vector_type(4)));
@@ -137,25 +137,27 @@ __device__ __forceinline__ lat_bf16x4 lds_tr16(const char* p) {
       (lds_ptr)(__attribute__((address_space(3))) char*)const_cast<char*>(p));
 }
 
-// NCT: 16-column value tiles per wave (4 waves cover RP <= 64 * NCT).
-// NPM: bound on the 16-byte pieces of a key tile per thread (exactly C / 32).
-// The next tile travels through registers while the current one is used.
-template <int MT, int NCT, int NPM>
-__global__ __launch_bounds__(256) void latent_decode_attn_kernel(
+// HT: head tiles (of 16 heads) per workgroup, four waves each; they share the
+// staged keys. NCT: 16-column value tiles per wave (4 waves cover RP <= 64 *
+// NCT). NPM: bound on the 16-byte pieces of a key tile per thread. The next
+// tile travels through registers while the current one is used.
+template <int HT, int NCT, int NPM>
+__global__ __launch_bounds__(256 * HT) void latent_decode_attn_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ cache, const int* __restrict__ slot,
     const int* __restrict__ pos, float* __restrict__ part_o, float* __restrict__ part_ml,
     int n_slots, int max_len, int H, int RP, int C, float scale) {
+  constexpr int NT = 256 * HT;
   extern __shared__ __attribute__((aligned(16))) char lds[];
   const int KS = C * 2 + 16;                      // LDS row stride: conflict-free b128 reads
   char* kt = lds;                                 // [64][KS]
-  char* qt = kt + LD_KEYS * KS;                   // [16 MT][KS]
-  char* pt = qt + 16 * MT * KS;                   // [16 MT][LD_PSTRIDE]
-  float* red = reinterpret_cast<float*>(pt + 16 * MT * LD_PSTRIDE);   // [4][16 MT]
+  char* qt = kt + LD_KEYS * KS;                   // [16 HT][KS]
+  char* pt = qt + 16 * HT * KS;                   // [16 HT][LD_PSTRIDE]
+  float* red = reinterpret_cast<float*>(pt + 16 * HT * LD_PSTRIDE);   // [HT][4][16]
 
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wid = (tid >> 6) & 3, ht = tid >> 8;
   const int lo16 = lane & 15, hi4 = lane >> 4;
   const int split = blockIdx.x, n_split = gridDim.x;
-  const int h0 = blockIdx.y * 16 * MT;
+  const int h0 = blockIdx.y * 16 * HT;
   const int r = blockIdx.z;
 
   const int sl = slot[r];
@@ -166,114 +168,100 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
   const bf16* base = cache + (long)(n > 0 ? sl : 0) * max_len * C;
 
   const int vecs = C / 8;                         // 16-byte pieces per row
-  const int np = C / 32;                          // pieces of a 64-row tile per thread
-  const unsigned magic = ((1u << 20) + vecs - 1) / vecs;    // i / vecs, exact for i < 64 vecs
+  const int pieces = LD_KEYS * vecs, np = (pieces + NT - 1) / NT;
+  const unsigned magic = ((1u << 20) + vecs - 1) / vecs;    // i / vecs, exact for i < 128 vecs
   lat_u32x4 pre[NPM];
   auto fetch = [&](int t) {
 #pragma unroll
     for (int j = 0; j < NPM; ++j) {
       if (j < np) {                               // uniform
-        const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+        const unsigned i = tid + j * NT, row = (i * magic) >> 20, c = i - row * vecs;
         const int key = min(t * LD_KEYS + (int)row, n - 1);   // rows past the end: masked below
         pre[j] = *reinterpret_cast<const lat_u32x4*>(base + (long)key * C + c * 8);
       }
     }
   };
   if (t_lo < t_hi) fetch(t_lo);
-  // queries: 16 MT rows of the same width, np / (4 / MT) pieces per thread
-  for (int i0 = tid; i0 < 16 * MT * vecs; i0 += 1024) {
+  for (int i0 = tid; i0 < 16 * HT * vecs; i0 += 4 * NT) {      // this workgroup's queries
     lat_u32x4 x[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
+      const unsigned i = i0 + j * NT, row = (i * magic) >> 20, c = i - row * vecs;
       x[j] = lat_u32x4{0u, 0u, 0u, 0u};
-      if (i < 16u * MT * vecs && h0 + (int)row < H)
+      if (i < 16u * HT * vecs && h0 + (int)row < H)
         x[j] = *reinterpret_cast<const lat_u32x4*>(q + ((long)r * H + h0 + row) * C + c * 8);
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      const unsigned i = i0 + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
-      if (i < 16u * MT * vecs) *reinterpret_cast<lat_u32x4*>(qt + row * KS + c * 16) = x[j];
+      const unsigned i = i0 + j * NT, row = (i * magic) >> 20, c = i - row * vecs;
+      if (i < 16u * HT * vecs) *reinterpret_cast<lat_u32x4*>(qt + row * KS + c * 16) = x[j];
     }
   }
 
-  lat_f32x4 acc[MT][NCT];
-  float m_run[MT][4], l_run[MT][4];
+  lat_f32x4 acc[NCT];
+  float m_run[4], l_run[4];
 #pragma unroll
-  for (int a = 0; a < MT; ++a) {
+  for (int c = 0; c < NCT; ++c) acc[c] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int c = 0; c < NCT; ++c) acc[a][c] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int i = 0; i < 4; ++i) m_run[a][i] = -1e30f, l_run[a][i] = 0.f;
-  }
+  for (int i = 0; i < 4; ++i) m_run[i] = -1e30f, l_run[i] = 0.f;
+  float* my_red = red + ht * 64;
+  char* my_pt = pt + ht * 16 * LD_PSTRIDE;
 
   for (int t = t_lo; t < t_hi; ++t) {
     const int k0 = t * LD_KEYS;
 #pragma unroll
     for (int j = 0; j < NPM; ++j) {
       if (j < np) {
-        const unsigned i = tid + j * 256, row = (i * magic) >> 20, c = i - row * vecs;
-        *reinterpret_cast<lat_u32x4*>(kt + row * KS + c * 16) = pre[j];
+        const unsigned i = tid + j * NT, row = (i * magic) >> 20, c = i - row * vecs;
+        if ((int)i < pieces) *reinterpret_cast<lat_u32x4*>(kt + row * KS + c * 16) = pre[j];
       }
     }
     __syncthreads();
     if (t + 1 < t_hi) fetch(t + 1);
 
     // scores: D[head = 4*hi4 + i][key = lo16] of this wave's 16 keys
-    lat_f32x4 s[MT];
-#pragma unroll
-    for (int a = 0; a < MT; ++a) s[a] = lat_f32x4{0.f, 0.f, 0.f, 0.f};
+    lat_f32x4 s = {0.f, 0.f, 0.f, 0.f};
     const char* kp = kt + (wid * 16 + lo16) * KS + hi4 * 16;
-    const char* qp = qt + lo16 * KS + hi4 * 16;
+    const char* qp = qt + (ht * 16 + lo16) * KS + hi4 * 16;
+#pragma unroll 6
     for (int c = 0; c < C * 2; c += 64) {
       const lat_bf16x8 b = *reinterpret_cast<const lat_bf16x8*>(kp + c);
-#pragma unroll
-      for (int a = 0; a < MT; ++a) {
-        const lat_bf16x8 x = *reinterpret_cast<const lat_bf16x8*>(qp + a * 16 * KS + c);
-        s[a] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, b, s[a], 0, 0, 0);
-      }
+      const lat_bf16x8 x = *reinterpret_cast<const lat_bf16x8*>(qp + c);
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, b, s, 0, 0, 0);
     }
     const bool live = k0 + wid * 16 + lo16 < n;
+    float mx[4];
 #pragma unroll
-    for (int a = 0; a < MT; ++a)
+    for (int i = 0; i < 4; ++i) s[i] = mx[i] = live ? s[i] * scale : -1e30f;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float v = live ? s[a][i] * scale : -1e30f;
-        s[a][i] = v;
-        float mx = v;
-        mx = fmaxf(mx, __shfl_xor(mx, 1));
-        mx = fmaxf(mx, __shfl_xor(mx, 2));
-        mx = fmaxf(mx, __shfl_xor(mx, 4));
-        mx = fmaxf(mx, __shfl_xor(mx, 8));
-        if (lo16 == 0) red[wid * 16 * MT + a * 16 + hi4 * 4 + i] = mx;
-      }
+    for (int d = 1; d < 16; d *= 2)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) mx[i] = fmaxf(mx[i], __shfl_xor(mx[i], d));
+    if (lo16 == 0)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) my_red[wid * 16 + hi4 * 4 + i] = mx[i];
     __syncthreads();
 #pragma unroll
-    for (int a = 0; a < MT; ++a)
+    for (int i = 0; i < 4; ++i) {
+      const int row = hi4 * 4 + i;
+      float mn = m_run[i];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int row = a * 16 + hi4 * 4 + i;
-        float mn = m_run[a][i];
+      for (int w = 0; w < 4; ++w) mn = fmaxf(mn, my_red[w * 16 + row]);
+      const float alpha = __expf(m_run[i] - mn);
+      const float p = live ? __expf(s[i] - mn) : 0.f;
+      l_run[i] = l_run[i] * alpha + p;
+      m_run[i] = mn;
+      *reinterpret_cast<bf16*>(my_pt + row * LD_PSTRIDE + (wid * 16 + lo16) * 2) = f2bf(p);
 #pragma unroll
-        for (int w = 0; w < 4; ++w) mn = fmaxf(mn, red[w * 16 * MT + row]);
-        const float alpha = __expf(m_run[a][i] - mn);
-        const float p = live ? __expf(s[a][i] - mn) : 0.f;
-        l_run[a][i] = l_run[a][i] * alpha + p;
-        m_run[a][i] = mn;
-        *reinterpret_cast<bf16*>(pt + row * LD_PSTRIDE + (wid * 16 + lo16) * 2) = f2bf(p);
-#pragma unroll
-        for (int c = 0; c < NCT; ++c) acc[a][c][i] *= alpha;
-      }
+      for (int c = 0; c < NCT; ++c) acc[c][i] *= alpha;
+    }
     __syncthreads();
 
     // O[head][column] += P[head][key] V[key][column], V = the tile's latents
 #pragma unroll
     for (int ks = 0; ks < LD_KEYS / 32; ++ks) {
-      lat_bf16x8 p[MT];
-#pragma unroll
-      for (int a = 0; a < MT; ++a)
-        p[a] = *reinterpret_cast<const lat_bf16x8*>(pt + (a * 16 + lo16) * LD_PSTRIDE +
-                                                    (ks * 32 + hi4 * 8) * 2);
+      const lat_bf16x8 p = *reinterpret_cast<const lat_bf16x8*>(my_pt + lo16 * LD_PSTRIDE +
+                                                                (ks * 32 + hi4 * 8) * 2);
 #pragma unroll
       for (int c = 0; c < NCT; ++c) {
         const int n0 = (wid * NCT + c) * 16;
@@ -281,48 +269,40 @@ __global__ __launch_bounds__(256) void latent_decode_attn_kernel(
           const char* vp = kt + (ks * 32 + hi4 * 8 + (lo16 >> 2)) * KS + (n0 + (lo16 & 3) * 4) * 2;
           const lat_bf16x4 v0 = lds_tr16(vp), v1 = lds_tr16(vp + 4 * KS);
           const lat_bf16x8 v = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
-#pragma unroll
-          for (int a = 0; a < MT; ++a)
-            acc[a][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p[a], v, acc[a][c], 0, 0, 0);
+          acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, v, acc[c], 0, 0, 0);
         }
       }
     }
     __syncthreads();                              // before the tile is overwritten
   }
 
-  // partial results of this split
+  // partial results of this split; an empty split stores zeros
 #pragma unroll
-  for (int a = 0; a < MT; ++a)
+  for (int i = 0; i < 4; ++i) {
+    float l = l_run[i];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      float l = l_run[a][i];
-      l += __shfl_xor(l, 1);
-      l += __shfl_xor(l, 2);
-      l += __shfl_xor(l, 4);
-      l += __shfl_xor(l, 8);
-      if (lo16 == 0) red[wid * 16 * MT + a * 16 + hi4 * 4 + i] = l;
-    }
+    for (int d = 1; d < 16; d *= 2) l += __shfl_xor(l, d);
+    if (lo16 == 0) my_red[wid * 16 + hi4 * 4 + i] = l;
+  }
   __syncthreads();
 #pragma unroll
-  for (int a = 0; a < MT; ++a)
+  for (int i = 0; i < 4; ++i) {
+    const int row = hi4 * 4 + i, h = h0 + ht * 16 + row;
+    if (h >= H) continue;
+    const long o = ((long)r * H + h) * n_split + split;
+    if (wid == 0 && lo16 == 0) {
+      float l = 0.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int row = a * 16 + hi4 * 4 + i, h = h0 + row;
-      if (h >= H) continue;
-      const long o = ((long)r * H + h) * n_split + split;
-      if (wid == 0 && lo16 == 0) {
-        float l = 0.f;
-#pragma unroll
-        for (int w = 0; w < 4; ++w) l += red[w * 16 * MT + row];
-        part_ml[o * 2] = m_run[a][i];
-        part_ml[o * 2 + 1] = l;
-      }
-#pragma unroll
-      for (int c = 0; c < NCT; ++c) {             // an empty split stores zeros
-        const int n0 = (wid * NCT + c) * 16;
-        if (n0 < RP) part_o[o * RP + n0 + lo16] = acc[a][c][i];
-      }
+      for (int w = 0; w < 4; ++w) l += my_red[w * 16 + row];
+      part_ml[o * 2] = m_run[i];
+      part_ml[o * 2 + 1] = l;
     }
+#pragma unroll
+    for (int c = 0; c < NCT; ++c) {
+      const int n0 = (wid * NCT + c) * 16;
+      if (n0 < RP) part_o[o * RP + n0 + lo16] = acc[c][i];
+    }
+  }
 }
 
 // ---------------------------------------------------------------------------
@@ -380,41 +360,49 @@ __global__ __launch_bounds__(256) void latent_decode_value_kernel(
   constexpr int NV = LC_ROWS / 4;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int h = blockIdx.y, r0 = blockIdx.z * RT;
+  const int nc = rank / V;                        // column c = chunk * V + j sits at [j][chunk]
   for (int i = tid; i < RT * rank; i += 256) {
-    const int r = min(r0 + i / rank, R - 1);
-    sm[i] = o_lat[((long)r * H + h) * stride + i % rank];
+    const int rr = i / rank, c = i % rank, r = min(r0 + rr, R - 1);
+    sm[rr * rank + (c % V) * nc + c / V] = o_lat[((long)r * H + h) * stride + c];
   }
   const int v0 = blockIdx.x * LC_ROWS + wid * NV;
   const T* w[NV];
 #pragma unroll
   for (int v = 0; v < NV; ++v) w[v] = w_uv + ((long)h * dv + min(v0 + v, dv - 1)) * rank;
-  float acc[NV][RT];
+  float acc[NV * RT];
 #pragma unroll
-  for (int v = 0; v < NV; ++v)
-#pragma unroll
-    for (int rr = 0; rr < RT; ++rr) acc[v][rr] = 0.f;
+  for (int i = 0; i < NV * RT; ++i) acc[i] = 0.f;
   __syncthreads();
-  for (int c = lane * V; c < rank; c += 64 * V) {
+  for (int c = lane; c < nc; c += 64) {
     LatPack<T, V> x[NV];
 #pragma unroll
-    for (int v = 0; v < NV; ++v) x[v] = *reinterpret_cast<const LatPack<T, V>*>(w[v] + c);
+    for (int v = 0; v < NV; ++v) x[v] = *reinterpret_cast<const LatPack<T, V>*>(w[v] + c * V);
 #pragma unroll
     for (int rr = 0; rr < RT; ++rr)
 #pragma unroll
       for (int j = 0; j < V; ++j) {
-        const float o = sm[rr * rank + c + j];
+        const float o = sm[rr * rank + j * nc + c];
 #pragma unroll
-        for (int v = 0; v < NV; ++v) acc[v][rr] = fmaf(lat_f(x[v].v[j]), o, acc[v][rr]);
+        for (int v = 0; v < NV; ++v) acc[rr * NV + v] = fmaf(lat_f(x[v].v[j]), o, acc[rr * NV + v]);
       }
   }
+  // all NV * RT sums over the wave at once: halve the set at every step, so
+  // that lane l ends with sum l / (64 / (NV * RT))
+  constexpr int NA = NV * RT;
+  int mask = 32;
 #pragma unroll
-  for (int v = 0; v < NV; ++v)
+  for (int n = NA; n > 1; n /= 2, mask /= 2) {
+    const bool up = lane & mask;
 #pragma unroll
-    for (int rr = 0; rr < RT; ++rr) {
-      const float a = wave_reduce_sum(acc[v][rr]);
-      if (lane == 0 && v0 + v < dv && r0 + rr < R)
-        out[((long)(r0 + rr) * H + h) * dv + v0 + v] = lat_t<T>(a);
+    for (int i = 0; i < n / 2; ++i) {
+      const float keep = up ? acc[i + n / 2] : acc[i], give = up ? acc[i] : acc[i + n / 2];
+      acc[i] = keep + __shfl_xor(give, mask);
     }
+  }
+  for (; mask > 0; mask /= 2) acc[0] += __shfl_xor(acc[0], mask);
+  const int idx = lane / (64 / NA), rr = idx / NV, v = idx % NV;
+  if (lane % (64 / NA) == 0 && v0 + v < dv && r0 + rr < R)
+    out[((long)(r0 + rr) * H + h) * dv + v0 + v] = lat_t<T>(acc[0]);
 }
 
 // ---------------------------------------------------------------------------
@@ -501,16 +489,16 @@ std::tuple<at::Tensor, at::Tensor> latent_decode_attn(const at::Tensor& q, const
   // head tiles per workgroup: both share the staged keys, but two workgroups
   // are better where the splits alone leave CUs idle
   const bool two = H > 16 && R * splits * ((H + 31) / 32) >= 256;
-#define LAUNCH1(MT, NCT, NPM)                                                                    \
+#define LAUNCH1(HT, NCT, NPM)                                                                    \
   do {                                                                                           \
-    const size_t smem = (LD_KEYS + 16 * MT) * (C * 2 + 16) + 16 * MT * (LD_PSTRIDE + 16);        \
+    const size_t smem = (LD_KEYS + 16 * HT) * (C * 2 + 16) + 16 * HT * (LD_PSTRIDE + 16);        \
     TORCH_CHECK(smem <= LDS_MAX, "latent_decode_attn: tile exceeds LDS");                        \
     static const hipError_t attr_ = hipFuncSetAttribute(                                         \
-        reinterpret_cast<const void*>(&latent_decode_attn_kernel<MT, NCT, NPM>),                 \
+        reinterpret_cast<const void*>(&latent_decode_attn_kernel<HT, NCT, NPM>),                 \
         hipFuncAttributeMaxDynamicSharedMemorySize, (int)LDS_MAX);                               \
     TORCH_CHECK(attr_ == hipSuccess, "latent_decode_attn: LDS attribute");                       \
-    latent_decode_attn_kernel<MT, NCT, NPM>                                                      \
-        <<<dim3(splits, (H + 16 * MT - 1) / (16 * MT), R), dim3(256), smem, stream>>>(           \
+    latent_decode_attn_kernel<HT, NCT, NPM>                                                      \
+        <<<dim3(splits, (H + 16 * HT - 1) / (16 * HT), R), dim3(256 * HT), smem, stream>>>(      \
             reinterpret_cast<const bf16*>(q.data_ptr()),                                         \
             reinterpret_cast<const bf16*>(cache.data_ptr()), slot.data_ptr<int>(),               \
             pos.data_ptr<int>(), part_o.data_ptr<float>(), part_ml.data_ptr<float>(),            \
@@ -518,7 +506,7 @@ std::tuple<at::Tensor, at::Tensor> latent_decode_attn(const at::Tensor& q, const
   } while (0)
 #define LAUNCH(NCT, NPM)                                                                         \
   do {                                                                                           \
-    if (two) LAUNCH1(2, NCT, NPM); else LAUNCH1(1, NCT, NPM);                                    \
+    if (two) LAUNCH1(2, NCT, (NPM + 1) / 2); else LAUNCH1(1, NCT, NPM);                          \
   } while (0)
   TORCH_CHECK(C / 32 <= 26, "latent_decode_attn: latent and rotated key too wide");
   if (RP <= 128 && C <= 256) LAUNCH(2, 8);
