@@ -51,12 +51,22 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     *reinterpret_cast<LatPack<T, V>*>(qo + h * QD + d) =
         *reinterpret_cast<const LatPack<T, V>*>(row + h * hd + d);
   }
-  for (int i = threadIdx.x; i < H * half; i += blockDim.x) {
-    const int h = i / half, d = i % half;
-    const float u = lat_f(row[h * hd + dn + d]), v = lat_f(row[h * hd + dn + half + d]);
-    const float c = cosr[d], s = sinr[d];
-    qo[h * QD + dn + d] = lat_t<T>(u * c - v * s);
-    qo[h * QD + dn + half + d] = lat_t<T>(v * c + u * s);
+  const int vh = half / V;
+  for (int i = threadIdx.x; i < H * vh; i += blockDim.x) {
+    using P = LatPack<T, V>;
+    const int h = i / vh, d = (i % vh) * V;
+    const P u = *reinterpret_cast<const P*>(row + h * hd + dn + d);
+    const P v = *reinterpret_cast<const P*>(row + h * hd + dn + half + d);
+    const LatPack<float, V> c = *reinterpret_cast<const LatPack<float, V>*>(cosr + d);
+    const LatPack<float, V> s = *reinterpret_cast<const LatPack<float, V>*>(sinr + d);
+    P a, b;
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      a.v[j] = lat_t<T>(lat_f(u.v[j]) * c.v[j] - lat_f(v.v[j]) * s.v[j]);
+      b.v[j] = lat_t<T>(lat_f(v.v[j]) * c.v[j] + lat_f(u.v[j]) * s.v[j]);
+    }
+    *reinterpret_cast<P*>(qo + h * QD + dn + d) = a;
+    *reinterpret_cast<P*>(qo + h * QD + dn + half + d) = b;
   }
   for (int i = threadIdx.x; i < H * vp; i += blockDim.x) {
     const int h = i / vp, d = hd + (i % vp) * V;
@@ -218,8 +228,11 @@ std::tuple<at::Tensor, at::Tensor, at::Tensor> latent_prep(
   auto kr = at::empty({rows_pad, dr}, qkv.options());
   if (rows_pad == 0) return {q, c, kr};
   auto stream = c10::hip::getCurrentHIPStream();
-  const bool vec = dn % 4 == 0 && (dn + dr) % 4 == 0 && head_pad % 4 == 0 && rank % 4 == 0 &&
-                   dr % 4 == 0;
+  // every offset and row start a multiple of the vector, tables included
+  auto all = [&](int64_t m) {
+    return dn % m == 0 && dr % (2 * m) == 0 && head_pad % m == 0 && rank % m == 0 &&
+           cos.size(1) % m == 0;
+  };
 #define LAUNCH(TT, VV)                                                                         \
   latent_prep_kernel<TT, VV><<<dim3(rows_pad), dim3(256), 0, stream>>>(                        \
       reinterpret_cast<const TT*>(qkv.data_ptr()), reinterpret_cast<const TT*>(w.data_ptr()),  \
@@ -229,9 +242,9 @@ std::tuple<at::Tensor, at::Tensor, at::Tensor> latent_prep(
       reinterpret_cast<TT*>(q.data_ptr()), (int)head_pad, reinterpret_cast<TT*>(c.data_ptr()), \
       reinterpret_cast<TT*>(kr.data_ptr()), (int)T, (int)heads, (int)dn, (int)dr, (int)rank)
   if (dt == at::kBFloat16) {
-    if (vec) LAUNCH(bf16, 4); else LAUNCH(bf16, 1);
+    if (all(8)) LAUNCH(bf16, 8); else if (all(4)) LAUNCH(bf16, 4); else LAUNCH(bf16, 1);
   } else {
-    if (vec) LAUNCH(float, 4); else LAUNCH(float, 1);
+    if (all(4)) LAUNCH(float, 4); else LAUNCH(float, 1);
   }
 #undef LAUNCH
   HIP_CHECK_KERNEL();
