@@ -39,6 +39,17 @@ def load_hf_state_dict(path: str) -> dict[str, torch.Tensor]:
     return sd
 
 
+def hf_tensor_shapes(path: str) -> dict[str, tuple[int, ...]]:
+    """Names and shapes of a checkpoint's tensors, from the file headers."""
+    from safetensors import safe_open
+
+    shapes: dict[str, tuple[int, ...]] = {}
+    for fn in _iter_safetensor_files(path):
+        with safe_open(fn, framework="pt") as f:
+            shapes.update((k, tuple(f.get_slice(k).get_shape())) for k in f.keys())
+    return shapes
+
+
 def load_hf_weights_streaming(model: torch.nn.Module, path: str,
                               strict: bool = True) -> None:
     """Shard-by-shard HF load into a DTensor-sharded model WITHOUT ever

@@ -1,6 +1,9 @@
 """Decoder building blocks around a 32-bit residual stream.
 
 * ``SquaredReluMLP``: up -> max(x, 0)^2 -> down.
+* ``ClampedGluMLP``: [gate; up] -> clamped gated unit -> down.
+* ``HyperConnection``: a sublayer's input norm and its weights towards several
+  residual streams (``ops/hyper.py``).
 * ``SandwichLayer``: every sublayer is normed before and after, and enters the
   residual with a constant factor. Consecutive layers hand the next normed
   input along, so that each residual update is one fused kernel.
@@ -14,6 +17,7 @@ from __future__ import annotations
 import torch
 import torch.nn as nn
 
+from automodel_amd.ops.hyper import clamped_glu, hyper_step
 from automodel_amd.ops.residual_norm import concat_cast, residual_add_norm
 from automodel_amd.ops.rms_norm import RMSNorm
 from automodel_amd.serving.decode_linear import project
@@ -27,6 +31,39 @@ class SquaredReluMLP(nn.Module):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         return project(self.down_proj, project(self.up_proj, h, relu2=True))
+
+
+class ClampedGluMLP(nn.Module):
+    """``gate_up_proj`` stacks the gate and the up projection."""
+
+    def __init__(self, width: int, inter: int, limit: float, alpha: float = 1.702):
+        super().__init__()
+        self.limit, self.alpha = limit, alpha
+        self.gate_up_proj = nn.Linear(width, 2 * inter, bias=False)
+        self.down_proj = nn.Linear(inter, width, bias=False)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return project(self.down_proj, clamped_glu(project(self.gate_up_proj, h), self.limit,
+                                                   self.alpha))
+
+
+class HyperConnection(nn.Module):
+    """Around one sublayer: ``norm`` and ``w_in`` [streams] make its input,
+    ``w_mix`` [from, to] and ``w_out`` [streams] the streams after it."""
+
+    def __init__(self, width: int, streams: int, eps: float, norm_backend: str = "hip"):
+        super().__init__()
+        self.eps = eps
+        self.norm = RMSNorm(width, eps, norm_backend)
+        self.w_in = nn.Parameter(torch.full((streams,), 1.0 / streams))
+        self.w_out = nn.Parameter(torch.ones(streams))
+        self.w_mix = nn.Parameter(torch.eye(streams))
+
+    def update(self, x, y, nxt: "HyperConnection | None", final_norm, keep: bool = True):
+        """Streams after this sublayer's output y, and the input of the next one
+        (or, without, the normed sum of the streams)."""
+        w_in, w_norm = (None, final_norm) if nxt is None else (nxt.w_in, nxt.norm.weight)
+        return hyper_step(x, y, self.w_mix, self.w_out, w_in, w_norm, self.eps, keep)
 
 
 class SandwichLayer(nn.Module):

@@ -1,0 +1,419 @@
+"""Papidra: a small decoder-only language model with hyper-connections.
+
+Several float32 residual streams run around two kinds of mixer: chunked grouped
+attention and a state-space recurrence side by side ('parallel', the mean of the
+two normed branches), and RWKV-style time mixing ('wkv'). A clamped gated
+feed-forward follows where a layer has one; the output is the embedding table.
+Every layer has its own kind and sizes.
+
+Built from the shared parts in ``models/common`` (grouped attention, recurrent
+mixers, hyper-connections) and decoded through
+``utils/kv_cache.MixerStateCache``.
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass, field
+from typing import Any
+
+import torch
+import torch.nn as nn
+
+from automodel_amd.models.common.backend import BackendConfig
+from automodel_amd.models.common.blocks import ClampedGluMLP, HyperConnection
+from automodel_amd.models.common.grouped import GroupedAttention
+from automodel_amd.models.common.recurrent import StateSpace, StateSpaceSpec, TimeMixing
+from automodel_amd.ops.grouped_attention import GroupedAttentionSpec
+from automodel_amd.ops.hyper import NormedPair, hyper_embed
+from automodel_amd.ops.packed_step import PackedStep
+from automodel_amd.ops.rms_norm import RMSNorm
+from automodel_amd.serving.decode_linear import project
+from automodel_amd.utils.kv_cache import MixerStateCache, active_kv_cache
+
+
+def _rope_scaling(scaling: dict | None) -> tuple | None:
+    if not scaling:
+        return None
+    return (("rope_type", "yarn"), ("factor", float(scaling["factor"])),
+            ("beta_fast", float(scaling["fast"])), ("beta_slow", float(scaling["slow"])),
+            ("original_max_position_embeddings", float(scaling["original"])))
+
+
+@dataclass
+class PapidraConfig:
+    """``layers`` holds one dict per layer, as the checkpoint's config does:
+    ``{"type": "parallel" | "wkv", "mixer": {...}, "mlp": {...} | None}``.
+    Without it, a stack that alternates the two is made from the scalar sizes.
+
+    ``wkv_rank`` is the decay's inner size: one number, or one per layer. A
+    checkpoint's config does not carry it (``complete_from_shapes``)."""
+
+    vocab_size: int = 32000
+    hidden_size: int = 2048
+    layers: list | None = None
+    streams: int = 2
+    embedding_scale: float = 1.0
+    rms_norm_eps: float = 1e-6
+    initializer_range: float = 0.02
+    wkv_rank: int | dict[int, int] = 64
+    # alternating stack (used when ``layers`` is not given)
+    num_hidden_layers: int = 4
+    num_attention_heads: int = 16
+    num_key_value_heads: int = 4
+    head_dim: int = 128
+    chunk_size: int = 8192
+    rope_theta: float = 500000.0
+    intermediate_size: int = 8192
+    glu_limit: float = 7.0
+    ssm_head_dim: int = 64
+    ssm_state_size: int = 128
+    ssm_groups: int = 8
+    conv_kernel: int = 4
+    wkv_head_dim: int = 64
+    num_wkv_heads: int | None = None
+    _kinds: tuple = field(default=("parallel", "wkv"), repr=False)
+
+    def __post_init__(self):
+        if self.layers is None:
+            self.layers = [self._uniform_layer(self._kinds[i % 2])
+                           for i in range(self.num_hidden_layers)]
+        self.num_hidden_layers = len(self.layers)
+        if self.streams < 1:
+            raise ValueError("at least one residual stream")
+        for i, layer in enumerate(self.layers):
+            if layer.get("type") not in self._kinds:
+                raise ValueError(f"layer {i}: unknown mixer type {layer.get('type')!r}")
+            mlp = layer.get("mlp")
+            if mlp is not None and mlp.get("kind") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+            if layer["type"] == "parallel":             # these validate the sizes
+                self.attention_spec(i), self.state_space_spec(i)
+
+    def _uniform_layer(self, kind: str) -> dict:
+        if kind == "parallel":
+            heads = max(1, 2 * self.hidden_size // self.ssm_head_dim)
+            groups = self.ssm_groups if heads % self.ssm_groups == 0 else 1
+            mixer = {"left": {"heads": self.num_attention_heads,
+                              "kv_heads": self.num_key_value_heads, "dim": self.head_dim,
+                              "vdim": self.head_dim, "scale": self.head_dim ** -0.5,
+                              "mask": {"size": self.chunk_size},
+                              "rot": {"base": self.rope_theta, "dims": self.head_dim}},
+                     "right": {"heads": heads, "vdim": self.ssm_head_dim,
+                               "state": self.ssm_state_size, "groups": groups,
+                               "norm_groups": groups, "conv": self.conv_kernel}}
+        else:
+            heads = self.num_wkv_heads or max(1, self.hidden_size // self.wkv_head_dim)
+            mixer = {"heads": heads, "dim": self.wkv_head_dim}
+        return {"type": kind, "mixer": mixer,
+                "mlp": {"kind": "dense", "ff": self.intermediate_size, "limit": self.glu_limit}}
+
+    def attention_spec(self, i: int) -> GroupedAttentionSpec:
+        m = self.layers[i]["mixer"]["left"]
+        rot = m["rot"]
+        return GroupedAttentionSpec(
+            heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+            scale=float(m["scale"]), rot_dim=rot["dims"], rope_base=float(rot["base"]),
+            rope_scaling=_rope_scaling(rot.get("scaling")), chunk=int(m["mask"]["size"]))
+
+    def state_space_spec(self, i: int) -> StateSpaceSpec:
+        m = self.layers[i]["mixer"]["right"]
+        return StateSpaceSpec(heads=m["heads"], vdim=m["vdim"], state=m["state"],
+                              groups=m["groups"], norm_groups=m["norm_groups"], conv=m["conv"],
+                              eps=self.rms_norm_eps)
+
+    def decay_rank(self, i: int) -> int:
+        return self.wkv_rank[i] if isinstance(self.wkv_rank, dict) else self.wkv_rank
+
+    def complete_from_shapes(self, shapes: dict[str, tuple[int, ...]]) -> None:
+        """Take the decays' inner sizes from a checkpoint's tensors, if there are any."""
+        ranks = {i: shapes[f"l{i}.mix.w1"][0] for i, layer in enumerate(self.layers)
+                 if layer["type"] == "wkv" and f"l{i}.mix.w1" in shapes}
+        if ranks:
+            self.wkv_rank = ranks
+
+    @classmethod
+    def from_hf_config(cls, hf: Any) -> "PapidraConfig":
+        if hasattr(hf, "to_dict"):
+            hf = hf.to_dict()
+        return cls(vocab_size=hf["vocab"], hidden_size=hf["width"], layers=hf["layers"],
+                   streams=int(hf["streams"]), embedding_scale=float(hf["embedding"]["scale"]),
+                   rms_norm_eps=float(hf["norm"]["eps"]))
+
+
+class ParallelMixer(nn.Module):
+    """Attention and state space on the same input; ``in_proj`` stacks the
+    projections of both (one GEMM)."""
+
+    def __init__(self, width: int, attn: GroupedAttentionSpec, ssm: StateSpaceSpec,
+                 norm_backend: str):
+        super().__init__()
+        self.in_proj = nn.Linear(width, attn.in_width + ssm.in_width, bias=False)
+        self.left = GroupedAttention(width, attn, sink=True)
+        self.right = StateSpace(width, ssm)
+        self.left_norm = RMSNorm(width, ssm.eps, norm_backend)
+        self.right_norm = RMSNorm(width, ssm.eps, norm_backend)
+
+    @property
+    def rope_spec(self) -> GroupedAttentionSpec:
+        return self.left.spec
+
+    def make_state(self, *where) -> dict[str, torch.Tensor]:
+        return {**self.left.make_state(*where), **self.right.make_state(*where)}
+
+    def forward(self, h: torch.Tensor, step: PackedStep, rope, state=None) -> NormedPair:
+        proj = project(self.in_proj, h)
+        return NormedPair(self.left(proj, step, rope, state),
+                          self.right(proj[:, self.left.spec.in_width:], step, state),
+                          self.left_norm.weight, self.right_norm.weight)
+
+
+class PapidraLayer(nn.Module):
+    def __init__(self, cfg: PapidraConfig, i: int, norm_backend: str):
+        super().__init__()
+        spec, W, eps = cfg.layers[i], cfg.hidden_size, cfg.rms_norm_eps
+        if spec["type"] == "parallel":
+            self.mixer = ParallelMixer(W, cfg.attention_spec(i), cfg.state_space_spec(i),
+                                       norm_backend)
+        else:
+            m = spec["mixer"]
+            self.mixer = TimeMixing(W, m["heads"], m["dim"], cfg.decay_rank(i), eps)
+        self.mixer_hc = HyperConnection(W, cfg.streams, eps, norm_backend)
+        mlp = spec.get("mlp")
+        self.mlp = self.mlp_hc = None
+        if mlp is not None:
+            self.mlp = ClampedGluMLP(W, mlp["ff"], float(mlp["limit"]))
+            self.mlp_hc = HyperConnection(W, cfg.streams, eps, norm_backend)
+
+
+class PapidraModel(nn.Module):
+    def __init__(self, cfg: PapidraConfig, backend: BackendConfig):
+        super().__init__()
+        self.cfg = cfg
+        self.embed_tokens = nn.Embedding(cfg.vocab_size, cfg.hidden_size)
+        self.layers = nn.ModuleList(PapidraLayer(cfg, i, backend.rms_norm)
+                                    for i in range(len(cfg.layers)))
+        self.norm = RMSNorm(cfg.hidden_size, cfg.rms_norm_eps, backend.rms_norm)
+        self._rope: dict[tuple, tuple[torch.Tensor, torch.Tensor]] = {}
+
+    def rope_tables(self, spec: GroupedAttentionSpec, n: int, device):
+        """cos/sin for at least ``n`` positions, kept per kind of rotation."""
+        key = (*spec.rope_key, str(device))
+        have = self._rope.get(key)
+        if have is None or have[0].shape[0] < n:
+            n = max(64, 1 << (n - 1).bit_length())
+            have = self._rope[key] = spec.rope_tables(n, device)
+        return have
+
+    def forward(self, ids: torch.Tensor, step: PackedStep, max_pos: int, cache=None,
+                final_rows: torch.Tensor | None = None) -> torch.Tensor:
+        """ids [T] packed tokens -> normed hidden rows (``final_rows`` only)."""
+        subs = []                                  # (layer, its sublayer, hyper-connection)
+        for layer in self.layers:
+            subs.append((layer.mixer, layer.mixer_hc))
+            if layer.mlp is not None:
+                subs.append((layer.mlp, layer.mlp_hc))
+        first, eps = subs[0][1], self.cfg.rms_norm_eps
+        x, h = hyper_embed(ids, self.embed_tokens.weight, self.cfg.embedding_scale, first.w_in,
+                           first.norm.weight, eps)
+        last_mixer = len(subs) - 1 - (self.layers[-1].mlp is not None)
+        for n, (sub, hc) in enumerate(subs):
+            if isinstance(sub, ClampedGluMLP):
+                y = sub(h)
+            else:
+                state = None if cache is None else cache.next_layer()
+                if isinstance(sub, ParallelMixer):
+                    rope = self.rope_tables(sub.rope_spec, max_pos, ids.device)
+                    y = sub(h, step, rope, state)
+                else:
+                    y = sub(h, step, state)
+            if n == last_mixer and final_rows is not None:
+                # what follows works on rows alone
+                x = x[final_rows]
+                y = y.rows(final_rows) if isinstance(y, NormedPair) else y[final_rows]
+            last = n + 1 == len(subs)
+            x, h = hc.update(x, y, None if last else subs[n + 1][1], self.norm.weight,
+                             keep=not last)
+        return h
+
+
+class PapidraForCausalLM(nn.Module):
+    hf_architectures = ("Papidra",)
+    config_class = PapidraConfig
+
+    @staticmethod
+    def config_from_hf(hf_cfg) -> PapidraConfig:
+        return PapidraConfig.from_hf_config(hf_cfg)
+
+    def __init__(self, config: PapidraConfig | dict,
+                 backend: BackendConfig | dict | None = None):
+        super().__init__()
+        if isinstance(config, dict):
+            config = PapidraConfig(**config)
+        backend = BackendConfig.resolve(
+            backend, "cuda" if torch.cuda.is_available() else "cpu")
+        self.config = config
+        self.backend = backend
+        self.model = PapidraModel(config, backend)
+        self.lm_head = nn.Linear(config.hidden_size, config.vocab_size, bias=False)
+        self.lm_head.weight = self.model.embed_tokens.weight
+        self.loss_fn = None
+        self.state_dict_adapter = PapidraStateDictAdapter(config)
+
+    def make_cache(self, batch: int, max_len: int) -> MixerStateCache:
+        p = self.lm_head.weight
+        return MixerStateCache([layer.mixer for layer in self.model.layers], batch, max_len,
+                               p.device, p.dtype)
+
+    def forward(self, input_ids: torch.Tensor, labels: torch.Tensor | None = None,
+                return_hidden: bool = False, **_: Any) -> torch.Tensor:
+        """[B, S] rectangular ids -> loss / hidden / logits [B, S, vocab].
+
+        Under a slot cache (``utils/kv_cache``) the ids are the packed tokens
+        of the cache's planned step, whatever their shape; returned are the
+        logits [n, vocab] of the rows the plan asks for (all without a list),
+        in float32.
+        """
+        cache = active_kv_cache()
+        if cache is not None:
+            step = cache.step
+            assert step is not None and input_ids.numel() == step.positions.numel(), (
+                "slot cache: plan a step of as many tokens as are given")
+            h = self.model(input_ids.reshape(-1), step, cache.max_len, cache, step.logit_rows)
+            return project(self.lm_head, h, out_f32=True)
+        B, S = input_ids.shape
+        step = PackedStep.for_prompts([S] * B, input_ids.device)
+        hidden = self.model(input_ids.reshape(-1), step, S).view(B, S, -1)
+        if labels is not None:
+            assert self.loss_fn is not None, "set model.loss_fn before passing labels"
+            return self.loss_fn(hidden, self.lm_head.weight, labels)
+        if return_hidden:
+            return hidden
+        return project(self.lm_head, hidden.reshape(B * S, -1)).view(B, S, -1)
+
+    @torch.no_grad()
+    def init_weights(self, device=None) -> None:
+        std = self.config.initializer_range
+        if device is not None:
+            self.to_empty(device=device)
+            self.lm_head.weight = self.model.embed_tokens.weight
+        for m in self.modules():
+            if isinstance(m, (nn.Linear, nn.Embedding)):
+                nn.init.normal_(m.weight, std=std)
+            elif isinstance(m, RMSNorm):
+                nn.init.ones_(m.weight)
+            elif isinstance(m, HyperConnection):
+                m.w_in.fill_(1.0 / m.w_in.numel())
+                m.w_out.fill_(1.0)
+                m.w_mix.copy_(torch.eye(m.w_in.numel()))
+            elif isinstance(m, GroupedAttention):
+                m.sink.zero_()
+            elif isinstance(m, StateSpace):
+                nn.init.normal_(m.conv_weight, std=m.spec.conv ** -0.5)
+                m.conv_bias.zero_()
+                m.dt_bias.fill_(-3.0)                # steps of about 0.05
+                m.A_log.copy_(torch.linspace(1.0, 16.0, m.spec.heads).log())
+                m.D.fill_(1.0)
+                m.norm_weight.fill_(1.0)
+            elif isinstance(m, TimeMixing):
+                m.mu.fill_(0.5)
+                m.decay_bias.copy_(torch.linspace(-6.0, -1.0, m.dim).repeat(m.heads))
+                m.bonus.zero_()
+                m.norm_weight.fill_(1.0)
+
+    def num_parameters(self) -> int:
+        return sum(p.numel() for p in self.parameters())
+
+
+class PapidraStateDictAdapter:
+    """Checkpoint tensors <-> parameters: names, and the stacked projections."""
+
+    _LAYER = {
+        "mix.left.sink": "mixer.left.sink", "mix.left.o": "mixer.left.o_proj.weight",
+        "mix.left.out": "mixer.left_norm.weight", "mix.right.out": "mixer.right_norm.weight",
+        "mix.right.conv": "mixer.right.conv_weight", "mix.right.conv.b": "mixer.right.conv_bias",
+        "mix.right.dt_bias": "mixer.right.dt_bias", "mix.right.A_log": "mixer.right.A_log",
+        "mix.right.D": "mixer.right.D", "mix.right.norm": "mixer.right.norm_weight",
+        "mix.right.o": "mixer.right.o_proj.weight",
+        "mix.w2": "mixer.decay_proj.weight", "mix.w0": "mixer.decay_bias",
+        "mix.u": "mixer.bonus", "mix.norm": "mixer.norm_weight", "mix.o": "mixer.o_proj.weight",
+        "mlp.down": "mlp.down_proj.weight",
+        **{f"{a}{i}{b}": f"{sub}_hc.{to}" for i, sub in ((1, "mixer"), (2, "mlp"))
+           for a, b, to in (("norm", "", "norm.weight"), ("hc", ".in", "w_in"),
+                            ("hc", ".out", "w_out"), ("hc", ".mix", "w_mix"))},
+    }
+    # one parameter from several tensors, stacked along dim 0
+    _STACKED = {
+        "mlp.gate_up_proj.weight": ("mlp.gate", "mlp.up"),
+        "parallel mixer.in_proj.weight": ("mix.left.q", "mix.left.k", "mix.left.v",
+                                          "mix.right.in"),
+        "wkv mixer.in_proj.weight": ("mix.r", "mix.k", "mix.v", "mix.g", "mix.w1"),
+        "mixer.mu": ("mix.mu.r", "mix.mu.k", "mix.mu.v", "mix.mu.g", "mix.mu.w"),
+    }
+    _TOP = {"embed": "model.embed_tokens.weight", "final.norm": "model.norm.weight"}
+    _TIED = "lm_head.weight"
+
+    def __init__(self, config: PapidraConfig):
+        self.config = config
+        self._part = {p: (to.split()[-1], parts.index(p), len(parts))
+                      for to, parts in self._STACKED.items() for p in parts}
+
+    def hf_key_targets(self, key: str) -> list[str]:
+        """Parameter name(s) a checkpoint key feeds."""
+        if key in self._TOP:
+            return [self._TOP[key]]
+        layer, _, name = key.partition(".")
+        if layer[:1] == "l" and layer[1:].isdigit():
+            p = f"model.layers.{layer[1:]}."
+            if name in self._LAYER:
+                return [p + self._LAYER[name]]
+            if name in self._part:
+                return [p + self._part[name][0]]
+        return [key]
+
+    def from_hf(self, sd: dict) -> dict:
+        out, stacked = {}, {}
+        for key, t in sd.items():
+            target = self.hf_key_targets(key)[0]
+            part = self._part.get(key.partition(".")[2]) if target != key else None
+            if part is None:
+                out[target] = t
+            else:
+                stacked.setdefault(target, [None] * part[2])[part[1]] = t
+        for target, parts in stacked.items():
+            if all(p is not None for p in parts):
+                out[target] = (torch.stack if target.endswith(".mu") else torch.cat)(parts)
+        if self._TOP["embed"] in out:
+            out[self._TIED] = out[self._TOP["embed"]]
+        return out
+
+    def _part_sizes(self, i: int, parts: tuple) -> list[int]:
+        cfg, spec = self.config, self.config.layers[i]
+        if parts[0] == "mlp.gate":
+            return [spec["mlp"]["ff"]] * 2
+        if parts[0] == "mix.r":
+            n = spec["mixer"]["heads"] * spec["mixer"]["dim"]
+            return [n] * 4 + [cfg.decay_rank(i)]
+        a = cfg.attention_spec(i)
+        return [a.heads * a.dim, a.kv_heads * a.dim, a.kv_heads * a.vdim,
+                cfg.state_space_spec(i).in_width]
+
+    def to_hf(self, sd: dict) -> dict:
+        top = {v: k for k, v in self._TOP.items()}
+        per_layer = {v: k for k, v in self._LAYER.items()}
+        out = {}
+        for key, t in sd.items():
+            if key == self._TIED:
+                continue
+            if key in top:
+                out[top[key]] = t
+                continue
+            _, _, i, name = key.split(".", 3)           # model.layers.<i>.<name>
+            if name in per_layer:
+                out[f"l{i}.{per_layer[name]}"] = t
+                continue
+            kind = self.config.layers[int(i)]["type"]
+            parts = self._STACKED.get(name) or self._STACKED[f"{kind} {name}"]
+            pieces = t.unbind(0) if name.endswith(".mu") else t.split(
+                self._part_sizes(int(i), parts))
+            out.update((f"l{i}.{p}", x) for p, x in zip(parts, pieces))
+        return out

@@ -388,6 +388,13 @@ def _ensure_builtin() -> None:
     except ImportError:
         pass
     try:
+        from automodel_amd.models.papidra.model import PapidraForCausalLM
+
+        for name in PapidraForCausalLM.hf_architectures:
+            _REGISTRY[name] = PapidraForCausalLM
+    except ImportError:
+        pass
+    try:
         from automodel_amd.models.rezadra.model import RezadraForCausalLM
 
         for name in RezadraForCausalLM.hf_architectures:
@@ -440,6 +447,11 @@ def build_model(
             from automodel_amd.models.llama.model import LlamaConfig
 
             model_cfg = LlamaConfig.from_hf_config(hf_cfg)
+        if hasattr(model_cfg, "complete_from_shapes"):
+            # sizes that only the checkpoint's tensors tell
+            from automodel_amd.checkpoint.hf_loader import hf_tensor_shapes
+
+            model_cfg.complete_from_shapes(hf_tensor_shapes(pretrained_path))
     else:
         assert config is not None, "build_model needs config= or pretrained_path="
         try:

@@ -4,8 +4,8 @@ Compiles every ``csrc/*.hip`` + ``csrc/bind.cpp`` with hipcc in parallel and
 links ``automodel_amd/ops/libamd_ops.so``. No JIT cache: the .so lives in the
 package so it travels with the repo snapshot to GPU boxes.
 
-``--decode`` links only the inference kernels (attention forward, latent
-attention, residual norms, decode GEMV) into ``libamd_ops_decode.so``: what a
+``--decode`` links only the inference kernels (attention forward, latent and
+grouped attention, linear recurrences, residual norms, decode GEMV) into ``libamd_ops_decode.so``: what a
 checkout with nothing built needs to generate, in a fraction of the time.
 
 Usage: ``python -m automodel_amd.ops.build [--force] [--decode]``
@@ -25,8 +25,9 @@ CSRC = os.path.join(PKG_DIR, "csrc")
 BUILD_DIR = os.path.join(PKG_DIR, "_build")
 SO_PATH = os.path.join(PKG_DIR, "libamd_ops.so")
 DECODE_SO_PATH = os.path.join(PKG_DIR, "libamd_ops_decode.so")
-DECODE_SOURCES = ("bind_decode.cpp", "flash_attn.hip", "gemv.hip",
-                  "latent_attn.hip", "latent_decode.hip", "residual_norm.hip")
+DECODE_SOURCES = ("bind_decode.cpp", "flash_attn.hip", "gemv.hip", "gqa_attn.hip",
+                  "hyper.hip", "latent_attn.hip", "latent_decode.hip", "linear_scan.hip",
+                  "residual_norm.hip")
 ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 

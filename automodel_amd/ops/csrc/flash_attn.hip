@@ -47,7 +47,7 @@ template <int DQK, int DV, int WAVES, bool VARLEN>
 __global__ __launch_bounds__(WAVES * WAVE_SIZE, 2) void flash_fwd_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k, const bf16* __restrict__ v,
     bf16* __restrict__ out, float* __restrict__ lse, const int* __restrict__ doc_start,
-    int B, int Sq, int Skv, int Hq, int Hk, int q_start, float scale, bool causal) {
+    const bf16* __restrict__ sink, int B, int Sq, int Skv, int Hq, int Hk, int q_start, float scale, bool causal) {
   constexpr int KB = pad256(DQK * 2);     // K tile row stride (bytes)
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* k_lds = smem;                               // KVBLK*KB
@@ -265,7 +265,10 @@ __global__ __launch_bounds__(WAVES * WAVE_SIZE, 2) void flash_fwd_kernel(
     __syncthreads();
   }
 
-  // ---- epilogue: normalize by l, write O and LSE
+  // ---- epilogue: normalize by l, write O and LSE. A sink is one more logit in
+  // the denominator, without a key (m_run bounds the scores, so that only a
+  // sink far above all of them can overflow: the output is 0 then, as it is)
+  if (sink) l_run += __expf(bf2f(sink[h]) - m_run);
   if (lane < 32) bcast[wid * 32 + lane] = (l_run > 0.f) ? 1.f / l_run : 0.f;
   __syncthreads();
 
@@ -290,7 +293,7 @@ __global__ __launch_bounds__(WAVES * WAVE_SIZE, 2) void flash_fwd_kernel(
 template <int DQK, int DV, int WAVES, bool VARLEN>
 static void launch_fwd(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
                        at::Tensor& out, at::Tensor& lse, const int* doc_start,
-                       int B, int Sq, int Skv, int Hq, int Hk, int q_start,
+                       const bf16* sink, int B, int Sq, int Skv, int Hq, int Hk, int q_start,
                        float scale, bool causal, hipStream_t stream) {
   const dim3 grid(Sq / (WAVES * QBLK), Hq, B);
   const size_t smem = KVBLK * pad256(DQK * 2) + sub_img_bytes<DV>() +
@@ -301,13 +304,14 @@ static void launch_fwd(const at::Tensor& q, const at::Tensor& k, const at::Tenso
                      reinterpret_cast<const bf16*>(k.data_ptr()),
                      reinterpret_cast<const bf16*>(v.data_ptr()),
                      reinterpret_cast<bf16*>(out.data_ptr()), lse.data_ptr<float>(),
-                     doc_start, B, Sq, Skv, Hq, Hk, q_start, scale, causal);
+                     doc_start, sink, B, Sq, Skv, Hq, Hk, q_start, scale, causal);
   HIP_CHECK_KERNEL();
 }
 
 std::tuple<at::Tensor, at::Tensor> flash_attn_fwd(
     const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, double scale,
-    bool causal, int64_t q_start, const std::optional<at::Tensor>& doc_start) {
+    bool causal, int64_t q_start, const std::optional<at::Tensor>& doc_start,
+    const std::optional<at::Tensor>& sink) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 4 && q.scalar_type() == at::kBFloat16,
               "flash_attn_fwd: q must be [B,S,Hq,D] bf16");
   const int B = q.size(0), Sq = q.size(1), Hq = q.size(2), Dqk = q.size(3);
@@ -318,6 +322,10 @@ std::tuple<at::Tensor, at::Tensor> flash_attn_fwd(
   const bool varlen = doc_start.has_value();
   const int* ds_ptr = varlen ? doc_start->data_ptr<int>() : nullptr;
   if (varlen) TORCH_CHECK(causal && B == 1, "varlen flash is causal with B==1");
+  if (sink)
+    TORCH_CHECK(sink->is_cuda() && sink->is_contiguous() && sink->numel() == Hq &&
+                    sink->scalar_type() == at::kBFloat16, "flash_attn_fwd: sink [Hq] bf16");
+  const bf16* sk_ptr = sink ? reinterpret_cast<const bf16*>(sink->data_ptr()) : nullptr;
   auto out = at::empty({B, Sq, Hq, Dv}, q.options());
   auto lse = at::empty({B, Hq, Sq}, q.options().dtype(at::kFloat));
   auto stream = c10::hip::getCurrentHIPStream().stream();
@@ -327,16 +335,16 @@ std::tuple<at::Tensor, at::Tensor> flash_attn_fwd(
   if (!done && Dqk == A && Dv == C) {                                                 \
     done = true;                                                                      \
     if (varlen && Sq % (8 * QBLK) == 0) {                                             \
-      launch_fwd<A, C, 8, true>(q, k, v, out, lse, ds_ptr, B, Sq, Skv, Hq, Hk,        \
+      launch_fwd<A, C, 8, true>(q, k, v, out, lse, ds_ptr, sk_ptr, B, Sq, Skv, Hq, Hk, \
                                 (int)q_start, (float)scale, causal, stream);          \
     } else if (varlen) {                                                              \
-      launch_fwd<A, C, 4, true>(q, k, v, out, lse, ds_ptr, B, Sq, Skv, Hq, Hk,        \
+      launch_fwd<A, C, 4, true>(q, k, v, out, lse, ds_ptr, sk_ptr, B, Sq, Skv, Hq, Hk, \
                                 (int)q_start, (float)scale, causal, stream);          \
     } else if (Sq % (8 * QBLK) == 0) {                                                \
-      launch_fwd<A, C, 8, false>(q, k, v, out, lse, nullptr, B, Sq, Skv, Hq, Hk,      \
+      launch_fwd<A, C, 8, false>(q, k, v, out, lse, nullptr, sk_ptr, B, Sq, Skv, Hq, Hk, \
                                  (int)q_start, (float)scale, causal, stream);         \
     } else {                                                                          \
-      launch_fwd<A, C, 4, false>(q, k, v, out, lse, nullptr, B, Sq, Skv, Hq, Hk,      \
+      launch_fwd<A, C, 4, false>(q, k, v, out, lse, nullptr, sk_ptr, B, Sq, Skv, Hq, Hk, \
                                  (int)q_start, (float)scale, causal, stream);         \
     }                                                                                 \
   }

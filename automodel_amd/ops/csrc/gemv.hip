@@ -39,7 +39,7 @@ template <int B>
 __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
     const bf16* __restrict__ W, const bf16* __restrict__ x,
     const bf16* __restrict__ bias, bf16* __restrict__ y, float* __restrict__ yf, bool relu2,
-    int N, int K) {
+    int N, int K, int group_n) {
   const int lane = threadIdx.x & (WAVE_SIZE - 1);
   const int wid = blockIdx.x * (blockDim.x / WAVE_SIZE) + (threadIdx.x / WAVE_SIZE);
   const int row0 = 2 * wid;
@@ -50,6 +50,7 @@ __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
   for (int b = 0; b < B; ++b) acc0[b] = acc1[b] = 0.f;
   const bf16* wrow0 = W + (long)row0 * K;
   const bf16* wrow1 = wrow0 + (two ? K : 0);
+  if (group_n) x += (long)(row0 / group_n) * B * K;   // group_n is even
   for (int k = lane * 8; k < K; k += WAVE_SIZE * 8) {
     const bf16x8 w0 = *reinterpret_cast<const bf16x8*>(wrow0 + k);
     const bf16x8 w1 = *reinterpret_cast<const bf16x8*>(wrow1 + k);
@@ -86,13 +87,20 @@ __global__ __launch_bounds__(256, 4) void gemv_bf16_kernel(
   }
 }
 
+// group_n > 0: x holds several [B, K] inputs one after another, and every
+// group_n rows of w take the next one.
 at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
-                     const c10::optional<at::Tensor>& bias, bool relu2, bool out_f32) {
+                     const c10::optional<at::Tensor>& bias, bool relu2, bool out_f32,
+                     int64_t group_n) {
   TORCH_CHECK(x.is_cuda() && w.is_cuda(), "gemv_bf16: GPU tensors required");
   TORCH_CHECK(x.dtype() == at::kBFloat16 && w.dtype() == at::kBFloat16,
               "gemv_bf16: bf16 only");
   TORCH_CHECK(x.dim() == 2 && w.dim() == 2, "gemv_bf16: x [B,K], w [N,K]");
-  const int B = (int)x.size(0), K = (int)x.size(1), N = (int)w.size(0);
+  const int K = (int)x.size(1), N = (int)w.size(0);
+  const int groups = group_n > 0 ? (int)((N + group_n - 1) / group_n) : 1;
+  TORCH_CHECK(group_n >= 0 && group_n % 2 == 0 && x.size(0) % groups == 0,
+              "gemv_bf16: an even group_n, and one [B,K] input per group");
+  const int B = (int)x.size(0) / groups;
   TORCH_CHECK(w.size(1) == K, "K mismatch");
   TORCH_CHECK(B >= 1 && B <= 16, "gemv_bf16: B in [1,16], got ", B,
               " (larger batches belong on hipBLASLt)");
@@ -113,7 +121,7 @@ at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
       reinterpret_cast<const bf16*>(wc.data_ptr()),                            \
       reinterpret_cast<const bf16*>(xc.data_ptr()), bptr,                      \
       out_f32 ? nullptr : reinterpret_cast<bf16*>(y.data_ptr()),               \
-      out_f32 ? y.data_ptr<float>() : nullptr, relu2, N, K)
+      out_f32 ? y.data_ptr<float>() : nullptr, relu2, N, K, (int)group_n)
   switch (B) {
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;
@@ -143,13 +151,14 @@ constexpr int SK_STRIDE = SK_KC * 2 + 16;         // LDS bytes per row
 template <int NB, int WAVES>
 __global__ __launch_bounds__(WAVES * WAVE_SIZE) void gemm_skinny_kernel(
     const bf16* __restrict__ W, const bf16* __restrict__ x, bf16* __restrict__ y,
-    float* __restrict__ yf, bool relu2, int B, int N, int K) {
+    float* __restrict__ yf, bool relu2, int B, int N, int K, int group_n) {
   constexpr int RED = WAVES * 16 * (16 * NB + 1) * 4;
   constexpr int TILE = 16 * (1 + NB) * SK_STRIDE;
   __shared__ __attribute__((aligned(16))) char lds[WAVES * TILE > RED ? WAVES * TILE : RED];
   const int lane = threadIdx.x & (WAVE_SIZE - 1), wid = threadIdx.x / WAVE_SIZE;
   const int lo16 = lane & 15, hi4 = lane >> 4;
   const int n0 = blockIdx.x * 16;
+  if (group_n) x += (long)(n0 / group_n) * B * K;       // group_n % 16 == 0
   char* wl = lds + wid * TILE;                    // [16][SK_STRIDE]
   char* xl = wl + 16 * SK_STRIDE;                 // [16 NB][SK_STRIDE]
 
@@ -225,11 +234,16 @@ __global__ __launch_bounds__(WAVES * WAVE_SIZE) void gemm_skinny_kernel(
   }
 }
 
-at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32) {
+at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32,
+                            int64_t group_n) {
   TORCH_CHECK(x.is_cuda() && w.is_cuda() && x.dtype() == at::kBFloat16 &&
                   w.dtype() == at::kBFloat16 && x.dim() == 2 && w.dim() == 2,
               "gemm_skinny_bf16: x [B,K], w [N,K] bf16 on the GPU");
-  const int B = (int)x.size(0), K = (int)x.size(1), N = (int)w.size(0);
+  const int K = (int)x.size(1), N = (int)w.size(0);
+  const int groups = group_n > 0 ? (int)((N + group_n - 1) / group_n) : 1;
+  TORCH_CHECK(group_n >= 0 && group_n % 16 == 0 && x.size(0) % groups == 0,
+              "gemm_skinny_bf16: group_n in whole tiles of 16, one [B,K] input per group");
+  const int B = (int)x.size(0) / groups;
   TORCH_CHECK(w.size(1) == K && K % 8 == 0 && K >= 8 && N >= 1, "gemm_skinny_bf16: K % 8 == 0");
   TORCH_CHECK(B >= 1 && B <= 64, "gemm_skinny_bf16: 1..64 rows, got ", B);
   auto xc = x.contiguous(), wc = w.contiguous();
@@ -241,7 +255,7 @@ at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2
           reinterpret_cast<const bf16*>(wc.data_ptr()),                                      \
           reinterpret_cast<const bf16*>(xc.data_ptr()),                                      \
           out_f32 ? nullptr : reinterpret_cast<bf16*>(y.data_ptr()),                         \
-          out_f32 ? y.data_ptr<float>() : nullptr, relu2, B, N, K)
+          out_f32 ? y.data_ptr<float>() : nullptr, relu2, B, N, K, (int)group_n)
   // waves per workgroup: enough of them across the chip, each with K left to
   // stream; LDS grows with the x rows
   const bool deep = K >= 2048;

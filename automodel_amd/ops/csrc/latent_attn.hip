@@ -114,7 +114,8 @@ template <typename T, typename TO>
 __global__ __launch_bounds__(256) void attn_rows_kernel(
     const T* __restrict__ q, long q_rs, long q_hs, const T* __restrict__ k, long k_rs, long k_hs,
     const T* __restrict__ v, long v_rs, long v_hs, const long* __restrict__ base,
-    const int* __restrict__ count, long n_rows, TO* __restrict__ out, int dq, int dv, float scale) {
+    const int* __restrict__ count, long n_rows, const T* __restrict__ sink, int per_k, int per_v,
+    TO* __restrict__ out, int dq, int dv, float scale) {
   extern __shared__ float sm[];
   float* qs = sm;                     // dq
   float* ps = sm + dq;                // 256
@@ -134,7 +135,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(
     const int j = j0 + tid;
     float s = -INFINITY;
     if (j < n) {
-      const T* kr = k + (b0 + j) * k_rs + h * k_hs;
+      const T* kr = k + (b0 + j) * k_rs + h / per_k * k_hs;
       float d = 0.f;
       for (int i = 0; i < dq; ++i) d = fmaf(qs[i], lat_f(kr[i]), d);
       s = d * scale;
@@ -157,14 +158,20 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(
     for (int c = 0; c < AR_COLS; ++c) {
       const int col = tid + c * 256;
       if (col >= dv) continue;
-      const T* vr = v + (b0 + j0) * v_rs + h * v_hs + col;
+      const T* vr = v + (b0 + j0) * v_rs + h / per_v * v_hs + col;
       float a = acc[c] * alpha;
       for (int jj = 0; jj < jn; ++jj) a = fmaf(ps[jj], lat_f(vr[jj * v_rs]), a);
       acc[c] = a;
     }
     __syncthreads();                              // before ps and red change
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float own = 1.f;
+  if (sink) {                                     // one more logit, without a key
+    const float s = lat_f(sink[h]), mn = fmaxf(m, s);
+    own = expf(m - mn);
+    l = l * own + expf(s - mn);
+  }
+  const float inv = l > 0.f ? own / l : 0.f;
 #pragma unroll
   for (int c = 0; c < AR_COLS; ++c) {
     const int col = tid + c * 256;
@@ -284,38 +291,43 @@ std::tuple<at::Tensor, at::Tensor> latent_assemble(const at::Tensor& kv, const a
   return {k, v};
 }
 
-// q [T, H, dq]; k/v [rows, Hk, d] with Hk == H or 1 (shared by all heads; v may
-// be a column slice of k). base [T] int64, count [T] int32. -> [T, H, dv]
+// q [T, H, dq]; k/v [rows, Hk, d], query heads in equal groups per key head (v
+// may be a column slice of k). base [T] int64, count [T] int32; sink [H], a
+// logit without a key. -> [T, H, dv]
 at::Tensor attn_rows(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
                      const at::Tensor& base, const at::Tensor& count, double scale,
-                     bool out_f32) {
+                     bool out_f32, const std::optional<at::Tensor>& sink) {
   TORCH_CHECK(is_t(q) && q.is_cuda() && q.dim() == 3 && k.dim() == 3 && v.dim() == 3,
-              "attn_rows: q [T,H,dq], k/v [rows,H or 1,d]");
+              "attn_rows: q [T,H,dq], k/v [rows,Hk,d]");
   const auto dt = q.scalar_type();
   TORCH_CHECK(k.is_cuda() && v.is_cuda() && k.scalar_type() == dt && v.scalar_type() == dt,
               "attn_rows: dtypes differ");
   TORCH_CHECK(q.stride(2) == 1 && k.stride(2) == 1 && v.stride(2) == 1,
               "attn_rows: head dims must be contiguous");
   const int64_t T = q.size(0), H = q.size(1), dq = q.size(2), dv = v.size(2);
-  TORCH_CHECK((k.size(1) == H || k.size(1) == 1) && (v.size(1) == H || v.size(1) == 1) &&
+  TORCH_CHECK(k.size(1) >= 1 && v.size(1) >= 1 && H % k.size(1) == 0 && H % v.size(1) == 0 &&
                   k.size(2) >= dq && k.size(0) == v.size(0),
               "attn_rows: k/v shapes");
   TORCH_CHECK(dq <= 8192 && dv <= 256 * AR_COLS && T <= 65535 * 16L, "attn_rows: sizes");
   TORCH_CHECK(base.is_cuda() && base.is_contiguous() && base.scalar_type() == at::kLong &&
                   base.numel() == T, "attn_rows: base int64 [T]");
   check_i32(count, T, "attn_rows count");
+  if (sink)
+    TORCH_CHECK(sink->is_cuda() && sink->is_contiguous() && sink->numel() == H &&
+                    sink->scalar_type() == dt, "attn_rows: sink [H]");
   auto out = at::empty({T, H, dv}, q.options().dtype(out_f32 ? at::kFloat : dt));
   if (T == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
   const size_t smem = (dq + 256 + 8) * sizeof(float);
-  const long khs = k.size(1) == 1 ? 0 : k.stride(1), vhs = v.size(1) == 1 ? 0 : v.stride(1);
+  const int per_k = (int)(H / k.size(1)), per_v = (int)(H / v.size(1));
   constexpr int64_t STEP = 32768;                       // grid.y limit is 65535
 #define LAUNCH(TT, TO)                                                                         \
   attn_rows_kernel<TT, TO><<<dim3(H, n), dim3(256), smem, stream>>>(                           \
       reinterpret_cast<const TT*>(q.data_ptr()) + t0 * q.stride(0), q.stride(0), q.stride(1),  \
-      reinterpret_cast<const TT*>(k.data_ptr()), k.stride(0), khs,                             \
-      reinterpret_cast<const TT*>(v.data_ptr()), v.stride(0), vhs,                             \
+      reinterpret_cast<const TT*>(k.data_ptr()), k.stride(0), k.stride(1),                     \
+      reinterpret_cast<const TT*>(v.data_ptr()), v.stride(0), v.stride(1),                     \
       base.data_ptr<long>() + t0, count.data_ptr<int>() + t0, (long)k.size(0),                 \
+      sink ? reinterpret_cast<const TT*>(sink->data_ptr()) : nullptr, per_k, per_v,             \
       reinterpret_cast<TO*>(out.data_ptr()) + t0 * H * dv, (int)dq, (int)dv, (float)scale)
   for (int64_t t0 = 0; t0 < T; t0 += STEP) {
     const int64_t n = std::min(STEP, T - t0);

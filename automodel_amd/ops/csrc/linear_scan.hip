@@ -1,0 +1,878 @@
+// Linear recurrences with a matrix state per head, over packed prompts and one
+// token at a time (inference). The state S [K, P] is f32 throughout.
+//
+//   state space   S_t = a_t S_(t-1) + dt_t B_t x_t^T,   y_t = S_t^T C_t + D x_t
+//                 one decay a_t = exp(-exp(A_log) dt_t) per head
+//   wkv           o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,
+//                 S_t = diag(w_t) S_(t-1) + k_t v_t^T, a decay per key channel
+//
+//   causal_conv_silu    short convolution per channel, with its cached inputs
+//   token_shift         h + (h' - h) * mu for several mu, h' the token before
+//   decay_cumsum        log decays summed within blocks of 16 tokens
+//   ssd_prompt / wkv_prompt   blocks of 16 tokens on the f32 matrix cores
+//   ssd_decode / wkv_decode   one token per sequence
+//   gated_group_norm    rms norm in equal groups, gated before or after
+//
+// The prompt kernels hold S in the accumulators of 16x16x4 f32 MFMAs: a wave
+// owns 16 columns of one head and walks its sequence. A lane (g, c) of S has
+// keys 4g..4g+3 of a tile, which is an MFMA operand once the summed index is
+// permuted in both operands alike; so S, the values and the 16x16 matrix within
+// a block are all used where they are, and only queries and keys pass through
+// LDS. Every exponent taken is of a non-positive sum, however strong the decay.
+
+#include <torch/library.h>
+#include <ATen/ATen.h>
+#include <c10/hip/HIPStream.h>
+
+#include "elem.h"
+#include "ops_api.h"
+
+namespace amd_ops {
+
+typedef float scan_f32x4 __attribute__((ext_vector_type(4)));
+
+namespace {
+
+constexpr int TB = 16;                 // tokens per block
+// A log decay below this is a factor of 0 in f32; the bound keeps sums of log
+// decays (of which differences are taken) accurate.
+constexpr float MIN_LOG = -90.f;
+
+__device__ __forceinline__ scan_f32x4 mfma4(float a, float b, scan_f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+// ---------------------------------------------------------------------------
+// short convolution and token shift
+// ---------------------------------------------------------------------------
+constexpr int CONV_TOKENS = 8;         // per workgroup: the taps stay in registers
+
+// TAPS 0: any number of them, weights from memory
+template <typename T, int V, int TAPS>
+__global__ __launch_bounds__(256) void conv_kernel(
+    const T* __restrict__ in, long ld, const T* __restrict__ w, const T* __restrict__ bias,
+    const int* __restrict__ pos, const int* __restrict__ slot, const int* __restrict__ seq_end,
+    T* __restrict__ state, int n_slots, T* __restrict__ out, int n_tok, int C, int taps_) {
+  const int taps = TAPS ? TAPS : taps_;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * V;
+  if (c >= C) return;
+  float wr[TAPS ? TAPS : 1][V], b[V];
+  load_vec<T, V>(bias + c, b);
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int e = 0; e < V; ++e) wr[j][e] = to_f32(w[(long)(c + e) * TAPS + j]);
+  }
+  const bool decode = seq_end == nullptr;
+  const int t1 = min(n_tok, (int)(blockIdx.x + 1) * CONV_TOKENS);
+  for (int t = blockIdx.x * CONV_TOKENS; t < t1; ++t) {
+    const int p = pos[t];
+    const int sl = state ? slot[t] : -1;
+    const bool has = sl >= 0 && sl < n_slots && taps > 1;
+    T* st = has ? state + (long)sl * (taps - 1) * C + c : nullptr;
+    float acc[V], x[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = b[e];
+#pragma unroll (TAPS ? TAPS : 1)
+    for (int j = 0; j < taps; ++j) {
+      const int back = taps - 1 - j;
+      if (p < back) continue;
+      if (back == 0 || !decode) {
+        load_vec<T, V>(in + (t - back) * ld + c, x);
+      } else {
+        if (!has) continue;
+        load_vec<T, V>(st + (long)((p - back) % (taps - 1)) * C, x);
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float wt = TAPS ? wr[TAPS ? j : 0][e] : to_f32(w[(long)(c + e) * taps + j]);
+        acc[e] = fmaf(wt, x[e], acc[e]);
+      }
+    }
+    // x is the token's own input here (the last tap)
+    if (has && (decode || t + taps - 1 >= seq_end[t]))
+      store_vec<T, V>(st + (long)(p % (taps - 1)) * C, x);
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = silu_f(acc[e]);
+    store_vec<T, V>(out + (long)t * C + c, acc);
+  }
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void token_shift_kernel(
+    const T* __restrict__ h, const T* __restrict__ mu, int n_mix, const int* __restrict__ pos,
+    const int* __restrict__ slot, const int* __restrict__ seq_end, T* __restrict__ state,
+    int n_slots, T* __restrict__ out, int W) {
+  const long t = blockIdx.x, n_tok = gridDim.x;
+  const bool decode = seq_end == nullptr;
+  const int sl = state ? slot[t] : -1;
+  T* st = sl >= 0 && sl < n_slots ? state + (long)sl * W : nullptr;
+  for (int i = threadIdx.x * V; i < W; i += blockDim.x * V) {
+    float a[V], d[V];
+    load_vec<T, V>(h + t * W + i, a);
+#pragma unroll
+    for (int e = 0; e < V; ++e) d[e] = 0.f;
+    if (pos[t] > 0) {
+      if (!decode) load_vec<T, V>(h + (t - 1) * W + i, d);
+      else if (st) load_vec<T, V>(st + i, d);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) d[e] -= a[e];
+    if (st && (decode || t + 1 == seq_end[t])) store_vec<T, V>(st + i, a);
+    for (int s = 0; s < n_mix; ++s) {
+      float m[V];
+      load_vec<T, V>(mu + (long)s * W + i, m);
+#pragma unroll
+      for (int e = 0; e < V; ++e) m[e] = fmaf(d[e], m[e], a[e]);
+      store_vec<T, V>(out + (s * n_tok + t) * W + i, m);
+    }
+  }
+}
+
+// low [T, C] -> sums of the log decays -exp(low + w0) from each block's start,
+// in place; blocks of TB tokens counted from every sequence's first.
+template <typename T>
+__global__ __launch_bounds__(256) void decay_cumsum_kernel(float* __restrict__ low,
+                                                           const T* __restrict__ w0,
+                                                           const int* __restrict__ cu, int C) {
+  const int c = blockIdx.z * 256 + threadIdx.x;
+  const int t0 = cu[blockIdx.y] + blockIdx.x * TB, t1 = min(t0 + TB, cu[blockIdx.y + 1]);
+  if (c >= C) return;
+  const float b = to_f32(w0[c]);
+  float s = 0.f;
+  for (int t = t0; t < t1; ++t) {
+    s += fmaxf(-expf(low[(long)t * C + c] + b), MIN_LOG);
+    low[(long)t * C + c] = s;
+  }
+}
+
+// ---------------------------------------------------------------------------
+// prompts: grid (column groups of 64, heads, sequences), one wave per 16 columns
+// ---------------------------------------------------------------------------
+template <typename T>
+struct ScanArgs {
+  const T *q, *k, *v;                  // row t, head h: base + t * ld + ...
+  long q_ld, k_ld, v_ld;
+  int q_hs, k_hs, per_group;           // head strides; heads per q/k group
+  const float* cum;                    // wkv: [T, H * K]
+  const T* u;                          // wkv: [H, K]
+  const T *dt, *dt_bias, *a_log, *d_skip;   // state space: dt row t at t * dt_ld
+  long dt_ld;
+  const int *cu, *slot;
+  float* state;                        // [slots, H, K, P] or null
+  int n_slots, H, K, P;
+  T* out;                              // [T, H * P]
+};
+
+template <typename T, int KT, bool WKV>
+__global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
+  constexpr int KP = KT * 16, LD = KP + 4;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float* qs = lds;                     // [TB][LD]
+  float* ks = qs + TB * LD;
+  float* cm = ks + TB * LD;            // wkv only from here
+  float* qd = cm + TB * LD;            // r times the decay since the block's start
+  float* kd = qd + TB * LD;            // k times the decay up to the block's end
+  float* es = kd + TB * LD;            // [KP] decay over the block
+  float* us = es + KP;                 // [KP]
+  float* am = us + KP;                 // [TB][TB + 4] weights within the block
+
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, lo = lane & 15, lg = lane >> 4;
+  const int h = blockIdx.y, seq = blockIdx.z;
+  const int s0 = a.cu[seq], len = a.cu[seq + 1] - s0;
+  const int col = (blockIdx.x * 4 + wid) * 16 + lo;
+  const bool live = col < a.P;
+  const int colc = live ? col : a.P - 1;
+  const T* qb = a.q + (long)(h / a.per_group) * a.q_hs;
+  const T* kb = a.k + (long)(h / a.per_group) * a.k_hs;
+  const T* vb = a.v + (long)h * a.P + colc;
+  const float* cb = WKV ? a.cum + (long)h * a.K : nullptr;
+
+  float decay_rate = 0.f, dt_bias = 0.f, d_skip = 0.f;
+  if constexpr (WKV) {
+    for (int i = tid; i < KP; i += 256) us[i] = i < a.K ? to_f32(a.u[(long)h * a.K + i]) : 0.f;
+    for (int i = tid; i < TB * (TB + 4); i += 256) am[i] = 0.f;
+  } else {
+    decay_rate = -expf(to_f32(a.a_log[h]));
+    dt_bias = to_f32(a.dt_bias[h]);
+    d_skip = to_f32(a.d_skip[h]);
+  }
+
+  scan_f32x4 S[KT];
+#pragma unroll
+  for (int i = 0; i < KT; ++i) S[i] = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+
+  // the next block's operands, loaded while this one is computed
+  float qr[KT], kr[KT], cr[WKV ? KT : 1], vr[4], dtr = 0.f;
+  auto fetch = [&](int c0) {
+    const int nt = min(TB, len - c0);
+    const long t0 = s0 + c0;
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const int e = tid + 256 * j, i = e / KP, ch = e % KP;
+      const bool in = i < nt && ch < a.K;
+      qr[j] = in ? to_f32(qb[(t0 + i) * a.q_ld + ch]) : 0.f;
+      kr[j] = in ? to_f32(kb[(t0 + i) * a.k_ld + ch]) : 0.f;
+      // past the end the sum of log decays stays where it is
+      if constexpr (WKV)
+        cr[j] = ch < a.K ? cb[(t0 + min(i, nt - 1)) * ((long)a.H * a.K) + ch] : 0.f;
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      vr[r] = lg * 4 + r < nt ? to_f32(vb[(t0 + lg * 4 + r) * a.v_ld]) : 0.f;
+    if constexpr (!WKV) dtr = lo < nt ? to_f32(a.dt[(t0 + lo) * a.dt_ld + h]) : 0.f;
+  };
+  if (len > 0) fetch(0);
+
+  for (int c0 = 0; c0 < len; c0 += TB) {
+    const int nt = min(TB, len - c0);
+    __syncthreads();                               // the last block has been read
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const int e = tid + 256 * j, at = (e / KP) * LD + e % KP;
+      qs[at] = qr[j];
+      ks[at] = kr[j];
+      if constexpr (WKV) cm[at] = cr[j];
+    }
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = vr[r];
+    float dt = 0.f;
+    if constexpr (!WKV) dt = lo < nt ? softplus_f(dtr + dt_bias) : 0.f;
+    __syncthreads();
+    if (c0 + TB < len) fetch(c0 + TB);
+
+    scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+    if constexpr (WKV) {
+#pragma unroll
+      for (int j = 0; j < KT; ++j) {
+        const int e = tid + 256 * j, i = e / KP, ch = e % KP, at = i * LD + ch;
+        qd[at] = qs[at] * (i > 0 ? expf(cm[at - LD]) : 1.f);
+        kd[at] = ks[at] * expf(cm[(TB - 1) * LD + ch] - cm[at]);
+        if (i == 0) es[ch] = expf(cm[(TB - 1) * LD + ch]);
+      }
+      // Weights of earlier tokens j for i within the block. Wave `wid` takes the
+      // pairs that part at half size hs: j in the lower, i in the upper half of
+      // a group of 2 hs, both measured against the group's middle.
+      const int hs = 8 >> wid;
+      const int mid = lo / (2 * hs) * (2 * hs) + hs - 1;
+      const bool upper = (lo & hs) != 0;
+      scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        const int ch = kt * 16 + lg * 4;
+        const float4 x = *reinterpret_cast<const float4*>((upper ? qs : ks) + lo * LD + ch);
+        const float4 cmid = *reinterpret_cast<const float4*>(cm + mid * LD + ch);
+        const float4 cown =
+            *reinterpret_cast<const float4*>(cm + (upper ? lo - 1 : lo) * LD + ch);
+        const float xs[4] = {x.x, x.y, x.z, x.w};
+        const float ds[4] = {cown.x - cmid.x, cown.y - cmid.y, cown.z - cmid.z, cown.w - cmid.w};
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float y = xs[r] * expf(upper ? ds[r] : -ds[r]);
+          g = mfma4(upper ? 0.f : y, upper ? y : 0.f, g);   // row j, column i
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = lg * 4 + r, i = lo;
+        if (upper && !(j & hs) && i / (2 * hs) == j / (2 * hs)) am[i * (TB + 4) + j] = g[r];
+      }
+      {                                            // the token itself, with the bonus
+        const int i = tid >> 4, part = tid & 15;
+        float d = 0.f;
+        for (int ch = part; ch < KP; ch += 16) d = fmaf(qs[i * LD + ch] * us[ch], ks[i * LD + ch], d);
+#pragma unroll
+        for (int off = 8; off > 0; off >>= 1) d += __shfl_xor(d, off);
+        if (part == 0) am[i * (TB + 4) + i] = d;
+      }
+      __syncthreads();
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        const float4 x = *reinterpret_cast<const float4*>(qd + lo * LD + kt * 16 + lg * 4);
+        o = mfma4(x.x, S[kt][0], o);
+        o = mfma4(x.y, S[kt][1], o);
+        o = mfma4(x.z, S[kt][2], o);
+        o = mfma4(x.w, S[kt][3], o);
+      }
+      const float4 w = *reinterpret_cast<const float4*>(am + lo * (TB + 4) + lg * 4);
+      o = mfma4(w.x, v[0], o);
+      o = mfma4(w.y, v[1], o);
+      o = mfma4(w.z, v[2], o);
+      o = mfma4(w.w, v[3], o);
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        const float4 e = *reinterpret_cast<const float4*>(es + kt * 16 + lg * 4);
+        S[kt][0] *= e.x;
+        S[kt][1] *= e.y;
+        S[kt][2] *= e.z;
+        S[kt][3] *= e.w;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[kt] = mfma4(kd[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
+      }
+    } else {
+      float cs = decay_rate * dt;                  // log decay up to and with token lo
+#pragma unroll
+      for (int off = 1; off < TB; off <<= 1) {
+        const float t = __shfl_up(cs, off, TB);
+        if (lo >= off) cs += t;
+      }
+      const float total = __shfl(cs, TB - 1, TB);
+      scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        const float4 x = *reinterpret_cast<const float4*>(qs + lo * LD + kt * 16 + lg * 4);
+        const float4 y = *reinterpret_cast<const float4*>(ks + lo * LD + kt * 16 + lg * 4);
+        g = mfma4(y.x, x.x, g);
+        o = mfma4(x.x, S[kt][0], o);
+        g = mfma4(y.y, x.y, g);
+        o = mfma4(x.y, S[kt][1], o);
+        g = mfma4(y.z, x.z, g);
+        o = mfma4(x.z, S[kt][2], o);
+        g = mfma4(y.w, x.w, g);
+        o = mfma4(x.w, S[kt][3], o);
+      }
+      float f[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float csj = __shfl(cs, lg * 4 + r, TB), dtj = __shfl(dt, lg * 4 + r, TB);
+        g[r] = lg * 4 + r <= lo ? g[r] * expf(cs - csj) * dtj : 0.f;
+        o[r] *= expf(csj);
+        f[r] = expf(total - csj) * dtj;
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
+      const float e = expf(total);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        o[r] = fmaf(d_skip, v[r], o[r]);
+        v[r] *= f[r];
+      }
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        S[kt] *= e;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[kt] = mfma4(ks[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (live && lg * 4 + r < nt)
+        a.out[(long)(s0 + c0 + lg * 4 + r) * a.H * a.P + (long)h * a.P + col] = from_f32<T>(o[r]);
+  }
+  if (a.state == nullptr || len <= 0) return;
+  const int sl = a.slot[s0];
+  if (sl < 0 || sl >= a.n_slots || !live) return;
+  float* st = a.state + ((long)sl * a.H + h) * a.K * a.P + col;
+#pragma unroll
+  for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int key = kt * 16 + lg * 4 + r;
+      if (key < a.K) st[(long)key * a.P] = S[kt][r];
+    }
+}
+
+// ---------------------------------------------------------------------------
+// one token: grid (heads, rows); a thread owns V columns and every ng-th key
+// ---------------------------------------------------------------------------
+// y[p] of the step in red[0][p]; S <- decay * S + k x^T. READ_OLD: y from the
+// state before the update (plus nothing), else after it.
+template <int V, bool READ_OLD>
+__device__ __forceinline__ void state_step(float* __restrict__ st, int K, int P,
+                                           const float* __restrict__ decay, bool per_key,
+                                           const float* __restrict__ k,
+                                           const float* __restrict__ q,
+                                           const float* __restrict__ x, float* __restrict__ red) {
+  const int units = P / V, wide = min(units, 256), ng = 256 / wide;
+  const int tid = threadIdx.x, p = tid % wide, g = tid / wide;
+  for (int u0 = 0; u0 < units; u0 += wide) {
+    const int u = u0 + p;
+    if (g >= ng || u >= units) continue;
+    float y[V], xv[V];
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      y[j] = 0.f;
+      xv[j] = x[u * V + j];
+    }
+#pragma unroll 4
+    for (int key = g; key < K; key += ng) {
+      float s[V];
+      load_vec<float, V>(st + (long)key * P + u * V, s);
+      const float dc = decay[per_key ? key : 0], kk = k[key], qq = q[key];
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        if (READ_OLD) y[j] = fmaf(qq, s[j], y[j]);
+        s[j] = fmaf(dc, s[j], kk * xv[j]);
+        if (!READ_OLD) y[j] = fmaf(qq, s[j], y[j]);
+      }
+      store_vec<float, V>(st + (long)key * P + u * V, s);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) red[g * P + u * V + j] = y[j];
+  }
+  __syncthreads();
+  for (int i = tid; i < P; i += 256) {
+    float y = 0.f;
+    for (int e = 0; e < ng; ++e) y += red[e * P + i];
+    red[i] = y;                                    // column i is this thread's alone
+  }
+  __syncthreads();
+}
+
+// Floats of red that state_step needs.
+int64_t step_scratch(int64_t P, int64_t V) {
+  const int64_t wide = std::min<int64_t>(P / V, 256);
+  return 256 / wide * P;
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void ssd_decode_kernel(
+    const T* __restrict__ xbc, int C, const T* __restrict__ dt_in, long dt_ld,
+    const T* __restrict__ dt_bias, const T* __restrict__ a_log, const T* __restrict__ d_skip,
+    const int* __restrict__ slot, float* __restrict__ state, int n_slots, int H, int G, int N,
+    int P, T* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float *k = lds, *q = k + N, *x = q + N, *dec = x + P, *red = dec + 4;
+  const int h = blockIdx.x, tid = threadIdx.x;
+  const long r = blockIdx.y;
+  const int sl = slot[r];
+  if (sl < 0 || sl >= n_slots) return;             // uniform over the block
+  const float dt = softplus_f(to_f32(dt_in[r * dt_ld + h]) + to_f32(dt_bias[h]));
+  const T* row = xbc + r * C;
+  const T* b = row + (long)H * P + (long)(h / (H / G)) * N;
+  for (int i = tid; i < N; i += 256) {
+    k[i] = dt * to_f32(b[i]);
+    q[i] = to_f32(b[(long)G * N + i]);
+  }
+  for (int i = tid; i < P; i += 256) x[i] = to_f32(row[(long)h * P + i]);
+  if (tid == 0) dec[0] = expf(-expf(to_f32(a_log[h])) * dt);
+  __syncthreads();
+  state_step<V, false>(state + ((long)sl * H + h) * N * P, N, P, dec, false, k, q, x, red);
+  const float d = to_f32(d_skip[h]);
+  for (int i = tid; i < P; i += 256)
+    out[(r * H + h) * P + i] = from_f32<T>(fmaf(d, x[i], red[i]));
+}
+
+// proj row: [r | k | v | g : H n each | low : rank]. Decay, recurrence, norm and
+// gate of one head.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void wkv_decode_kernel(
+    const T* __restrict__ proj, long ld, const T* __restrict__ w2, int rank,
+    const T* __restrict__ w0, const T* __restrict__ u, const T* __restrict__ w_norm, float eps,
+    const int* __restrict__ slot, float* __restrict__ state, int n_slots, int H, int n,
+    T* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float *q = lds, *k = q + n, *x = k + n, *dec = x + n, *low = dec + n;
+  float *sm = low + rank, *red = sm + 8;
+  const int h = blockIdx.x, tid = threadIdx.x;
+  const long r = blockIdx.y, hn = (long)H * n;
+  const int sl = slot[r];
+  if (sl < 0 || sl >= n_slots) return;             // uniform over the block
+  const T* row = proj + r * ld;
+  for (int i = tid; i < rank; i += 256) low[i] = tanhf(to_f32(row[4 * hn + i]));
+  float ruk = 0.f;
+  for (int i = tid; i < n; i += 256) {
+    q[i] = to_f32(row[h * n + i]);
+    k[i] = to_f32(row[hn + h * n + i]);
+    x[i] = to_f32(row[2 * hn + h * n + i]);
+    ruk = fmaf(q[i] * to_f32(u[h * n + i]), k[i], ruk);
+  }
+  ruk = block_reduce_sum(ruk, sm);                 // also: low, q, k, x are written
+  for (int c = tid >> 2; c < (n + 63) / 64 * 64; c += 64) {
+    float d = 0.f;
+    if (c < n)
+      for (int j = tid & 3; j < rank; j += 4)
+        d = fmaf(to_f32(w2[((long)h * n + c) * rank + j]), low[j], d);
+    d += __shfl_xor(d, 1);
+    d += __shfl_xor(d, 2);
+    if (c < n && (tid & 3) == 0)
+      dec[c] = expf(fmaxf(-expf(d + to_f32(w0[h * n + c])), MIN_LOG));
+  }
+  __syncthreads();
+  state_step<V, true>(state + ((long)sl * H + h) * n * n, n, n, dec, true, k, q, x, red);
+  float ss = 0.f;
+  for (int i = tid; i < n; i += 256) {
+    const float o = fmaf(ruk, x[i], red[i]);
+    red[i] = o;
+    ss = fmaf(o, o, ss);
+  }
+  const float inv = 1.0f / sqrtf(block_reduce_sum(ss, sm) / (float)n + eps);
+  for (int i = tid; i < n; i += 256)
+    out[r * hn + h * n + i] = from_f32<T>(red[i] * inv * to_f32(w_norm[h * n + i]) *
+                                          silu_f(to_f32(row[3 * hn + h * n + i])));
+}
+
+// groups of `size` columns, `TPG` threads each
+template <typename T, int V, int TPG>
+__global__ __launch_bounds__(256) void gated_group_norm_kernel(
+    const T* __restrict__ y, const T* __restrict__ z, long z_ld, const T* __restrict__ w,
+    T* __restrict__ out, long n_groups, int groups, int size, float eps, bool gate_first) {
+  __shared__ float red[4];
+  const long gi = (long)blockIdx.x * (256 / TPG) + threadIdx.x / TPG;
+  if (gi >= n_groups) return;                      // whole waves; whole blocks if TPG = 256
+  const long t = gi / groups;
+  const int c0 = (int)(gi % groups) * size;
+  const int lane = threadIdx.x % TPG;
+  const T* yr = y + t * groups * size + c0;
+  const T* zr = z + t * z_ld + c0;
+  float ss = 0.f;
+  for (int i = lane * V; i < size; i += TPG * V) {
+    float a[V], b[V];
+    load_vec<T, V>(yr + i, a);
+    if (gate_first) {
+      load_vec<T, V>(zr + i, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) a[j] *= silu_f(b[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) ss = fmaf(a[j], a[j], ss);
+  }
+  ss = TPG == 64 ? wave_reduce_sum(ss) : block_reduce_sum(ss, red);
+  const float inv = 1.0f / sqrtf(ss / (float)size + eps);
+  for (int i = lane * V; i < size; i += TPG * V) {
+    float a[V], b[V], g[V];
+    load_vec<T, V>(yr + i, a);
+    load_vec<T, V>(zr + i, b);
+    load_vec<T, V>(w + c0 + i, g);
+#pragma unroll
+    for (int j = 0; j < V; ++j) a[j] = a[j] * silu_f(b[j]) * inv * g[j];
+    store_vec<T, V>(out + t * groups * size + c0 + i, a);
+  }
+}
+
+// ---------------------------------------------------------------------------
+bool is_elem(const at::Tensor& x) {
+  return x.scalar_type() == at::kBFloat16 || x.scalar_type() == at::kFloat;
+}
+void check_t(const at::Tensor& t, at::ScalarType dt, int64_t n, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == dt && t.numel() == n, what,
+              ": contiguous GPU tensor of ", n, " ", dt, " elements expected, got ", t.sizes());
+}
+// rows of a wider matrix: unit column stride
+void check_rows(const at::Tensor& t, at::ScalarType dt, int64_t T, int64_t n, const char* what) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.size(0) == T && t.size(1) == n &&
+                  (n == 1 || t.stride(1) == 1) && t.stride(0) >= n && t.scalar_type() == dt,
+              what, ": [", T, ", ", n, "] rows of the activation dtype expected");
+}
+void check_i32(const at::Tensor& x, int64_t n, const char* what) {
+  TORCH_CHECK(x.is_cuda() && x.is_contiguous() && x.scalar_type() == at::kInt && x.numel() == n,
+              what, ": contiguous int32 GPU tensor of ", n, " expected");
+}
+bool aligned16(const at::Tensor& t) {
+  return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0 &&
+         (t.dim() < 2 || t.stride(0) * t.element_size() % 16 == 0);
+}
+constexpr int64_t MAX_KEYS = 256;
+
+template <typename T, bool WKV>
+void launch_scan(const ScanArgs<T>& a, int64_t n_seqs, hipStream_t stream) {
+  const dim3 grid((a.P + 63) / 64, a.H, n_seqs);
+#define LAUNCH(KT)                                                                              \
+  do {                                                                                          \
+    const size_t row = TB * (KT * 16 + 4);                                                      \
+    const size_t n = WKV ? 5 * row + 2 * KT * 16 + TB * (TB + 4) : 2 * row;                     \
+    scan_prompt_kernel<T, KT, WKV><<<grid, dim3(256), n * sizeof(float), stream>>>(a);          \
+  } while (0)
+  if (a.K <= 16) LAUNCH(1);
+  else if (a.K <= 32) LAUNCH(2);
+  else if (a.K <= 64) LAUNCH(4);
+  else if (a.K <= 128) LAUNCH(8);
+  else LAUNCH(16);
+#undef LAUNCH
+}
+
+int64_t check_bounds(const at::Tensor& cu, int64_t T, const std::optional<at::Tensor>& slot,
+                     const std::optional<at::Tensor>& state, const char* who) {
+  const int64_t n = cu.numel() - 1;
+  TORCH_CHECK(n >= 1 && n <= 65535, who, ": cu_seqlens [n + 1]");
+  check_i32(cu, n + 1, who);
+  if (state) {
+    TORCH_CHECK(slot, who, ": a state needs slots");
+    check_i32(*slot, T, who);
+  }
+  return n;
+}
+
+}  // namespace
+
+#define PTR(t) reinterpret_cast<scalar*>((t).data_ptr())
+#define OPT_I(t) ((t).has_value() ? (t)->data_ptr<int>() : nullptr)
+
+// x [T, C] (rows may be strided) -> silu(conv) [T, C]. Prompt steps give
+// seq_end; decode steps take the earlier inputs from state [slots, taps-1, C].
+at::Tensor causal_conv_silu(const at::Tensor& x, const at::Tensor& w, const at::Tensor& bias,
+                            const at::Tensor& pos, const std::optional<at::Tensor>& slot,
+                            const std::optional<at::Tensor>& seq_end,
+                            const std::optional<at::Tensor>& state) {
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && is_elem(x), "causal_conv_silu: x [T, C], w [C, n]");
+  const int64_t T = x.size(0), C = x.size(1), taps = w.size(1);
+  const auto dt = x.scalar_type();
+  check_rows(x, dt, T, C, "causal_conv_silu x");
+  check_t(w, dt, C * taps, "causal_conv_silu w");
+  check_t(bias, dt, C, "causal_conv_silu bias");
+  check_i32(pos, T, "causal_conv_silu pos");
+  TORCH_CHECK(taps >= 1 && taps <= 1024, "causal_conv_silu: 1..1024 taps");
+  int64_t n_slots = 0;
+  if (state) {
+    TORCH_CHECK(slot && state->dim() == 3, "causal_conv_silu: state [slots, taps-1, C]");
+    n_slots = state->size(0);
+    check_t(*state, dt, n_slots * (taps - 1) * C, "causal_conv_silu state");
+    check_i32(*slot, T, "causal_conv_silu slot");
+  }
+  TORCH_CHECK(seq_end || state, "causal_conv_silu: decoding needs a state");
+  if (seq_end) check_i32(*seq_end, T, "causal_conv_silu seq_end");
+  auto out = at::empty({T, C}, x.options());
+  if (T == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream();
+#define LAUNCH(TAPS)                                                                          \
+  conv_kernel<scalar, V, TAPS>                                                                \
+      <<<dim3((T + CONV_TOKENS - 1) / CONV_TOKENS, (C / V + 255) / 256), dim3(256), 0,        \
+         stream>>>(PTR(x), x.stride(0), PTR(w), PTR(bias), pos.data_ptr<int>(), OPT_I(slot),  \
+                   OPT_I(seq_end), state && taps > 1 ? PTR(*state) : nullptr, (int)n_slots,   \
+                   PTR(out), (int)T, (int)C, (int)taps)
+  AMD_DISPATCH_T_V(dt, C % 8 == 0 && aligned16(x), {
+    if (taps == 2) LAUNCH(2);
+    else if (taps == 3) LAUNCH(3);
+    else if (taps == 4) LAUNCH(4);
+    else LAUNCH(0);
+  });
+#undef LAUNCH
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// h [T, W], mu [n, W] -> [n, T, W]
+at::Tensor token_shift(const at::Tensor& h, const at::Tensor& mu, const at::Tensor& pos,
+                       const std::optional<at::Tensor>& slot,
+                       const std::optional<at::Tensor>& seq_end,
+                       const std::optional<at::Tensor>& state) {
+  TORCH_CHECK(h.dim() == 2 && mu.dim() == 2 && is_elem(h), "token_shift: h [T, W], mu [n, W]");
+  const int64_t T = h.size(0), W = h.size(1), n = mu.size(0);
+  const auto dt = h.scalar_type();
+  check_t(h, dt, T * W, "token_shift h");
+  check_t(mu, dt, n * W, "token_shift mu");
+  check_i32(pos, T, "token_shift pos");
+  int64_t n_slots = 0;
+  if (state) {
+    TORCH_CHECK(slot && state->dim() == 2, "token_shift: state [slots, W]");
+    n_slots = state->size(0);
+    check_t(*state, dt, n_slots * W, "token_shift state");
+    check_i32(*slot, T, "token_shift slot");
+  }
+  TORCH_CHECK(seq_end || state, "token_shift: decoding needs a state");
+  if (seq_end) check_i32(*seq_end, T, "token_shift seq_end");
+  auto out = at::empty({n, T, W}, h.options());
+  if (T == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream();
+  AMD_DISPATCH_T_V(dt, W % 8 == 0, {
+    token_shift_kernel<scalar, V><<<dim3(T), dim3(256), 0, stream>>>(
+        PTR(h), PTR(mu), (int)n, pos.data_ptr<int>(), OPT_I(slot), OPT_I(seq_end),
+        state ? PTR(*state) : nullptr, (int)n_slots, PTR(out), (int)W);
+  });
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// z [T, I] may be strided rows of a wider matrix.
+at::Tensor gated_group_norm(const at::Tensor& y, const at::Tensor& z, const at::Tensor& w,
+                            int64_t groups, double eps, bool gate_first) {
+  TORCH_CHECK(y.dim() == 2 && is_elem(y), "gated_group_norm: y [T, I]");
+  const int64_t T = y.size(0), I = y.size(1);
+  const auto dt = y.scalar_type();
+  check_t(y, dt, T * I, "gated_group_norm y");
+  check_rows(z, dt, T, I, "gated_group_norm z");
+  check_t(w, dt, I, "gated_group_norm w");
+  TORCH_CHECK(groups >= 1 && I % groups == 0, "gated_group_norm: groups");
+  const int64_t size = I / groups, n = T * groups;
+  auto out = at::empty_like(y);
+  if (n == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream();
+#define LAUNCH(TPG)                                                                            \
+  gated_group_norm_kernel<scalar, V, TPG>                                                      \
+      <<<dim3((n + 256 / TPG - 1) / (256 / TPG)), dim3(256), 0, stream>>>(                     \
+          PTR(y), PTR(z), z.stride(0), PTR(w), PTR(out), n, (int)groups, (int)size, (float)eps, \
+          gate_first)
+  AMD_DISPATCH_T_V(dt, size % 8 == 0 && aligned16(z), {
+    if (size <= 512) LAUNCH(64);
+    else LAUNCH(256);
+  });
+#undef LAUNCH
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// xbc [T, H*P + 2*G*N] = [x | B | C]; dt [T, H] rows before bias and softplus
+at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
+                      const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& cu,
+                      const std::optional<at::Tensor>& slot,
+                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N) {
+  TORCH_CHECK(xbc.dim() == 2 && is_elem(xbc), "ssd_prompt: xbc [T, C]");
+  const int64_t T = xbc.size(0), H = a_log.numel(), C = xbc.size(1);
+  const int64_t P = H > 0 ? (C - 2 * groups * N) / H : 0;
+  const auto dt = xbc.scalar_type();
+  TORCH_CHECK(H >= 1 && groups >= 1 && H % groups == 0 && N >= 1 && N <= MAX_KEYS && P >= 1 &&
+                  C == H * P + 2 * groups * N && H <= 65535,
+              "ssd_prompt: sizes (state up to ", MAX_KEYS, ")");
+  check_t(xbc, dt, T * C, "ssd_prompt xbc");
+  check_rows(dt_in, dt, T, H, "ssd_prompt dt");
+  check_t(dt_bias, dt, H, "ssd_prompt dt_bias");
+  check_t(a_log, dt, H, "ssd_prompt A_log");
+  check_t(d_skip, dt, H, "ssd_prompt D");
+  const int64_t n = check_bounds(cu, T, slot, state, "ssd_prompt");
+  if (state) check_t(*state, at::kFloat, state->size(0) * H * N * P, "ssd_prompt state");
+  auto out = at::empty({T, H * P}, xbc.options());
+  if (T == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  AMD_DISPATCH_T(dt, {
+    ScanArgs<scalar> a{};
+    a.v = PTR(xbc);
+    a.k = PTR(xbc) + H * P;
+    a.q = a.k + groups * N;
+    a.q_ld = a.k_ld = a.v_ld = C;
+    a.q_hs = a.k_hs = (int)N;
+    a.per_group = (int)(H / groups);
+    a.dt = PTR(dt_in);
+    a.dt_ld = dt_in.stride(0);
+    a.dt_bias = PTR(dt_bias);
+    a.a_log = PTR(a_log);
+    a.d_skip = PTR(d_skip);
+    a.cu = cu.data_ptr<int>();
+    a.slot = OPT_I(slot);
+    a.state = state ? state->data_ptr<float>() : nullptr;
+    a.n_slots = state ? (int)state->size(0) : 0;
+    a.H = (int)H;
+    a.K = (int)N;
+    a.P = (int)P;
+    a.out = PTR(out);
+    launch_scan<scalar, false>(a, n, stream);
+  });
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+at::Tensor ssd_decode(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
+                      const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& slot,
+                      at::Tensor state, int64_t groups, int64_t N) {
+  TORCH_CHECK(xbc.dim() == 2 && is_elem(xbc), "ssd_decode: xbc [R, C]");
+  const int64_t R = xbc.size(0), H = a_log.numel(), C = xbc.size(1);
+  const int64_t P = H > 0 ? (C - 2 * groups * N) / H : 0;
+  const auto dt = xbc.scalar_type();
+  TORCH_CHECK(H >= 1 && groups >= 1 && H % groups == 0 && N >= 1 && P >= 1 && P <= 2048 &&
+                  N <= 4096 && C == H * P + 2 * groups * N && R <= 65535,
+              "ssd_decode: sizes");
+  check_t(xbc, dt, R * C, "ssd_decode xbc");
+  check_rows(dt_in, dt, R, H, "ssd_decode dt");
+  check_t(dt_bias, dt, H, "ssd_decode dt_bias");
+  check_t(a_log, dt, H, "ssd_decode A_log");
+  check_t(d_skip, dt, H, "ssd_decode D");
+  check_i32(slot, R, "ssd_decode slot");
+  check_t(state, at::kFloat, state.size(0) * H * N * P, "ssd_decode state");
+  auto out = at::empty({R, H * P}, xbc.options());
+  if (R == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream();
+#define LAUNCH(V)                                                                              \
+  ssd_decode_kernel<scalar, V>                                                                 \
+      <<<dim3(H, R), dim3(256), (2 * N + P + 4 + step_scratch(P, V)) * sizeof(float),          \
+         stream>>>(PTR(xbc), (int)C, PTR(dt_in), dt_in.stride(0), PTR(dt_bias), PTR(a_log),    \
+                   PTR(d_skip), slot.data_ptr<int>(), state.data_ptr<float>(),                 \
+                   (int)state.size(0), (int)H, (int)groups, (int)N, (int)P, PTR(out))
+  AMD_DISPATCH_T(dt, {
+    if (P % 4 == 0) LAUNCH(4);
+    else LAUNCH(1);
+  });
+#undef LAUNCH
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// r, k, v [T, H*n] (rows may be strided) of the activation dtype, low [T, H*n]
+// f32 (overwritten) the decay's projection before w0
+at::Tensor wkv_prompt(const at::Tensor& r, const at::Tensor& k, const at::Tensor& v,
+                      at::Tensor low, const at::Tensor& w0, const at::Tensor& u,
+                      const at::Tensor& cu, const std::optional<at::Tensor>& slot,
+                      const std::optional<at::Tensor>& state, int64_t max_len) {
+  TORCH_CHECK(r.dim() == 2 && u.dim() == 2 && is_elem(r), "wkv_prompt: r [T, H*n], u [H, n]");
+  const int64_t T = r.size(0), H = u.size(0), n = u.size(1);
+  const auto dt = r.scalar_type();
+  TORCH_CHECK(n >= 1 && n <= MAX_KEYS && H >= 1 && H <= 65535 && max_len >= 0,
+              "wkv_prompt: heads of up to ", MAX_KEYS);
+  check_rows(r, dt, T, H * n, "wkv_prompt r");
+  check_rows(k, dt, T, H * n, "wkv_prompt k");
+  check_rows(v, dt, T, H * n, "wkv_prompt v");
+  check_t(low, at::kFloat, T * H * n, "wkv_prompt low");
+  check_t(w0, dt, H * n, "wkv_prompt w0");
+  check_t(u, dt, H * n, "wkv_prompt u");
+  const int64_t seqs = check_bounds(cu, T, slot, state, "wkv_prompt");
+  if (state) check_t(*state, at::kFloat, state->size(0) * H * n * n, "wkv_prompt state");
+  auto out = at::empty({T, H * n}, r.options());
+  if (T == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream().stream();
+  AMD_DISPATCH_T(dt, {
+    decay_cumsum_kernel<scalar>
+        <<<dim3((max_len + TB - 1) / TB, seqs, (H * n + 255) / 256), dim3(256), 0, stream>>>(
+            low.data_ptr<float>(), PTR(w0), cu.data_ptr<int>(), (int)(H * n));
+    ScanArgs<scalar> a{};
+    a.q = PTR(r);
+    a.k = PTR(k);
+    a.v = PTR(v);
+    a.q_ld = r.stride(0);
+    a.k_ld = k.stride(0);
+    a.v_ld = v.stride(0);
+    a.q_hs = a.k_hs = (int)n;
+    a.per_group = 1;
+    a.cum = low.data_ptr<float>();
+    a.u = PTR(u);
+    a.cu = cu.data_ptr<int>();
+    a.slot = OPT_I(slot);
+    a.state = state ? state->data_ptr<float>() : nullptr;
+    a.n_slots = state ? (int)state->size(0) : 0;
+    a.H = (int)H;
+    a.K = a.P = (int)n;
+    a.out = PTR(out);
+    launch_scan<scalar, true>(a, seqs, stream);
+  });
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// proj [R, 4*H*n + rank] = [r | k | v | g | low] -> gated, normed heads [R, H*n]
+at::Tensor wkv_decode(const at::Tensor& proj, const at::Tensor& w2, const at::Tensor& w0,
+                      const at::Tensor& u, const at::Tensor& w_norm, double eps,
+                      const at::Tensor& slot, at::Tensor state) {
+  TORCH_CHECK(proj.dim() == 2 && w2.dim() == 2 && u.dim() == 2 && is_elem(proj),
+              "wkv_decode: proj [R, 4*H*n + rank], w2 [H*n, rank], u [H, n]");
+  const int64_t R = proj.size(0), H = u.size(0), n = u.size(1), rank = w2.size(1);
+  const auto dt = proj.scalar_type();
+  TORCH_CHECK(H >= 1 && n >= 1 && n <= 1024 && rank >= 1 && rank <= 4096 && R <= 65535,
+              "wkv_decode: sizes");
+  check_t(proj, dt, R * (4 * H * n + rank), "wkv_decode proj");
+  check_t(w2, dt, H * n * rank, "wkv_decode w2");
+  check_t(w0, dt, H * n, "wkv_decode w0");
+  check_t(u, dt, H * n, "wkv_decode u");
+  check_t(w_norm, dt, H * n, "wkv_decode norm");
+  check_i32(slot, R, "wkv_decode slot");
+  check_t(state, at::kFloat, state.size(0) * H * n * n, "wkv_decode state");
+  auto out = at::empty({R, H * n}, proj.options());
+  if (R == 0) return out;
+  auto stream = c10::hip::getCurrentHIPStream();
+#define LAUNCH(V)                                                                               \
+  wkv_decode_kernel<scalar, V>                                                                  \
+      <<<dim3(H, R), dim3(256), (4 * n + rank + 8 + step_scratch(n, V)) * sizeof(float),        \
+         stream>>>(PTR(proj), proj.size(1), PTR(w2), (int)rank, PTR(w0), PTR(u), PTR(w_norm),   \
+                   (float)eps, slot.data_ptr<int>(), state.data_ptr<float>(),                   \
+                   (int)state.size(0), (int)H, (int)n, PTR(out))
+  AMD_DISPATCH_T(dt, {
+    if (n % 4 == 0) LAUNCH(4);
+    else LAUNCH(1);
+  });
+#undef LAUNCH
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+#undef PTR
+#undef OPT_I
+
+}  // namespace amd_ops

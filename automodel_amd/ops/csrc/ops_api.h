@@ -28,7 +28,8 @@ void adamw_step(at::Tensor param, at::Tensor grad, at::Tensor master, at::Tensor
 std::tuple<at::Tensor, at::Tensor> flash_attn_fwd(
     const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, double scale,
     bool causal, int64_t q_start,
-    const std::optional<at::Tensor>& doc_start = std::nullopt);
+    const std::optional<at::Tensor>& doc_start = std::nullopt,
+    const std::optional<at::Tensor>& sink = std::nullopt);
 std::tuple<at::Tensor, at::Tensor, at::Tensor> flash_attn_bwd(
     const at::Tensor& dout, const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
     const at::Tensor& o, const at::Tensor& lse, double scale, bool causal,
@@ -70,8 +71,9 @@ at::Tensor sgmv_fused_fwd(const at::Tensor& x, const at::Tensor& A,
 
 at::Tensor gemv_bf16(const at::Tensor& x, const at::Tensor& w,
                      const c10::optional<at::Tensor>& bias, bool relu2 = false,
-                     bool out_f32 = false);
-at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32);
+                     bool out_f32 = false, int64_t group_n = 0);
+at::Tensor gemm_skinny_bf16(const at::Tensor& x, const at::Tensor& w, bool relu2, bool out_f32,
+                            int64_t group_n = 0);
 
 std::tuple<at::Tensor, at::Tensor, at::Tensor> build_group_plan(
     const at::Tensor& counts, int64_t M, int64_t bm = 128);
@@ -114,7 +116,8 @@ std::tuple<at::Tensor, at::Tensor> latent_assemble(const at::Tensor& kv, const a
                                                    int64_t heads, int64_t dn, int64_t dv,
                                                    int64_t k_pad, int64_t v_pad, int64_t n_tok);
 at::Tensor attn_rows(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
-                     const at::Tensor& base, const at::Tensor& count, double scale, bool out_f32);
+                     const at::Tensor& base, const at::Tensor& count, double scale, bool out_f32,
+                     const std::optional<at::Tensor>& sink = std::nullopt);
 at::Tensor latent_decode_prep(const at::Tensor& qkv, const at::Tensor& w_uk,
                               const at::Tensor& w_norm, double eps, const at::Tensor& cos,
                               const at::Tensor& sin, const at::Tensor& pos, const at::Tensor& slot,
@@ -126,5 +129,54 @@ std::tuple<at::Tensor, at::Tensor> latent_decode_attn(const at::Tensor& q, const
 at::Tensor latent_decode_combine(const at::Tensor& part_o,
                                  const std::optional<at::Tensor>& part_ml, const at::Tensor& w_uv,
                                  int64_t dv);
+
+// --- inference: grouped attention, chunks, sinks (gqa_attn.hip) ---
+std::tuple<at::Tensor, at::Tensor, at::Tensor> gqa_prep(
+    const at::Tensor& proj, const at::Tensor& cos, const at::Tensor& sin, const at::Tensor& pos,
+    const std::optional<at::Tensor>& slot, const std::optional<at::Tensor>& seq_end,
+    const std::optional<at::Tensor>& cu_seqlens, const std::optional<at::Tensor>& k_cache,
+    const std::optional<at::Tensor>& v_cache, int64_t chunk, int64_t heads, int64_t kv_heads,
+    int64_t d, int64_t dv, int64_t head_pad, int64_t v_pad, int64_t rows_pad, bool decode);
+at::Tensor gqa_decode_attn(const at::Tensor& q, const at::Tensor& k_cache,
+                           const at::Tensor& v_cache, const at::Tensor& slot,
+                           const at::Tensor& pos, const std::optional<at::Tensor>& sink,
+                           int64_t chunk, int64_t dv, double scale, int64_t splits);
+
+// --- inference: hyper-connections (hyper.hip) ---
+std::tuple<at::Tensor, at::Tensor> hyper_embed(const at::Tensor& ids, const at::Tensor& table,
+                                               double scale, const at::Tensor& w_in,
+                                               const at::Tensor& w_norm, double eps);
+at::Tensor hyper_step(at::Tensor x, const at::Tensor& y, const std::optional<at::Tensor>& y2,
+                      const std::optional<at::Tensor>& w_y, const std::optional<at::Tensor>& w_y2,
+                      const at::Tensor& w_mix, const at::Tensor& w_out,
+                      const std::optional<at::Tensor>& w_in, const at::Tensor& w_norm, double eps,
+                      bool keep);
+at::Tensor clamped_glu(const at::Tensor& gu, double limit, double alpha);
+
+// --- inference: linear recurrences (linear_scan.hip) ---
+at::Tensor causal_conv_silu(const at::Tensor& x, const at::Tensor& w, const at::Tensor& bias,
+                            const at::Tensor& pos, const std::optional<at::Tensor>& slot,
+                            const std::optional<at::Tensor>& seq_end,
+                            const std::optional<at::Tensor>& state);
+at::Tensor token_shift(const at::Tensor& h, const at::Tensor& mu, const at::Tensor& pos,
+                       const std::optional<at::Tensor>& slot,
+                       const std::optional<at::Tensor>& seq_end,
+                       const std::optional<at::Tensor>& state);
+at::Tensor gated_group_norm(const at::Tensor& y, const at::Tensor& z, const at::Tensor& w,
+                            int64_t groups, double eps, bool gate_first);
+at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
+                      const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& cu,
+                      const std::optional<at::Tensor>& slot,
+                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N);
+at::Tensor ssd_decode(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
+                      const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& slot,
+                      at::Tensor state, int64_t groups, int64_t N);
+at::Tensor wkv_prompt(const at::Tensor& r, const at::Tensor& k, const at::Tensor& v,
+                      at::Tensor low, const at::Tensor& w0, const at::Tensor& u,
+                      const at::Tensor& cu, const std::optional<at::Tensor>& slot,
+                      const std::optional<at::Tensor>& state, int64_t max_len);
+at::Tensor wkv_decode(const at::Tensor& proj, const at::Tensor& w2, const at::Tensor& w0,
+                      const at::Tensor& u, const at::Tensor& w_norm, double eps,
+                      const at::Tensor& slot, at::Tensor state);
 
 }  // namespace amd_ops

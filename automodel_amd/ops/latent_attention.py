@@ -20,7 +20,6 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
-import numpy as np
 import torch
 import torch.nn.functional as F
 
@@ -29,8 +28,9 @@ from automodel_amd.ops.attention import (
     _target_dims,
     flash_attention_varlen,
 )
+from automodel_amd.ops.packed_step import PackedStep
 from automodel_amd.ops.residual_norm import rms_f32, use_hip
-from automodel_amd.ops.rope import build_rope_cache
+from automodel_amd.ops.rope import rope_half_tables  # noqa: F401  (callers import it from here)
 
 FLASH_MAX_HEAD_DIM = 256
 MFMA_MAX_RANK = 512
@@ -64,51 +64,6 @@ class LatentAttentionSpec:
     def cache_width(self) -> int:
         """Elements of a cache row: latent and rotated key, each padded to 32."""
         return pad32(self.kv_rank) + pad32(self.rot_dim)
-
-
-@dataclass
-class PackedStep:
-    """Where the packed tokens of one step belong.
-
-    ``positions``/``slots`` are int32 ``[T]``. A prompt step also carries the
-    sequence bounds; in a decode step every token attends the cached prefix of
-    its slot up to its own position.
-    """
-
-    positions: torch.Tensor
-    slots: torch.Tensor | None = None
-    prompt: bool = True
-    cu_seqlens: torch.Tensor | None = None      # int32 [n + 1], prompt steps
-    doc_start: torch.Tensor | None = None       # int32 [rows padded to 256]
-    logit_rows: torch.Tensor | None = None      # rows whose logits are wanted
-    n_seqs: int = 1
-
-    @classmethod
-    def for_prompts(cls, lengths: list[int], device, slots: list[int] | None = None,
-                    logit_rows: list[int] | None = None) -> "PackedStep":
-        lens = np.asarray(lengths, dtype=np.int32)
-        cu = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
-        total = int(cu[-1])
-        start = np.repeat(cu[:-1], lens)
-        parts = {
-            "positions": np.arange(total, dtype=np.int32) - start,
-            # padding rows form a document of their own after the last one
-            "doc_start": np.concatenate([start, np.full((-total) % 256, total, np.int32)]),
-            "cu_seqlens": cu,
-            "slots": None if slots is None else np.repeat(np.asarray(slots, np.int32), lens),
-            "logit_rows": None if logit_rows is None else np.asarray(logit_rows, np.int32),
-        }
-        parts = {k: v for k, v in parts.items() if v is not None}
-        flat = torch.from_numpy(np.concatenate(list(parts.values())).astype(np.int32)).to(device)
-        views = dict(zip(parts, flat.split([len(v) for v in parts.values()])))
-        return cls(**views, n_seqs=len(lengths))
-
-
-def rope_half_tables(rot_dim: int, n: int, base: float, device) -> tuple[torch.Tensor, torch.Tensor]:
-    """cos/sin [n, rot_dim / 2] float32; angles are formed in float64."""
-    cos, sin = build_rope_cache(rot_dim, n, base, angle_dtype=torch.float64)
-    half = rot_dim // 2
-    return (cos[:, :half].contiguous().to(device), sin[:, :half].contiguous().to(device))
 
 
 def _rotate(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.Tensor:

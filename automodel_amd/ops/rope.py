@@ -56,7 +56,7 @@ def build_rope_cache(
             if scaling.get("truncate", True):
                 low, high = _m.floor(low), _m.ceil(high)
             low, high = max(low, 0), min(high, dim - 1)
-            ramp = ((torch.arange(dim // 2, dtype=torch.float32) - low)
+            ramp = ((torch.arange(dim // 2, dtype=angle_dtype) - low)
                     / max(high - low, 1e-3)).clamp(0.0, 1.0)
             extrap_mask = 1.0 - ramp
             inv_freq = inv_freq * (1 - extrap_mask) / factor + inv_freq * extrap_mask
@@ -93,6 +93,14 @@ def build_rope_cache(
     if device is not None:
         cos, sin = cos.to(device), sin.to(device)
     return cos, sin
+
+
+def rope_half_tables(rot_dim: int, n: int, base: float, device,
+                     scaling: dict | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+    """cos/sin [n, rot_dim / 2] float32; angles are formed in float64."""
+    cos, sin = build_rope_cache(rot_dim, n, base, scaling, angle_dtype=torch.float64)
+    half = rot_dim // 2
+    return (cos[:, :half].contiguous().to(device), sin[:, :half].contiguous().to(device))
 
 
 def _rotate_half(x: torch.Tensor) -> torch.Tensor:

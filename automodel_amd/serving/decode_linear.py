@@ -72,6 +72,36 @@ def project(lin: nn.Module, x: torch.Tensor, relu2: bool = False,
     return rn.relu2(y) if relu2 else y
 
 
+def project_grouped(lin: nn.Module, xs: torch.Tensor, group: int) -> list[torch.Tensor]:
+    """Several inputs through one stacked projection: rows [i * group, (i+1) *
+    group) of the weight apply to xs[i], xs [n, T, K]; the last part may be
+    smaller. -> the n outputs [T, <= group].
+
+    Up to 64 bf16 rows on the GPU are one launch (the outputs are slices of one
+    [T, N] tensor then, see ``grouped_rows``); more take a GEMM each."""
+    y = grouped_rows(lin, xs, group)
+    if y is not None:
+        return list(y.split(group, dim=1))
+    return [F.linear(x, w) for x, w in zip(xs, lin.weight.split(group))]
+
+
+def grouped_rows(lin: nn.Module, xs: torch.Tensor, group: int) -> torch.Tensor | None:
+    """The one-launch form of ``project_grouped``, [T, N], if it applies."""
+    from automodel_amd.ops import residual_norm as rn
+
+    n, T, K = xs.shape
+    w = lin.weight
+    if not (rn.use_hip(xs) and xs.dtype == torch.bfloat16 and 1 <= T <= 64 and K % 8 == 0
+            and group % (2 if T <= 4 else 16) == 0 and -(-w.shape[0] // group) == n):
+        return None
+    from automodel_amd.ops._backend import hip_ops
+
+    x = xs.reshape(n * T, K)
+    if T <= 4:
+        return hip_ops().gemv_bf16(x, w, None, False, False, group)
+    return hip_ops().gemm_skinny_bf16(x, w, False, False, group)
+
+
 class DecodeLinear(nn.Linear):
     """nn.Linear that runs decode-shaped inputs on the in-tree GEMV."""
 

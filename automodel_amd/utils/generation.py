@@ -53,7 +53,7 @@ class DecodeSession:
 
     ``prefill`` starts sequences from whole prompts, ``decode`` moves sequences
     on by one token, ``release`` ends some. Sequences are named by the handles
-    that ``prefill`` returns. With a ragged cache (LatentKVCache) prompts may
+    that ``prefill`` returns. With a ragged cache (SlotCache) prompts may
     differ in length, tokens are packed without padding, and a batch shrinks as
     its sequences end; the dense K/V cache holds one rectangular batch that
     ends as a whole.

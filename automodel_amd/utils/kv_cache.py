@@ -12,7 +12,8 @@ varlen context in ops/attention.py): attention layers call
 full prefix k/v and records the new slots; otherwise it is a no-op.
 
 Models with another kind of cache build it in ``model.make_cache(batch,
-max_len)`` (``make_cache`` below asks for it); latent attention's is here too.
+max_len)`` (``make_cache`` below asks for it); the slot caches of latent
+attention and of mixers with states are here too.
 """
 
 from __future__ import annotations
@@ -21,9 +22,10 @@ from contextlib import contextmanager
 
 import torch
 
-from automodel_amd.ops.latent_attention import LatentAttentionSpec, PackedStep
+from automodel_amd.ops.latent_attention import LatentAttentionSpec
+from automodel_amd.ops.packed_step import PackedStep
 
-_ACTIVE: "KVCache | LatentKVCache | None" = None
+_ACTIVE: "KVCache | SlotCache | None" = None
 
 
 class KVCache:
@@ -127,25 +129,23 @@ class StaticKVCache(KVCache):
         self.pos_dev.add_(1)
 
 
-class LatentKVCache:
-    """Cache of latent-attention models: per LAYER RUN (a looped layer counts
-    once per pass) one [slots, max_len, row] tensor whose rows hold a token's
-    normed latent and its shared rotated key.
+class SlotCache:
+    """What the layer runs of a model keep of its sequences: per LAYER RUN (a
+    looped layer counts once per pass) one entry of ``layers``, whose tensors
+    have the slot as their first dimension.
 
     Sequences live in slots with their own lengths, so a batch may be ragged
     and may shrink: ``plan_prompts`` / ``plan_decode`` describe the next
     forward as packed tokens, ``free`` gives a finished sequence's slot back.
-    A slot needs no clearing before reuse: a sequence only ever reads the rows
-    it has written itself.
+    A slot needs no clearing before reuse: a sequence only ever reads what it
+    has written itself.
     """
 
     ragged = True
 
-    def __init__(self, specs: list[LatentAttentionSpec], n_slots: int, max_len: int,
-                 device, dtype):
+    def __init__(self, layers: list, n_slots: int, max_len: int, device):
         self.n_slots, self.max_len = n_slots, max_len
-        self.rows = [torch.zeros(n_slots, max_len, s.cache_width, device=device, dtype=dtype)
-                     for s in specs]
+        self.layers = layers
         self.device = torch.device(device)
         self.lens = [0] * n_slots
         self._free = list(range(n_slots - 1, -1, -1))
@@ -155,7 +155,7 @@ class LatentKVCache:
     # -- slots -----------------------------------------------------------------
     def alloc(self, n: int) -> list[int]:
         if n > len(self._free):
-            raise RuntimeError(f"latent cache: {n} slots wanted, {len(self._free)} free "
+            raise RuntimeError(f"cache: {n} slots wanted, {len(self._free)} free "
                                f"of {self.n_slots}")
         return [self._free.pop() for _ in range(n)]
 
@@ -190,15 +190,15 @@ class LatentKVCache:
     def begin_forward(self) -> None:
         self._layer = 0
 
-    def next_layer(self) -> torch.Tensor:
-        """Rows of the next layer run, consumed in execution order."""
+    def next_layer(self):
+        """The entry of the next layer run, consumed in execution order."""
         self._layer += 1
-        return self.rows[self._layer - 1]
+        return self.layers[self._layer - 1]
 
     def advance(self) -> None:
         """Account for the planned step after its forward."""
-        assert self._layer == len(self.rows), (
-            "model did not consult the latent cache in every layer run")
+        assert self._layer == len(self.layers), (
+            "model did not consult the cache in every layer run")
         for s, n in self._pending:
             self.lens[s] += n
         self._pending = []
@@ -209,8 +209,33 @@ class LatentKVCache:
         self.step.positions.add_(1)
 
 
+class LatentKVCache(SlotCache):
+    """Latent attention's: one [slots, max_len, row] tensor per layer run, whose
+    rows hold a token's normed latent and its shared rotated key."""
+
+    def __init__(self, specs: list[LatentAttentionSpec], n_slots: int, max_len: int,
+                 device, dtype):
+        super().__init__([torch.zeros(n_slots, max_len, s.cache_width, device=device, dtype=dtype)
+                          for s in specs], n_slots, max_len, device)
+
+    @property
+    def rows(self) -> list[torch.Tensor]:
+        return self.layers
+
+
+class MixerStateCache(SlotCache):
+    """One dict of tensors per layer run, made by the run's mixer
+    (``mixer.make_state(n_slots, max_len, device, dtype)``): keys and values of
+    the part of a sequence that attention can still reach, inputs of short
+    convolutions, recurrent states. Mixers of different kinds mix freely."""
+
+    def __init__(self, mixers: list, n_slots: int, max_len: int, device, dtype):
+        super().__init__([m.make_state(n_slots, max_len, device, dtype) for m in mixers],
+                         n_slots, max_len, device)
+
+
 @contextmanager
-def kv_cache_context(cache: KVCache):
+def kv_cache_context(cache: "KVCache | SlotCache"):
     global _ACTIVE
     prev = _ACTIVE
     _ACTIVE = cache
@@ -220,7 +245,7 @@ def kv_cache_context(cache: KVCache):
         _ACTIVE = prev
 
 
-def active_kv_cache() -> KVCache | LatentKVCache | None:
+def active_kv_cache() -> KVCache | SlotCache | None:
     return _ACTIVE
 
 

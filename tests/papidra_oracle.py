@@ -1,0 +1,340 @@
+"""Plain, slow implementation of the Papidra design, one function per mechanism.
+
+Independent of the product code: no import from ``automodel_amd``, no cache,
+no batching, no fused weights; recurrences run token by token. Everything is
+computed in the dtype of the weights it is given (the tests pass float64 or
+float32). Weights are a flat ``{name: tensor}`` dict under the checkpoint's own
+names; the configuration is the checkpoint's own config dict.
+
+Planted mistakes (``fault=...``) let a test show that its inputs are able to
+expose a given error; they exist only here.
+"""
+
+from __future__ import annotations
+
+import math
+
+import torch
+
+
+def unit_rms(x, eps):
+    return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+
+def rms(x, w, eps):
+    return unit_rms(x, eps) * w
+
+
+def silu(z):
+    return z / (1 + torch.exp(-z))
+
+
+def softplus(z):
+    return torch.log1p(torch.exp(-z.abs())) + z.clamp(min=0)
+
+
+# -- hyper-connections ----------------------------------------------------------
+
+def streams_in(xs, w_in):
+    return sum(w_in[s] * x for s, x in enumerate(xs))
+
+
+def streams_out(xs, y, w_mix, w_out, fault=None):
+    n = len(xs)
+    if fault == "mix_transposed":
+        w_mix = w_mix.T
+    return [sum(w_mix[s, t] * xs[s] for s in range(n)) + w_out[t] * y for t in range(n)]
+
+
+# -- rotary positions --------------------------------------------------------------
+
+def frequencies(rot):
+    n, base = rot["dims"], rot["base"]
+    f = [base ** (-2.0 * i / n) for i in range(n // 2)]
+    sc = rot.get("scaling")
+    if not sc:
+        return f, 1.0
+
+    def turns_at(t):
+        return n * math.log(sc["original"] / (2 * math.pi * t)) / (2 * math.log(base))
+
+    lo = max(math.floor(turns_at(sc["fast"])), 0)
+    hi = min(math.ceil(turns_at(sc["slow"])), n - 1)
+    out = []
+    for i, fi in enumerate(f):
+        r = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        out.append(fi / sc["factor"] * r + fi * (1 - r))
+    return out, 0.1 * math.log(sc["factor"]) + 1.0
+
+
+def rotate(x, positions, rot):
+    """x [T, ..., dim]: the first rot.dims turn, in pairs (i, i + dims / 2)."""
+    n = rot["dims"]
+    f, m = frequencies(rot)
+    out = x.clone()
+    for i in range(n // 2):
+        angle = positions.double() * f[i]
+        c, s = (torch.cos(angle) * m).to(x.dtype), (torch.sin(angle) * m).to(x.dtype)
+        while c.dim() < x.dim() - 1:
+            c, s = c.unsqueeze(-1), s.unsqueeze(-1)
+        u, v = x[..., i], x[..., i + n // 2]
+        out[..., i] = u * c - v * s
+        out[..., i + n // 2] = v * c + u * s
+    return out
+
+
+# -- chunked grouped attention with a sink -----------------------------------------
+
+def seen_by(i, size, fault=None):
+    """Keys that position i attends."""
+    start = i // size * size
+    keys = list(range(start, i + 1))
+    if fault == "edge_in":                      # one key too few at the chunk's edge
+        keys = keys[1:] if len(keys) > 1 else keys
+    elif fault == "edge_out":                   # one key too many
+        keys = ([start - 1] if start else []) + keys
+    elif isinstance(fault, tuple) and fault[0] == "lost" and i > 0:
+        keys = [j for j in keys if j != (i if fault[1] == "own" else fault[1])] or [i]
+    return keys
+
+
+def chunked_attention(h, w, p, m, fault=None):
+    """h [T, width] of ONE sequence from position 0 -> [T, width]."""
+    T = h.shape[0]
+    H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    pos = torch.arange(T)
+    q = rotate((h @ w[p + "q"].T).view(T, H, d), pos, m["rot"])
+    k = rotate((h @ w[p + "k"].T).view(T, G, d), pos, m["rot"])
+    v = (h @ w[p + "v"].T).view(T, G, dv)
+    sink = w[p + "sink"]
+    out = torch.empty(T, H, dv, dtype=h.dtype)
+    for i in range(T):
+        keys = seen_by(i, m["mask"]["size"], fault)
+        for a in range(H):
+            g = a // (H // G)
+            s = (k[keys, g] @ q[i, a]) * m["scale"]
+            top = max(s.max(), sink[a])
+            e = torch.exp(s - top)
+            total = e.sum()
+            if fault != "no_sink":
+                total = total + torch.exp(sink[a] - top)
+            out[i, a] = (e / total) @ v[keys, g]
+    return out.reshape(T, H * dv) @ w[p + "o"].T
+
+
+# -- state space, scalar decay per head --------------------------------------------
+
+def causal_conv(x, taps, bias):
+    """x [T, C], taps [C, n] (last column: the current token) -> silu'd [T, C]."""
+    T, n = x.shape[0], taps.shape[1]
+    out = bias.expand(T, -1).clone()
+    for t in range(T):
+        for j in range(n):
+            back = n - 1 - j
+            if t - back >= 0:
+                out[t] = out[t] + x[t - back] * taps[:, j]
+    return silu(out)
+
+
+def ssd_recurrence(x, B, C, dt, a_log, D):
+    """x [T,H,P], B/C [T,G,N], dt [T,H] -> y [T,H,P]"""
+    T, H, P = x.shape
+    per = H // B.shape[1]
+    y = torch.empty_like(x)
+    for a in range(H):
+        S = torch.zeros(B.shape[2], P, dtype=x.dtype)
+        decay = -torch.exp(a_log[a])
+        for t in range(T):
+            b, c = B[t, a // per], C[t, a // per]
+            S = torch.exp(decay * dt[t, a]) * S + dt[t, a] * torch.outer(b, x[t, a])
+            y[t, a] = S.T @ c + D[a] * x[t, a]
+    return y
+
+
+def gated_group_norm(y, z, w, groups, eps):
+    y = y * silu(z)
+    return unit_rms(y.view(y.shape[0], groups, -1), eps).reshape(y.shape) * w
+
+
+def state_space(h, w, p, m, eps):
+    T = h.shape[0]
+    H, P, N, G = m["heads"], m["vdim"], m["state"], m["groups"]
+    inner = H * P
+    z, xbc, dt = (h @ w[p + "in"].T).split([inner, inner + 2 * G * N, H], -1)
+    xbc = causal_conv(xbc, w[p + "conv"], w[p + "conv.b"])
+    x, B, C = xbc.split([inner, G * N, G * N], -1)
+    y = ssd_recurrence(x.reshape(T, H, P), B.reshape(T, G, N), C.reshape(T, G, N),
+                       softplus(dt + w[p + "dt_bias"]), w[p + "A_log"], w[p + "D"])
+    y = gated_group_norm(y.reshape(T, inner), z, w[p + "norm"], m["norm_groups"], eps)
+    return y @ w[p + "o"].T
+
+
+def parallel_mixer(h, w, p, m, eps, fault=None):
+    left = chunked_attention(h, w, p + "left.", m["left"], fault)
+    right = state_space(h, w, p + "right.", m["right"], eps)
+    return 0.5 * (rms(left, w[p + "left.out"], eps) + rms(right, w[p + "right.out"], eps))
+
+
+# -- time mixing with a decay per channel -------------------------------------------
+
+def token_mix(h, mu, fault=None):
+    before = torch.cat([torch.zeros_like(h[:1]), h[:-1]])
+    if fault == "no_shift":
+        before = h
+    return h + (before - h) * mu
+
+
+def wkv_recurrence(r, k, v, w, u):
+    """r/k/w [T,H,n], v [T,H,n], u [H,n] -> o [T,H,n]"""
+    T, H, n = r.shape
+    o = torch.empty_like(v)
+    for a in range(H):
+        S = torch.zeros(n, v.shape[2], dtype=r.dtype)
+        for t in range(T):
+            kv = torch.outer(k[t, a], v[t, a])
+            o[t, a] = (S + u[a][:, None] * kv).T @ r[t, a]
+            S = w[t, a][:, None] * S + kv
+    return o
+
+
+def time_mixing(h, w, p, m, eps, fault=None):
+    T, H, n = h.shape[0], m["heads"], m["dim"]
+    mix = {s: token_mix(h, w[p + "mu." + s], fault) for s in "rkvgw"}
+    r, k, v = ((mix[s] @ w[p + s].T).view(T, H, n) for s in "rkv")
+    gate = silu(mix["g"] @ w[p + "g"].T)
+    low = torch.tanh(mix["w"] @ w[p + "w1"].T) @ w[p + "w2"].T + w[p + "w0"]
+    o = wkv_recurrence(r, k, v, torch.exp(-torch.exp(low)).view(T, H, n), w[p + "u"])
+    o = unit_rms(o, eps).reshape(T, H * n) * w[p + "norm"] * gate
+    return o @ w[p + "o"].T
+
+
+# -- feed-forward, layers, model -------------------------------------------------------
+
+def clamped_glu(h, w, p, limit):
+    g = (h @ w[p + "gate"].T).clamp(max=limit)
+    u = (h @ w[p + "up"].T).clamp(-limit, limit)
+    return (g / (1 + torch.exp(-1.702 * g)) * (u + 1)) @ w[p + "down"].T
+
+
+def layer(xs, w, i, spec, eps, fault=None):
+    p = f"l{i}."
+
+    def sublayer(q, fn):
+        u = streams_in(xs, w[f"{p}hc{q}.in"])
+        y = fn(rms(u, w[f"{p}norm{q}"], eps))
+        return streams_out(xs, y, w[f"{p}hc{q}.mix"], w[f"{p}hc{q}.out"], fault)
+
+    mixer = {"parallel": parallel_mixer, "wkv": time_mixing}[spec["type"]]
+    xs = sublayer(1, lambda h: mixer(h, w, p + "mix.", spec["mixer"], eps, fault))
+    if spec.get("mlp") is not None:
+        xs = sublayer(2, lambda h: clamped_glu(h, w, p + "mlp.", spec["mlp"]["limit"]))
+    return xs
+
+
+def forward(tokens, w, cfg, trace=None, fault=None):
+    """tokens: list of ids of one sequence -> logits [T, vocab]."""
+    eps = cfg["norm"]["eps"]
+    x = w["embed"][torch.as_tensor(tokens)] * cfg["embedding"]["scale"]
+    xs = [x] * cfg["streams"]
+    for i, spec in enumerate(cfg["layers"]):
+        xs = layer(xs, w, i, spec, eps, fault)
+        if trace is not None:
+            trace.append(sum(xs))
+    return rms(sum(xs), w["final.norm"], eps) @ w["embed"].T
+
+
+def greedy(prompt, n, w, cfg):
+    ids = list(prompt)
+    for _ in range(n):
+        ids.append(int(forward(ids, w, cfg)[-1].argmax()))
+    return ids
+
+
+# -- small configurations and random weights ----------------------------------------
+
+def make_config(vocab=61, width=40, streams=3, layers=None, eps=1e-5, embed_scale=3.0):
+    return {"architecture": "Papidra", "embedding": {"scale": embed_scale}, "layers": layers,
+            "norm": {"eps": eps}, "streams": streams, "vocab": vocab, "width": width}
+
+
+def make_parallel(heads=4, kv_heads=2, dim=16, vdim=24, size=12, dims=None, base=1000.0,
+                  scaling=(3.0, 20.0, 64, 1.0), scale=None, ssm_heads=4, ssm_vdim=8, state=16,
+                  groups=2, norm_groups=2, conv=4, ff=56, limit=1.3):
+    rot = {"base": base, "dims": dims or dim}
+    if scaling:
+        rot["scaling"] = dict(zip(("factor", "fast", "original", "slow"), scaling))
+    return {"type": "parallel",
+            "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+                               "mask": {"size": size}, "rot": rot,
+                               "scale": scale or 1.0 / math.sqrt(dim)},
+                      "right": {"heads": ssm_heads, "vdim": ssm_vdim, "state": state,
+                                "groups": groups, "norm_groups": norm_groups, "conv": conv}},
+            "mlp": None if ff is None else {"kind": "dense", "ff": ff, "limit": limit}}
+
+
+def make_wkv(heads=3, dim=16, ff=None, limit=0.9):
+    return {"type": "wkv", "mixer": {"heads": heads, "dim": dim},
+            "mlp": None if ff is None else {"kind": "dense", "ff": ff, "limit": limit}}
+
+
+def make_weights(cfg, seed=0, rank=12):
+    """bfloat16 tensors under the checkpoint's names."""
+    g = torch.Generator().manual_seed(seed)
+    W, S = cfg["width"], cfg["streams"]
+
+    def rnd(*shape, mean=0.0, std=1.0):
+        return (mean + std * torch.randn(*shape, generator=g)).bfloat16()
+
+    def lin(o, i, gain=1.0):
+        return rnd(o, i, std=gain / math.sqrt(i))
+
+    def nrm(n):
+        return rnd(n, mean=1.0, std=0.3)
+
+    w = {"embed": lin(cfg["vocab"], W, 1.5), "final.norm": nrm(W)}
+    for i, spec in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", spec["mixer"]
+        subs = 1 if spec["mlp"] is None else 2
+        for q in range(1, subs + 1):
+            w[f"{p}norm{q}"] = nrm(W)
+            w[f"{p}hc{q}.in"] = rnd(S, mean=1.0 / S, std=0.3)
+            w[f"{p}hc{q}.out"] = rnd(S, mean=1.0, std=0.3)
+            w[f"{p}hc{q}.mix"] = (torch.eye(S) * 0.8 + 0.15 * torch.randn(S, S, generator=g)) \
+                .bfloat16()
+        if spec["type"] == "parallel":
+            a, b = m["left"], m["right"]
+            q = p + "mix.left."
+            w[q + "q"] = lin(a["heads"] * a["dim"], W, 1.5)
+            w[q + "k"] = lin(a["kv_heads"] * a["dim"], W, 1.5)
+            w[q + "v"] = lin(a["kv_heads"] * a["vdim"], W)
+            w[q + "sink"] = rnd(a["heads"])
+            w[q + "o"] = lin(W, a["heads"] * a["vdim"])
+            q = p + "mix.right."
+            inner, gn = b["heads"] * b["vdim"], b["groups"] * b["state"]
+            w[q + "in"] = lin(2 * inner + 2 * gn + b["heads"], W)
+            w[q + "conv"] = rnd(inner + 2 * gn, b["conv"], std=0.6)
+            w[q + "conv.b"] = rnd(inner + 2 * gn, std=0.3)
+            w[q + "dt_bias"] = rnd(b["heads"], mean=-1.0)
+            w[q + "A_log"] = rnd(b["heads"], std=0.7)
+            w[q + "D"] = rnd(b["heads"])
+            w[q + "norm"] = nrm(inner)
+            w[q + "o"] = lin(W, inner)
+            w[p + "mix.left.out"], w[p + "mix.right.out"] = nrm(W), nrm(W)
+        else:
+            n = m["heads"] * m["dim"]
+            q = p + "mix."
+            for s in "rkvgw":
+                w[q + "mu." + s] = torch.rand(W, generator=g).bfloat16()
+            for s in "rkvg":
+                w[q + s] = lin(n, W)
+            w[q + "w1"], w[q + "w2"] = lin(rank, W), lin(n, rank)
+            # decays from a few tokens to hundreds
+            w[q + "w0"] = (torch.rand(n, generator=g) * 6 - 5).bfloat16()
+            w[q + "u"] = rnd(m["heads"], m["dim"])
+            w[q + "norm"] = nrm(n)
+            w[q + "o"] = lin(W, n)
+        if spec["mlp"] is not None:
+            ff = spec["mlp"]["ff"]
+            w[p + "mlp.gate"], w[p + "mlp.up"] = lin(ff, W, 1.5), lin(ff, W, 1.5)
+            w[p + "mlp.down"] = lin(W, ff)
+    return w
