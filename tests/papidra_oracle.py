@@ -298,7 +298,7 @@ def make_weights(cfg, seed=0, rank=12):
         for q in range(1, subs + 1):
             w[f"{p}norm{q}"] = nrm(W)
             w[f"{p}hc{q}.in"] = rnd(S, mean=1.0 / S, std=0.3)
-            w[f"{p}hc{q}.out"] = rnd(S, mean=1.0, std=0.3)
+            w[f"{p}hc{q}.out"] = rnd(S, mean=0.35, std=0.15)
             w[f"{p}hc{q}.mix"] = (torch.eye(S) * 0.8 + 0.15 * torch.randn(S, S, generator=g)) \
                 .bfloat16()
         if spec["type"] == "parallel":
@@ -327,10 +327,15 @@ def make_weights(cfg, seed=0, rank=12):
                 w[q + "mu." + s] = torch.rand(W, generator=g).bfloat16()
             for s in "rkvg":
                 w[q + s] = lin(n, W)
+            # Keys that resemble the receptance, and a positive bonus: else a first
+            # token's output is a number near zero times v, normed, so that its
+            # sign alone is left and rounding decides it.
+            w[q + "mu.k"] = w[q + "mu.r"].clone()
+            w[q + "k"] = (0.8 * w[q + "r"].float() + 0.6 * w[q + "k"].float()).bfloat16()
             w[q + "w1"], w[q + "w2"] = lin(rank, W), lin(n, rank)
             # decays from a few tokens to hundreds
             w[q + "w0"] = (torch.rand(n, generator=g) * 6 - 5).bfloat16()
-            w[q + "u"] = rnd(m["heads"], m["dim"])
+            w[q + "u"] = (0.5 + rnd(m["heads"], m["dim"]).float().abs()).bfloat16()
             w[q + "norm"] = nrm(n)
             w[q + "o"] = lin(W, n)
         if spec["mlp"] is not None:
