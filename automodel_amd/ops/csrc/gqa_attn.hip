@@ -284,23 +284,46 @@ __global__ __launch_bounds__(256) void gqa_decode_attn_kernel(
   }
 }
 
-__global__ void gqa_decode_merge_kernel(const float* __restrict__ part_o,
-                                        const float* __restrict__ part_ml,
-                                        const bf16* __restrict__ sink, bf16* __restrict__ out,
-                                        int H, int splits, int vd, int dv) {
-  const int h = blockIdx.x;
+// One (row, head) per workgroup: the splits' weights once, then their sum with
+// every group of vd / 4 threads taking some of the splits.
+constexpr int MAX_SPLITS = 256;
+__global__ __launch_bounds__(256) void gqa_decode_merge_kernel(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml,
+    const bf16* __restrict__ sink, bf16* __restrict__ out, int H, int splits, int vd, int dv) {
+  __shared__ float w[MAX_SPLITS], red[8];
+  __shared__ __attribute__((aligned(16))) float sum[1024];
+  const int h = blockIdx.x, tid = threadIdx.x;
   const long rh = (long)blockIdx.y * H + h;
   const float* ml = part_ml + rh * splits * 2;
-  float m = sink ? bf2f(sink[h]) : -INFINITY;
-  for (int s = 0; s < splits; ++s) m = fmaxf(m, ml[2 * s]);
-  const float base = m > -INFINITY ? m : 0.f;
-  float l = sink ? __expf(bf2f(sink[h]) - base) : 0.f;
-  for (int s = 0; s < splits; ++s) l += ml[2 * s + 1] * __expf(ml[2 * s] - base);
+  const float sk = sink ? bf2f(sink[h]) : -INFINITY;
+  const float ms = tid < splits ? ml[2 * tid] : -INFINITY;
+  const float ls = tid < splits ? ml[2 * tid + 1] : 0.f;
+  const float wm = wave_reduce_max(ms);
+  if ((tid & 63) == 0) red[tid >> 6] = wm;
+  __syncthreads();
+  float m = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), sk);
+  m = m > -INFINITY ? m : 0.f;
+  const float e = __expf(ms - m);
+  w[tid] = e;
+  const float l = block_reduce_sum(ls * e, red + 4) + __expf(sk - m);   // w is written
   const float inv = l > 0.f ? 1.f / l : 0.f;
-  for (int c = threadIdx.x; c < dv; c += blockDim.x) {
+  const int units = vd / 4, ng = 256 / units, u = tid % units, g = tid / units;
+  if (g < ng) {
+    float4 a{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int s = g; s < splits; s += ng) {
+      const float4 o = *reinterpret_cast<const float4*>(part_o + (rh * splits + s) * vd + u * 4);
+      a.x = fmaf(o.x, w[s], a.x);
+      a.y = fmaf(o.y, w[s], a.y);
+      a.z = fmaf(o.z, w[s], a.z);
+      a.w = fmaf(o.w, w[s], a.w);
+    }
+    *reinterpret_cast<float4*>(sum + (g * units + u) * 4) = a;
+  }
+  __syncthreads();
+  for (int c = tid; c < dv; c += 256) {
     float a = 0.f;
-    for (int s = 0; s < splits; ++s)
-      a = fmaf(part_o[(rh * splits + s) * vd + c], __expf(ml[2 * s] - base), a);
+    for (int i = 0; i < ng; ++i) a += sum[i * vd + c];
     out[rh * dv + c] = f2bf(a * inv);
   }
 }
@@ -416,7 +439,7 @@ at::Tensor gqa_decode_attn(const at::Tensor& q, const at::Tensor& k_cache,
   const int64_t R = q.size(0), H = q.size(1), kd = q.size(2), G = k_cache.size(1);
   GqaCache cache = cache_of(k_cache, v_cache, at::kBFloat16, G, kd, dv);
   TORCH_CHECK(cache.blocked && cache.kd == kd && H % G == 0, "gqa_decode_attn: cache shapes");
-  TORCH_CHECK(splits >= 1 && splits <= 256 && chunk >= 1 && chunk <= INT_MAX && R <= 65535,
+  TORCH_CHECK(splits >= 1 && splits <= MAX_SPLITS && chunk >= 1 && chunk <= INT_MAX && R <= 65535,
               "gqa_decode_attn: sizes");
   check_i32(slot, R, "gqa_decode_attn slot");
   check_i32(pos, R, "gqa_decode_attn pos");
@@ -445,7 +468,7 @@ at::Tensor gqa_decode_attn(const at::Tensor& q, const at::Tensor& k_cache,
   else LAUNCH(256);
 #undef LAUNCH
   HIP_CHECK_KERNEL();
-  gqa_decode_merge_kernel<<<dim3(H, R), dim3(dv <= 64 ? 64 : 128), 0, stream>>>(
+  gqa_decode_merge_kernel<<<dim3(H, R), dim3(256), 0, stream>>>(
       part.data_ptr<float>(), ml.data_ptr<float>(),
       sink ? reinterpret_cast<const bf16*>(sink->data_ptr()) : nullptr,
       reinterpret_cast<bf16*>(out.data_ptr()), (int)H, (int)splits, cache.vd, (int)dv);

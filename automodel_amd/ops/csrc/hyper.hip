@@ -157,10 +157,9 @@ __global__ void hyper_step_kernel(float* __restrict__ x, const T* __restrict__ y
 template <typename T, int V>
 __global__ void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, long rows,
                                    int F, float limit, float alpha) {
-  const long n = rows * F;
-  const long step = (long)gridDim.x * blockDim.x * V;
-  for (long i = ((long)blockIdx.x * blockDim.x + threadIdx.x) * V; i < n; i += step) {
-    const long r = i / F, c = i % F;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= F) return;
+  for (long r = blockIdx.x; r < rows; r += gridDim.x) {
     float g[V], u[V];
     load_vec<T, V>(gu + r * 2 * F + c, g);
     load_vec<T, V>(gu + r * 2 * F + F + c, u);
@@ -170,7 +169,7 @@ __global__ void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out
       const float b = fminf(fmaxf(u[j], -limit), limit);
       g[j] = a * sigmoid_f(alpha * a) * (b + 1.f);
     }
-    store_vec<T, V>(out + i, g);
+    store_vec<T, V>(out + r * F + c, g);
   }
 }
 
@@ -272,8 +271,9 @@ at::Tensor clamped_glu(const at::Tensor& gu, double limit, double alpha) {
   if (T * F == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
   AMD_DISPATCH_T_V(gu.scalar_type(), F % 8 == 0, {
-    const int blocks = (int)std::min<int64_t>((T * F / V + 255) / 256, 8192);
-    clamped_glu_kernel<scalar, V><<<dim3(blocks), dim3(256), 0, stream>>>(
+    const int threads = std::min(256, ceil_div_i(F, V * WAVE_SIZE) * WAVE_SIZE);
+    const dim3 grid(std::min<int64_t>(T, 2048), ceil_div_i(F, V * threads));
+    clamped_glu_kernel<scalar, V><<<grid, dim3(threads), 0, stream>>>(
         PTR(gu), PTR(out), T, (int)F, (float)limit, (float)alpha);
   });
   HIP_CHECK_KERNEL();

@@ -24,6 +24,8 @@
 #include <ATen/ATen.h>
 #include <c10/hip/HIPStream.h>
 
+#include <type_traits>
+
 #include "elem.h"
 #include "ops_api.h"
 
@@ -45,58 +47,98 @@ __device__ __forceinline__ scan_f32x4 mfma4(float a, float b, scan_f32x4 c) {
 // ---------------------------------------------------------------------------
 // short convolution and token shift
 // ---------------------------------------------------------------------------
-constexpr int CONV_TOKENS = 8;         // per workgroup: the taps stay in registers
+constexpr int CONV_TOKENS = 16;        // per workgroup: taps and inputs stay in registers
 
-// TAPS 0: any number of them, weights from memory
+// Prompts. TAPS 0: any number of taps, weights and inputs from memory.
 template <typename T, int V, int TAPS>
-__global__ __launch_bounds__(256) void conv_kernel(
+__global__ __launch_bounds__(256) void conv_prompt_kernel(
     const T* __restrict__ in, long ld, const T* __restrict__ w, const T* __restrict__ bias,
     const int* __restrict__ pos, const int* __restrict__ slot, const int* __restrict__ seq_end,
     T* __restrict__ state, int n_slots, T* __restrict__ out, int n_tok, int C, int taps_) {
   const int taps = TAPS ? TAPS : taps_;
   const int c = (blockIdx.y * 256 + threadIdx.x) * V;
   if (c >= C) return;
-  float wr[TAPS ? TAPS : 1][V], b[V];
+  const int t0 = blockIdx.x * CONV_TOKENS, t1 = min(n_tok, t0 + CONV_TOKENS);
+  float b[V];
   load_vec<T, V>(bias + c, b);
+  auto finish = [&](int t, float (&acc)[V], const float (&own)[V]) {
+    if (state && taps > 1 && t + taps - 1 >= seq_end[t]) {
+      const int sl = slot[t];
+      if (sl >= 0 && sl < n_slots)
+        store_vec<T, V>(state + ((long)sl * (taps - 1) + pos[t] % (taps - 1)) * C + c, own);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = silu_f(acc[e]);
+    store_vec<T, V>(out + (long)t * C + c, acc);
+  };
   if constexpr (TAPS > 0) {
+    float wr[TAPS][V], x[TAPS][V];                 // x[j]: the input of tap j
 #pragma unroll
     for (int j = 0; j < TAPS; ++j)
 #pragma unroll
       for (int e = 0; e < V; ++e) wr[j][e] = to_f32(w[(long)(c + e) * TAPS + j]);
-  }
-  const bool decode = seq_end == nullptr;
-  const int t1 = min(n_tok, (int)(blockIdx.x + 1) * CONV_TOKENS);
-  for (int t = blockIdx.x * CONV_TOKENS; t < t1; ++t) {
-    const int p = pos[t];
-    const int sl = state ? slot[t] : -1;
-    const bool has = sl >= 0 && sl < n_slots && taps > 1;
-    T* st = has ? state + (long)sl * (taps - 1) * C + c : nullptr;
-    float acc[V], x[V];
 #pragma unroll
-    for (int e = 0; e < V; ++e) acc[e] = b[e];
-#pragma unroll (TAPS ? TAPS : 1)
-    for (int j = 0; j < taps; ++j) {
-      const int back = taps - 1 - j;
-      if (p < back) continue;
-      if (back == 0 || !decode) {
-        load_vec<T, V>(in + (t - back) * ld + c, x);
-      } else {
-        if (!has) continue;
-        load_vec<T, V>(st + (long)((p - back) % (taps - 1)) * C, x);
-      }
+    for (int j = 0; j + 1 < TAPS; ++j)             // before the tile: j = TAPS - 1 is t0
+      load_vec<T, V>(in + (long)max(t0 - (TAPS - 1 - j), 0) * ld + c, x[j]);
+#pragma unroll 4
+    for (int t = t0; t < t1; ++t) {
+      load_vec<T, V>(in + t * ld + c, x[TAPS - 1]);
+      const int p = pos[t];
+      float acc[V];
 #pragma unroll
-      for (int e = 0; e < V; ++e) {
-        const float wt = TAPS ? wr[TAPS ? j : 0][e] : to_f32(w[(long)(c + e) * taps + j]);
-        acc[e] = fmaf(wt, x[e], acc[e]);
-      }
+      for (int e = 0; e < V; ++e) acc[e] = b[e];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < V; ++e)
+          acc[e] = fmaf(wr[j][e], p >= TAPS - 1 - j ? x[j][e] : 0.f, acc[e]);
+      finish(t, acc, x[TAPS - 1]);
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < V; ++e) x[j][e] = x[j + 1][e];
     }
-    // x is the token's own input here (the last tap)
-    if (has && (decode || t + taps - 1 >= seq_end[t]))
-      store_vec<T, V>(st + (long)(p % (taps - 1)) * C, x);
+  } else {
+    for (int t = t0; t < t1; ++t) {
+      float acc[V], x[V];
 #pragma unroll
-    for (int e = 0; e < V; ++e) acc[e] = silu_f(acc[e]);
-    store_vec<T, V>(out + (long)t * C + c, acc);
+      for (int e = 0; e < V; ++e) acc[e] = b[e];
+      for (int j = max(0, taps - 1 - pos[t]); j < taps; ++j) {
+        load_vec<T, V>(in + (t - (taps - 1 - j)) * ld + c, x);
+#pragma unroll
+        for (int e = 0; e < V; ++e)
+          acc[e] = fmaf(to_f32(w[(long)(c + e) * taps + j]), x[e], acc[e]);
+      }
+      finish(t, acc, x);                           // x: the last tap's, the token's own
+    }
   }
+}
+
+// One token per sequence, the earlier inputs from the state; V columns a thread.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void conv_decode_kernel(
+    const T* __restrict__ in, long ld, const T* __restrict__ w, const T* __restrict__ bias,
+    const int* __restrict__ pos, const int* __restrict__ slot, T* __restrict__ state, int n_slots,
+    T* __restrict__ out, int C, int taps) {
+  const long t = blockIdx.x;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * V, sl = slot[t], p = pos[t];
+  if (c >= C || sl < 0 || sl >= n_slots || p < 0) return;
+  T* st = state + (long)sl * (taps - 1) * C + c;
+  float acc[V], own[V];
+  load_vec<T, V>(bias + c, acc);
+  load_vec<T, V>(in + t * ld + c, own);
+#pragma unroll 4
+  for (int j = max(0, taps - 1 - p); j < taps - 1; ++j) {
+    float x[V];
+    load_vec<T, V>(st + (long)((p - (taps - 1 - j)) % (taps - 1)) * C, x);
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = fmaf(to_f32(w[(long)(c + e) * taps + j]), x[e], acc[e]);
+  }
+#pragma unroll
+  for (int e = 0; e < V; ++e)
+    acc[e] = silu_f(fmaf(to_f32(w[(long)(c + e) * taps + taps - 1]), own[e], acc[e]));
+  if (taps > 1) store_vec<T, V>(st + (long)(p % (taps - 1)) * C, own);
+  store_vec<T, V>(out + t * C + c, acc);
 }
 
 template <typename T, int V>
@@ -108,7 +150,8 @@ __global__ __launch_bounds__(256) void token_shift_kernel(
   const bool decode = seq_end == nullptr;
   const int sl = state ? slot[t] : -1;
   T* st = sl >= 0 && sl < n_slots ? state + (long)sl * W : nullptr;
-  for (int i = threadIdx.x * V; i < W; i += blockDim.x * V) {
+  const int i = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (i < W) {
     float a[V], d[V];
     load_vec<T, V>(h + t * W + i, a);
 #pragma unroll
@@ -150,6 +193,35 @@ __global__ __launch_bounds__(256) void decay_cumsum_kernel(float* __restrict__ l
 // ---------------------------------------------------------------------------
 // prompts: grid (column groups of 64, heads, sequences), one wave per 16 columns
 // ---------------------------------------------------------------------------
+// KT consecutive floats of LDS, 16 bytes at a time where there are as many
+template <int N>
+__device__ __forceinline__ void put(float* p, const float (&x)[N]) {
+  if constexpr (N >= 4) {
+#pragma unroll
+    for (int j = 0; j < N; j += 4)
+      *reinterpret_cast<float4*>(p + j) = float4{x[j], x[j + 1], x[j + 2], x[j + 3]};
+  } else {
+#pragma unroll
+    for (int j = 0; j < N; ++j) p[j] = x[j];
+  }
+}
+template <int N>
+__device__ __forceinline__ void get(const float* p, float (&x)[N]) {
+  if constexpr (N >= 4) {
+#pragma unroll
+    for (int j = 0; j < N; j += 4) {
+      const float4 t = *reinterpret_cast<const float4*>(p + j);
+      x[j] = t.x;
+      x[j + 1] = t.y;
+      x[j + 2] = t.z;
+      x[j + 3] = t.w;
+    }
+  } else {
+#pragma unroll
+    for (int j = 0; j < N; ++j) x[j] = p[j];
+  }
+}
+
 template <typename T>
 struct ScanArgs {
   const T *q, *k, *v;                  // row t, head h: base + t * ld + ...
@@ -162,6 +234,7 @@ struct ScanArgs {
   const int *cu, *slot;
   float* state;                        // [slots, H, K, P] or null
   int n_slots, H, K, P;
+  bool vec;                            // K = KT * 16 and rows aligned to 16 bytes
   T* out;                              // [T, H * P]
 };
 
@@ -203,54 +276,86 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
 #pragma unroll
   for (int i = 0; i < KT; ++i) S[i] = scan_f32x4{0.f, 0.f, 0.f, 0.f};
 
-  // the next block's operands, loaded while this one is computed
-  float qr[KT], kr[KT], cr[WKV ? KT : 1], vr[4], dtr = 0.f;
+  // The next block's operands, loaded while this one is computed: as they are,
+  // and from clamped places without a branch, so that all loads are in flight
+  // at once. A thread has KT neighbouring channels of one token.
+  const int own_i = tid >> 4, own_ch = (tid & 15) * KT;
+  T qr[KT], kr[KT], vr[4], dtr = T{};
+  float cr[WKV ? KT : 1];
+  auto fetch_row = [&](const auto* row, auto (&to)[KT], bool vec) {
+    using E = std::remove_reference_t<decltype(to[0])>;
+    if (vec) {
+      constexpr int N = KT * sizeof(E) > 16 ? 16 / sizeof(E) : KT;   // elements per load
+#pragma unroll
+      for (int j = 0; j < KT; j += N) {
+        const ElemPack<E, N> t = *reinterpret_cast<const ElemPack<E, N>*>(row + own_ch + j);
+#pragma unroll
+        for (int e = 0; e < N; ++e) to[j + e] = t.v[e];
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < KT; ++j) to[j] = row[min(own_ch + j, a.K - 1)];
+    }
+  };
   auto fetch = [&](int c0) {
     const int nt = min(TB, len - c0);
-    const long t0 = s0 + c0;
+    const long t = s0 + c0 + min(own_i, nt - 1);
+    fetch_row(qb + t * a.q_ld, qr, a.vec);
+    fetch_row(kb + t * a.k_ld, kr, a.vec);
+    // past the end the sum of log decays stays where it is
+    if constexpr (WKV) fetch_row(cb + t * ((long)a.H * a.K), cr, a.vec);
 #pragma unroll
-    for (int j = 0; j < KT; ++j) {
-      const int e = tid + 256 * j, i = e / KP, ch = e % KP;
-      const bool in = i < nt && ch < a.K;
-      qr[j] = in ? to_f32(qb[(t0 + i) * a.q_ld + ch]) : 0.f;
-      kr[j] = in ? to_f32(kb[(t0 + i) * a.k_ld + ch]) : 0.f;
-      // past the end the sum of log decays stays where it is
-      if constexpr (WKV)
-        cr[j] = ch < a.K ? cb[(t0 + min(i, nt - 1)) * ((long)a.H * a.K) + ch] : 0.f;
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      vr[r] = lg * 4 + r < nt ? to_f32(vb[(t0 + lg * 4 + r) * a.v_ld]) : 0.f;
-    if constexpr (!WKV) dtr = lo < nt ? to_f32(a.dt[(t0 + lo) * a.dt_ld + h]) : 0.f;
+    for (int r = 0; r < 4; ++r) vr[r] = vb[(long)(s0 + c0 + min(lg * 4 + r, nt - 1)) * a.v_ld];
+    if constexpr (!WKV) dtr = a.dt[(long)(s0 + c0 + min(lo, nt - 1)) * a.dt_ld + h];
   };
   if (len > 0) fetch(0);
 
   for (int c0 = 0; c0 < len; c0 += TB) {
     const int nt = min(TB, len - c0);
     __syncthreads();                               // the last block has been read
+    {
+      float x[KT], y[KT];
 #pragma unroll
-    for (int j = 0; j < KT; ++j) {
-      const int e = tid + 256 * j, at = (e / KP) * LD + e % KP;
-      qs[at] = qr[j];
-      ks[at] = kr[j];
-      if constexpr (WKV) cm[at] = cr[j];
+      for (int j = 0; j < KT; ++j) {
+        const bool in = own_i < nt && own_ch + j < a.K;
+        x[j] = in ? to_f32(qr[j]) : 0.f;
+        y[j] = in ? to_f32(kr[j]) : 0.f;
+      }
+      put(qs + own_i * LD + own_ch, x);
+      put(ks + own_i * LD + own_ch, y);
+      if constexpr (WKV) {
+#pragma unroll
+        for (int j = 0; j < KT; ++j) x[j] = own_ch + j < a.K ? cr[j] : 0.f;
+        put(cm + own_i * LD + own_ch, x);
+      }
     }
     float v[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = vr[r];
+    for (int r = 0; r < 4; ++r) v[r] = lg * 4 + r < nt ? to_f32(vr[r]) : 0.f;
     float dt = 0.f;
-    if constexpr (!WKV) dt = lo < nt ? softplus_f(dtr + dt_bias) : 0.f;
+    if constexpr (!WKV) dt = lo < nt ? softplus_f(to_f32(dtr) + dt_bias) : 0.f;
     __syncthreads();
     if (c0 + TB < len) fetch(c0 + TB);
 
     scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f};
     if constexpr (WKV) {
+      {
+        float x[KT], y[KT], c[KT], before[KT], end[KT];
+        const int at = own_i * LD + own_ch;
+        get(qs + at, x);
+        get(ks + at, y);
+        get(cm + at, c);
+        get(cm + max(at - LD, own_ch), before);
+        get(cm + (TB - 1) * LD + own_ch, end);
 #pragma unroll
-      for (int j = 0; j < KT; ++j) {
-        const int e = tid + 256 * j, i = e / KP, ch = e % KP, at = i * LD + ch;
-        qd[at] = qs[at] * (i > 0 ? expf(cm[at - LD]) : 1.f);
-        kd[at] = ks[at] * expf(cm[(TB - 1) * LD + ch] - cm[at]);
-        if (i == 0) es[ch] = expf(cm[(TB - 1) * LD + ch]);
+        for (int j = 0; j < KT; ++j) {
+          x[j] *= own_i > 0 ? __expf(before[j]) : 1.f;
+          y[j] *= __expf(end[j] - c[j]);
+          end[j] = __expf(end[j]);
+        }
+        put(qd + at, x);
+        put(kd + at, y);
+        if (own_i == 0) put(es + own_ch, end);
       }
       // Weights of earlier tokens j for i within the block. Wave `wid` takes the
       // pairs that part at half size hs: j in the lower, i in the upper half of
@@ -270,7 +375,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         const float ds[4] = {cown.x - cmid.x, cown.y - cmid.y, cown.z - cmid.z, cown.w - cmid.w};
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float y = xs[r] * expf(upper ? ds[r] : -ds[r]);
+          const float y = xs[r] * __expf(upper ? ds[r] : -ds[r]);
           g = mfma4(upper ? 0.f : y, upper ? y : 0.f, g);   // row j, column i
         }
       }
@@ -337,13 +442,13 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const float csj = __shfl(cs, lg * 4 + r, TB), dtj = __shfl(dt, lg * 4 + r, TB);
-        g[r] = lg * 4 + r <= lo ? g[r] * expf(cs - csj) * dtj : 0.f;
-        o[r] *= expf(csj);
-        f[r] = expf(total - csj) * dtj;
+        g[r] = lg * 4 + r <= lo ? g[r] * __expf(cs - csj) * dtj : 0.f;
+        o[r] *= __expf(csj);
+        f[r] = __expf(total - csj) * dtj;
       }
 #pragma unroll
       for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
-      const float e = expf(total);
+      const float e = __expf(total);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         o[r] = fmaf(d_skip, v[r], o[r]);
@@ -377,51 +482,76 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
 // ---------------------------------------------------------------------------
 // one token: grid (heads, rows); a thread owns V columns and every ng-th key
 // ---------------------------------------------------------------------------
-// y[p] of the step in red[0][p]; S <- decay * S + k x^T. READ_OLD: y from the
-// state before the update (plus nothing), else after it.
-template <int V, bool READ_OLD>
-__device__ __forceinline__ void state_step(float* __restrict__ st, int K, int P,
-                                           const float* __restrict__ decay, bool per_key,
-                                           const float* __restrict__ k,
-                                           const float* __restrict__ q,
-                                           const float* __restrict__ x, float* __restrict__ red) {
-  const int units = P / V, wide = min(units, 256), ng = 256 / wide;
-  const int tid = threadIdx.x, p = tid % wide, g = tid / wide;
-  for (int u0 = 0; u0 < units; u0 += wide) {
-    const int u = u0 + p;
-    if (g >= ng || u >= units) continue;
-    float y[V], xv[V];
+// A thread's share of one head's state: V columns of every ng-th key. The first
+// PRE of them are loaded early, while the step's vectors are still being made.
+constexpr int PRE = 8;
+template <int V>
+struct StatePart {
+  float* st;
+  int K, P, units, wide, ng, p, g;
+  float s[PRE][V];
+  __device__ __forceinline__ StatePart(float* st_, int K_, int P_) : st(st_), K(K_), P(P_) {
+    units = P / V;
+    wide = min(units, 256);
+    ng = 256 / wide;
+    p = threadIdx.x % wide;
+    g = threadIdx.x / wide;
 #pragma unroll
-    for (int j = 0; j < V; ++j) {
-      y[j] = 0.f;
-      xv[j] = x[u * V + j];
-    }
-#pragma unroll 4
-    for (int key = g; key < K; key += ng) {
-      float s[V];
-      load_vec<float, V>(st + (long)key * P + u * V, s);
-      const float dc = decay[per_key ? key : 0], kk = k[key], qq = q[key];
+    for (int j = 0; j < PRE; ++j)
+      load_vec<float, V>(st + (long)min(g % ng + j * ng, K - 1) * P + p * V, s[j]);
+  }
+  // y[p] of the step in red[p]; S <- decay * S + k x^T. READ_OLD: y from the
+  // state before the update, else after it.
+  template <bool READ_OLD>
+  __device__ __forceinline__ void step(const float* __restrict__ decay, bool per_key,
+                                       const float* __restrict__ k, const float* __restrict__ q,
+                                       const float* __restrict__ x, float* __restrict__ red) {
+    for (int u0 = 0; u0 < units; u0 += wide) {
+      const int u = u0 + p;
+      if (g >= ng || u >= units) continue;
+      float y[V], xv[V];
 #pragma unroll
       for (int j = 0; j < V; ++j) {
-        if (READ_OLD) y[j] = fmaf(qq, s[j], y[j]);
-        s[j] = fmaf(dc, s[j], kk * xv[j]);
-        if (!READ_OLD) y[j] = fmaf(qq, s[j], y[j]);
+        y[j] = 0.f;
+        xv[j] = x[u * V + j];
       }
-      store_vec<float, V>(st + (long)key * P + u * V, s);
-    }
+      auto one = [&](int key, float (&v)[V]) {
+        const float dc = decay[per_key ? key : 0], kk = k[key], qq = q[key];
 #pragma unroll
-    for (int j = 0; j < V; ++j) red[g * P + u * V + j] = y[j];
+        for (int j = 0; j < V; ++j) {
+          if (READ_OLD) y[j] = fmaf(qq, v[j], y[j]);
+          v[j] = fmaf(dc, v[j], kk * xv[j]);
+          if (!READ_OLD) y[j] = fmaf(qq, v[j], y[j]);
+        }
+        store_vec<float, V>(st + (long)key * P + u * V, v);
+      };
+      int key = g;
+      if (u0 == 0) {
+#pragma unroll
+        for (int j = 0; j < PRE; ++j)
+          if (g + j * ng < K) one(g + j * ng, s[j]);
+        key = g + PRE * ng;
+      }
+#pragma unroll 4
+      for (; key < K; key += ng) {
+        float v[V];
+        load_vec<float, V>(st + (long)key * P + u * V, v);
+        one(key, v);
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) red[g * P + u * V + j] = y[j];
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < P; i += 256) {
+      float y = 0.f;
+      for (int e = 0; e < ng; ++e) y += red[e * P + i];
+      red[i] = y;                                  // column i is this thread's alone
+    }
+    __syncthreads();
   }
-  __syncthreads();
-  for (int i = tid; i < P; i += 256) {
-    float y = 0.f;
-    for (int e = 0; e < ng; ++e) y += red[e * P + i];
-    red[i] = y;                                    // column i is this thread's alone
-  }
-  __syncthreads();
-}
+};
 
-// Floats of red that state_step needs.
+// Floats of red that StatePart::step needs.
 int64_t step_scratch(int64_t P, int64_t V) {
   const int64_t wide = std::min<int64_t>(P / V, 256);
   return 256 / wide * P;
@@ -439,6 +569,7 @@ __global__ __launch_bounds__(256) void ssd_decode_kernel(
   const long r = blockIdx.y;
   const int sl = slot[r];
   if (sl < 0 || sl >= n_slots) return;             // uniform over the block
+  StatePart<V> part(state + ((long)sl * H + h) * N * P, N, P);
   const float dt = softplus_f(to_f32(dt_in[r * dt_ld + h]) + to_f32(dt_bias[h]));
   const T* row = xbc + r * C;
   const T* b = row + (long)H * P + (long)(h / (H / G)) * N;
@@ -449,7 +580,7 @@ __global__ __launch_bounds__(256) void ssd_decode_kernel(
   for (int i = tid; i < P; i += 256) x[i] = to_f32(row[(long)h * P + i]);
   if (tid == 0) dec[0] = expf(-expf(to_f32(a_log[h])) * dt);
   __syncthreads();
-  state_step<V, false>(state + ((long)sl * H + h) * N * P, N, P, dec, false, k, q, x, red);
+  part.template step<false>(dec, false, k, q, x, red);
   const float d = to_f32(d_skip[h]);
   for (int i = tid; i < P; i += 256)
     out[(r * H + h) * P + i] = from_f32<T>(fmaf(d, x[i], red[i]));
@@ -470,6 +601,7 @@ __global__ __launch_bounds__(256) void wkv_decode_kernel(
   const long r = blockIdx.y, hn = (long)H * n;
   const int sl = slot[r];
   if (sl < 0 || sl >= n_slots) return;             // uniform over the block
+  StatePart<V> part(state + ((long)sl * H + h) * n * n, n, n);
   const T* row = proj + r * ld;
   for (int i = tid; i < rank; i += 256) low[i] = tanhf(to_f32(row[4 * hn + i]));
   float ruk = 0.f;
@@ -482,16 +614,24 @@ __global__ __launch_bounds__(256) void wkv_decode_kernel(
   ruk = block_reduce_sum(ruk, sm);                 // also: low, q, k, x are written
   for (int c = tid >> 2; c < (n + 63) / 64 * 64; c += 64) {
     float d = 0.f;
-    if (c < n)
+    if (c < n && rank % 32 == 0) {                 // a quarter of the row per lane
+      for (int j = (tid & 3) * 8; j < rank; j += 32) {
+        float w[8];
+        load_vec<T, 8>(w2 + ((long)h * n + c) * rank + j, w);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) d = fmaf(w[e], low[j + e], d);
+      }
+    } else if (c < n) {
       for (int j = tid & 3; j < rank; j += 4)
         d = fmaf(to_f32(w2[((long)h * n + c) * rank + j]), low[j], d);
+    }
     d += __shfl_xor(d, 1);
     d += __shfl_xor(d, 2);
     if (c < n && (tid & 3) == 0)
       dec[c] = expf(fmaxf(-expf(d + to_f32(w0[h * n + c])), MIN_LOG));
   }
   __syncthreads();
-  state_step<V, true>(state + ((long)sl * H + h) * n * n, n, n, dec, true, k, q, x, red);
+  part.template step<true>(dec, true, k, q, x, red);
   float ss = 0.f;
   for (int i = tid; i < n; i += 256) {
     const float o = fmaf(ruk, x[i], red[i]);
@@ -504,41 +644,75 @@ __global__ __launch_bounds__(256) void wkv_decode_kernel(
                                           silu_f(to_f32(row[3 * hn + h * n + i])));
 }
 
-// groups of `size` columns, `TPG` threads each
-template <typename T, int V, int TPG>
+// Groups of `size` columns, TPG threads each; up to NIT vectors of a thread stay
+// in registers (NIT 0: any size, read twice).
+template <typename T, int V, int TPG, int NIT>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(
     const T* __restrict__ y, const T* __restrict__ z, long z_ld, const T* __restrict__ w,
     T* __restrict__ out, long n_groups, int groups, int size, float eps, bool gate_first) {
   __shared__ float red[4];
   const long gi = (long)blockIdx.x * (256 / TPG) + threadIdx.x / TPG;
-  if (gi >= n_groups) return;                      // whole waves; whole blocks if TPG = 256
-  const long t = gi / groups;
-  const int c0 = (int)(gi % groups) * size;
+  const bool live = gi < n_groups;                 // else it helps with the shuffles only
+  const long t = live ? gi / groups : 0;
+  const int c0 = live ? (int)(gi % groups) * size : 0;
   const int lane = threadIdx.x % TPG;
   const T* yr = y + t * groups * size + c0;
   const T* zr = z + t * z_ld + c0;
+  T* to = out + t * groups * size + c0;
   float ss = 0.f;
-  for (int i = lane * V; i < size; i += TPG * V) {
-    float a[V], b[V];
-    load_vec<T, V>(yr + i, a);
-    if (gate_first) {
-      load_vec<T, V>(zr + i, b);
-#pragma unroll
-      for (int j = 0; j < V; ++j) a[j] *= silu_f(b[j]);
-    }
-#pragma unroll
-    for (int j = 0; j < V; ++j) ss = fmaf(a[j], a[j], ss);
-  }
-  ss = TPG == 64 ? wave_reduce_sum(ss) : block_reduce_sum(ss, red);
-  const float inv = 1.0f / sqrtf(ss / (float)size + eps);
-  for (int i = lane * V; i < size; i += TPG * V) {
-    float a[V], b[V], g[V];
+  float kept[NIT ? NIT : 1][V], gate[NIT ? NIT : 1][V];
+  auto read = [&](int i, float (&a)[V], float (&b)[V]) {
     load_vec<T, V>(yr + i, a);
     load_vec<T, V>(zr + i, b);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      b[j] = silu_f(b[j]);
+      if (gate_first) a[j] *= b[j];
+    }
+  };
+  auto write = [&](int i, float inv, float (&a)[V], float (&b)[V]) {
+    float g[V];
     load_vec<T, V>(w + c0 + i, g);
 #pragma unroll
-    for (int j = 0; j < V; ++j) a[j] = a[j] * silu_f(b[j]) * inv * g[j];
-    store_vec<T, V>(out + t * groups * size + c0 + i, a);
+    for (int j = 0; j < V; ++j) a[j] = a[j] * inv * g[j] * (gate_first ? 1.f : b[j]);
+    store_vec<T, V>(to + i, a);
+  };
+  if constexpr (NIT > 0) {
+#pragma unroll
+    for (int n = 0; n < NIT; ++n) {
+      const int i = (n * TPG + lane) * V;
+      if (i < size) {
+        read(i, kept[n], gate[n]);
+#pragma unroll
+        for (int j = 0; j < V; ++j) ss = fmaf(kept[n][j], kept[n][j], ss);
+      }
+    }
+  } else {
+    for (int i = lane * V; i < size; i += TPG * V) {
+      read(i, kept[0], gate[0]);
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss = fmaf(kept[0][j], kept[0][j], ss);
+    }
+  }
+  if constexpr (TPG == 256) {
+    ss = block_reduce_sum(ss, red);
+  } else {
+#pragma unroll
+    for (int off = TPG / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off);
+  }
+  if (!live) return;
+  const float inv = 1.0f / sqrtf(ss / (float)size + eps);
+  if constexpr (NIT > 0) {
+#pragma unroll
+    for (int n = 0; n < NIT; ++n) {
+      const int i = (n * TPG + lane) * V;
+      if (i < size) write(i, inv, kept[n], gate[n]);
+    }
+  } else {
+    for (int i = lane * V; i < size; i += TPG * V) {
+      read(i, kept[0], gate[0]);
+      write(i, inv, kept[0], gate[0]);
+    }
   }
 }
 
@@ -567,7 +741,12 @@ bool aligned16(const at::Tensor& t) {
 constexpr int64_t MAX_KEYS = 256;
 
 template <typename T, bool WKV>
-void launch_scan(const ScanArgs<T>& a, int64_t n_seqs, hipStream_t stream) {
+void launch_scan(ScanArgs<T> a, int64_t n_seqs, hipStream_t stream) {
+  auto ok = [](const void* p, int64_t ld) {
+    return reinterpret_cast<uintptr_t>(p) % 16 == 0 && ld * sizeof(T) % 16 == 0;
+  };
+  a.vec = (a.K == 16 || a.K == 32 || a.K == 64 || a.K == 128 || a.K == 256) && ok(a.q, a.q_ld) &&
+          ok(a.k, a.k_ld) && ok(a.cum, 16);
   const dim3 grid((a.P + 63) / 64, a.H, n_seqs);
 #define LAUNCH(KT)                                                                              \
   do {                                                                                          \
@@ -627,17 +806,29 @@ at::Tensor causal_conv_silu(const at::Tensor& x, const at::Tensor& w, const at::
   if (T == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
 #define LAUNCH(TAPS)                                                                          \
-  conv_kernel<scalar, V, TAPS>                                                                \
-      <<<dim3((T + CONV_TOKENS - 1) / CONV_TOKENS, (C / V + 255) / 256), dim3(256), 0,        \
+  conv_prompt_kernel<scalar, V, TAPS>                                                         \
+      <<<dim3((T + CONV_TOKENS - 1) / CONV_TOKENS, ceil_div_i(C, 256 * V)), dim3(256), 0,     \
          stream>>>(PTR(x), x.stride(0), PTR(w), PTR(bias), pos.data_ptr<int>(), OPT_I(slot),  \
                    OPT_I(seq_end), state && taps > 1 ? PTR(*state) : nullptr, (int)n_slots,   \
                    PTR(out), (int)T, (int)C, (int)taps)
-  AMD_DISPATCH_T_V(dt, C % 8 == 0 && aligned16(x), {
-    if (taps == 2) LAUNCH(2);
-    else if (taps == 3) LAUNCH(3);
-    else if (taps == 4) LAUNCH(4);
-    else LAUNCH(0);
-  });
+  const bool vec = C % 8 == 0 && aligned16(x);
+  if (seq_end) {
+    AMD_DISPATCH_T_V(dt, vec, {
+      if (taps == 2) LAUNCH(2);
+      else if (taps == 3) LAUNCH(3);
+      else if (taps == 4) LAUNCH(4);
+      else LAUNCH(0);
+    });
+  } else {
+    AMD_DISPATCH_T(dt, {
+      if (vec) conv_decode_kernel<scalar, 2><<<dim3(T, ceil_div_i(C, 512)), dim3(256), 0, stream>>>(
+          PTR(x), x.stride(0), PTR(w), PTR(bias), pos.data_ptr<int>(), slot->data_ptr<int>(),
+          PTR(*state), (int)n_slots, PTR(out), (int)C, (int)taps);
+      else conv_decode_kernel<scalar, 1><<<dim3(T, ceil_div_i(C, 256)), dim3(256), 0, stream>>>(
+          PTR(x), x.stride(0), PTR(w), PTR(bias), pos.data_ptr<int>(), slot->data_ptr<int>(),
+          PTR(*state), (int)n_slots, PTR(out), (int)C, (int)taps);
+    });
+  }
 #undef LAUNCH
   HIP_CHECK_KERNEL();
   return out;
@@ -667,7 +858,9 @@ at::Tensor token_shift(const at::Tensor& h, const at::Tensor& mu, const at::Tens
   if (T == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
   AMD_DISPATCH_T_V(dt, W % 8 == 0, {
-    token_shift_kernel<scalar, V><<<dim3(T), dim3(256), 0, stream>>>(
+    const int threads = std::min(256, ceil_div_i(W, V * WAVE_SIZE) * WAVE_SIZE);
+    token_shift_kernel<scalar, V>
+        <<<dim3(T, ceil_div_i(W, V * threads)), dim3(threads), 0, stream>>>(
         PTR(h), PTR(mu), (int)n, pos.data_ptr<int>(), OPT_I(slot), OPT_I(seq_end),
         state ? PTR(*state) : nullptr, (int)n_slots, PTR(out), (int)W);
   });
@@ -689,14 +882,17 @@ at::Tensor gated_group_norm(const at::Tensor& y, const at::Tensor& z, const at::
   auto out = at::empty_like(y);
   if (n == 0) return out;
   auto stream = c10::hip::getCurrentHIPStream();
-#define LAUNCH(TPG)                                                                            \
-  gated_group_norm_kernel<scalar, V, TPG>                                                      \
+#define LAUNCH(TPG, NIT)                                                                       \
+  gated_group_norm_kernel<scalar, V, TPG, NIT>                                                 \
       <<<dim3((n + 256 / TPG - 1) / (256 / TPG)), dim3(256), 0, stream>>>(                     \
           PTR(y), PTR(z), z.stride(0), PTR(w), PTR(out), n, (int)groups, (int)size, (float)eps, \
           gate_first)
   AMD_DISPATCH_T_V(dt, size % 8 == 0 && aligned16(z), {
-    if (size <= 512) LAUNCH(64);
-    else LAUNCH(256);
+    if (size <= 8 * V) LAUNCH(8, 1);
+    else if (size <= 64 * V) LAUNCH(64, 1);
+    else if (size <= 128 * V) LAUNCH(64, 2);
+    else if (size <= 1024 * V) LAUNCH(256, 4);
+    else LAUNCH(256, 0);
   });
 #undef LAUNCH
   HIP_CHECK_KERNEL();

@@ -51,7 +51,7 @@ def parse_args():
                    help="disable fused qkv/gate_up projections")
     p.add_argument("--profile-steps", type=int, default=0,
                    help="if >0, run this many steps (no JSON contract) for rocprof")
-    p.add_argument("--serving", default=None, choices=["rezadra"],
+    p.add_argument("--serving", default=None, choices=["rezadra", "papidra"],
                    help="instead of the training step, measure this design's prefill and "
                         "decode throughput beside the closest in-tree models (one GPU)")
     p.add_argument("--serving-part", default="all",
@@ -121,7 +121,7 @@ def main():
     if args.serving:
         from benchmarks.serving_bench import main as serving_main
 
-        serving_main(args.serving_part, args.steps, args.warmup)
+        serving_main(args.serving, args.serving_part, args.steps, args.warmup)
         return
     world = int(os.environ.get("WORLD_SIZE", 1))
     rank = int(os.environ.get("RANK", 0))

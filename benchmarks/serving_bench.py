@@ -1,15 +1,19 @@
-"""Prefill and decode throughput of Rezadra beside the closest in-tree models.
+"""Prefill and decode throughput of a design beside the closest in-tree models.
 
-Same width, layer runs, attention heads and parameter count per layer, random
-weights, bf16, one GPU:
+Same width, layer runs, attention heads and parameter count per layer (Papidra:
+on average over its two kinds of layer), random weights, bf16, one GPU:
 
-* prefill against DeepSeek-V3 (latent attention, every layer dense), which
-  shares the flash kernel; both without logits for the inner positions;
-* decode against Llama (the family with a captured decode step), both as
-  hipGraph replays of the one-token step.
+* Rezadra: prefill against DeepSeek-V3 (latent attention, every layer dense),
+  which shares the flash kernel; decode against Llama;
+* Papidra: prefill against Falcon-H1 (attention and a state space side by side
+  in every layer) and Rezadra; decode against Rezadra, which has the other slot
+  cache with kernels of its own, and Llama.
 
-Run as ``python bench.py --serving rezadra`` (``--serving-part`` picks one
-part, e.g. for a profile). One JSON line per measurement.
+Prefill is without logits for the inner positions; decode is hipGraph replays of
+the one-token step.
+
+Run as ``python bench.py --serving rezadra|papidra`` (``--serving-part`` picks
+one part, e.g. for a profile). One JSON line per measurement.
 """
 
 from __future__ import annotations
@@ -21,9 +25,12 @@ import torch
 
 SIZES = {
     # width, heads, layer runs, feed-forward of the squared-ReLU MLP (two
-    # matrices) and of the gated MLP (three), equal in parameters
-    "2b-layer": dict(width=2048, heads=16, runs=12, ff=9216, gated=6144, kv_heads=4),
-    "8b-layer": dict(width=4096, heads=32, runs=12, ff=21504, gated=14336, kv_heads=8),
+    # matrices) and of the gated MLP (three), of the gated MLP beside a
+    # Papidra or a Falcon-H1 mixer; all equal in parameters
+    "2b-layer": dict(width=2048, heads=16, runs=12, ff=9216, gated=6144, kv_heads=4,
+                     papidra=3072, falcon=1792),
+    "8b-layer": dict(width=4096, heads=32, runs=12, ff=21504, gated=14336, kv_heads=8,
+                     papidra=8192, falcon=5632),
 }
 VOCAB = 32768
 MLA = dict(kv_lora_rank=512, qk_nope_head_dim=128, qk_rope_head_dim=64, v_head_dim=128)
@@ -49,6 +56,25 @@ def rezadra(size: dict):
         vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=layers, loop=loop,
         num_attention_heads=size["heads"], intermediate_size=size["ff"],
         residual_multiplier=0.5, **MLA))
+
+
+def papidra(size: dict):
+    return _build("Papidra", dict(
+        vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=size["runs"], streams=2,
+        num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=128,
+        intermediate_size=size["papidra"], chunk_size=8192))
+
+
+def falcon(size: dict):
+    return _build("FalconH1ForCausalLM", dict(
+        vocab_size=VOCAB, hidden_size=size["width"], num_hidden_layers=size["runs"],
+        num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], head_dim=128,
+        intermediate_size=size["falcon"], mamba_n_heads=size["width"] // 32, mamba_d_head=64,
+        mamba_d_state=128, mamba_n_groups=8, mamba_chunk_size=128,
+        max_position_embeddings=8192))
+
+
+SLOT_MODELS = {"rezadra": rezadra, "papidra": papidra}
 
 
 def deepseek(size: dict):
@@ -87,14 +113,14 @@ def prefill(name: str, which: str, batch: int, seq: int, steps: int, warmup: int
     size = SIZES[name]
     torch.manual_seed(0)
     ids = torch.randint(0, VOCAB, (batch, seq))
-    if which == "rezadra":
-        session = DecodeSession(rezadra(size), batch, seq)
+    if which in SLOT_MODELS:
+        session = DecodeSession(SLOT_MODELS[which](size), batch, seq)
         prompts = ids.tolist()
 
         def run():
             session.release(session.prefill(prompts)[0])
     else:
-        model, dev_ids = deepseek(size), ids.cuda()
+        model, dev_ids = PEERS[which](size), ids.cuda()
 
         def run():
             hidden = model(dev_ids, return_hidden=True)
@@ -111,7 +137,7 @@ def decode(name: str, which: str, batch: int, context: int, steps: int, warmup: 
 
     size = SIZES[name]
     torch.manual_seed(0)
-    model = rezadra(size) if which == "rezadra" else llama(size, batch)
+    model = SLOT_MODELS[which](size) if which in SLOT_MODELS else llama(size, batch)
     session = DecodeSession(model, batch, context + steps + warmup + 8, static=True)
     handles, logits = session.prefill(torch.randint(0, VOCAB, (batch, context)).tolist())
     with kv_cache_context(session.cache):
@@ -136,16 +162,23 @@ DECODE = [("2b-layer", 1, 2048), ("2b-layer", 16, 2048), ("8b-layer", 1, 4096),
           ("8b-layer", 4, 4096), ("8b-layer", 32, 4096)]
 
 
-def main(part: str = "all", steps: int = 10, warmup: int = 3) -> None:
+PEERS = {"deepseek-v3-dense": deepseek, "falcon-h1": falcon}
+BESIDE = {                          # design -> models of (prefill, decode)
+    "rezadra": (("rezadra", "deepseek-v3-dense"), ("rezadra", "llama")),
+    "papidra": (("papidra", "falcon-h1", "rezadra"), ("papidra", "rezadra", "llama")),
+}
+
+
+def main(design: str, part: str = "all", steps: int = 10, warmup: int = 3) -> None:
     assert torch.cuda.is_available(), "the serving bench needs a GPU"
-    for kind, fn, cases, peer in (("prefill", prefill, PREFILL, "deepseek-v3-dense"),
-                                  ("decode", decode, DECODE, "llama")):
+    for kind, fn, cases, models in (("prefill", prefill, PREFILL, BESIDE[design][0]),
+                                    ("decode", decode, DECODE, BESIDE[design][1])):
         if part not in ("all", kind) and not part.startswith(kind + ":"):
             continue
         only = part.split(":")[1:]                    # e.g. decode:rezadra:8b-layer:1
         n = steps if kind == "prefill" else 10 * steps
         for name, batch, length in cases:
-            for which in ("rezadra", peer):
+            for which in models:
                 tag = [which, name, str(batch)]
                 if tag[:len(only)] == only:
                     fn(name, which, batch, length, n, warmup)
