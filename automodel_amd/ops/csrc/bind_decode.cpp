@@ -95,7 +95,8 @@ TORCH_LIBRARY_FRAGMENT(amd_ops, m) {
   m.impl("gated_group_norm", &amd_ops::gated_group_norm);
   m.def(
       "ssd_prompt(Tensor xbc, Tensor dt, Tensor dt_bias, Tensor a_log, Tensor d_skip, "
-      "Tensor cu_seqlens, Tensor? slot, Tensor(a!)? state, int groups, int n) -> Tensor");
+      "Tensor cu_seqlens, Tensor? slot, Tensor(a!)? state, int groups, int n, int max_len) "
+      "-> Tensor");
   m.impl("ssd_prompt", &amd_ops::ssd_prompt);
   m.def(
       "ssd_decode(Tensor xbc, Tensor dt, Tensor dt_bias, Tensor a_log, Tensor d_skip, "

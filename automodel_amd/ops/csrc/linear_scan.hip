@@ -191,7 +191,11 @@ __global__ __launch_bounds__(256) void decay_cumsum_kernel(float* __restrict__ l
 }
 
 // ---------------------------------------------------------------------------
-// prompts: grid (column groups of 64, heads, sequences), one wave per 16 columns
+// prompts: grid (column groups of 64, heads, sequences x segments), one wave per
+// 16 columns. Few heads and long sequences leave most of the chip idle, so a
+// sequence may be cut into segments: a first pass (STATES) makes every segment's
+// state from zero and its decay, scan_link_kernel turns these into the states
+// that the segments begin with, and the main pass runs all segments at once.
 // ---------------------------------------------------------------------------
 // KT consecutive floats of LDS, 16 bytes at a time where there are as many
 template <int N>
@@ -233,12 +237,15 @@ struct ScanArgs {
   long dt_ld;
   const int *cu, *slot;
   float* state;                        // [slots, H, K, P] or null
+  int segs, seg_len;                   // segments per sequence, in whole blocks
+  float* seg_state;                    // [seqs, segs, H, K, P] if segs > 1
+  float* seg_decay;                    // [seqs, segs, H, K] (wkv) or [seqs, segs, H]
   int n_slots, H, K, P;
   bool vec;                            // K = KT * 16 and rows aligned to 16 bytes
   T* out;                              // [T, H * P]
 };
 
-template <typename T, int KT, bool WKV>
+template <typename T, int KT, bool WKV, bool STATES>
 __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
   constexpr int KP = KT * 16, LD = KP + 4;
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -252,8 +259,12 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
   float* am = us + KP;                 // [TB][TB + 4] weights within the block
 
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, lo = lane & 15, lg = lane >> 4;
-  const int h = blockIdx.y, seq = blockIdx.z;
-  const int s0 = a.cu[seq], len = a.cu[seq + 1] - s0;
+  const int h = blockIdx.y, seq = blockIdx.z / a.segs, seg = blockIdx.z % a.segs;
+  const int left = a.cu[seq + 1] - a.cu[seq] - seg * a.seg_len;
+  const int s0 = a.cu[seq] + seg * a.seg_len, len = min(left, a.seg_len);
+  const bool last = left <= a.seg_len;
+  if (len <= 0 || (STATES && last)) return;        // uniform over the block
+  const long sh = (long)blockIdx.z * a.H + h;
   const int col = (blockIdx.x * 4 + wid) * 16 + lo;
   const bool live = col < a.P;
   const int colc = live ? col : a.P - 1;
@@ -275,6 +286,18 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
   scan_f32x4 S[KT];
 #pragma unroll
   for (int i = 0; i < KT; ++i) S[i] = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+  if (!STATES && seg > 0) {
+    const float* st = a.seg_state + sh * a.K * a.P + colc;
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = kt * 16 + lg * 4 + r;
+        S[kt][r] = st[(long)min(key, a.K - 1) * a.P];
+        if (key >= a.K) S[kt][r] = 0.f;
+      }
+  }
+  float log_decay = 0.f;                           // STATES: over the segment
 
   // The next block's operands, loaded while this one is computed: as they are,
   // and from clamped places without a branch, so that all loads are in flight
@@ -300,7 +323,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
   auto fetch = [&](int c0) {
     const int nt = min(TB, len - c0);
     const long t = s0 + c0 + min(own_i, nt - 1);
-    fetch_row(qb + t * a.q_ld, qr, a.vec);
+    if constexpr (!STATES) fetch_row(qb + t * a.q_ld, qr, a.vec);
     fetch_row(kb + t * a.k_ld, kr, a.vec);
     // past the end the sum of log decays stays where it is
     if constexpr (WKV) fetch_row(cb + t * ((long)a.H * a.K), cr, a.vec);
@@ -308,7 +331,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
     for (int r = 0; r < 4; ++r) vr[r] = vb[(long)(s0 + c0 + min(lg * 4 + r, nt - 1)) * a.v_ld];
     if constexpr (!WKV) dtr = a.dt[(long)(s0 + c0 + min(lo, nt - 1)) * a.dt_ld + h];
   };
-  if (len > 0) fetch(0);
+  fetch(0);
 
   for (int c0 = 0; c0 < len; c0 += TB) {
     const int nt = min(TB, len - c0);
@@ -318,10 +341,10 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
 #pragma unroll
       for (int j = 0; j < KT; ++j) {
         const bool in = own_i < nt && own_ch + j < a.K;
-        x[j] = in ? to_f32(qr[j]) : 0.f;
+        x[j] = !STATES && in ? to_f32(qr[j]) : 0.f;
         y[j] = in ? to_f32(kr[j]) : 0.f;
       }
-      put(qs + own_i * LD + own_ch, x);
+      if constexpr (!STATES) put(qs + own_i * LD + own_ch, x);
       put(ks + own_i * LD + own_ch, y);
       if constexpr (WKV) {
 #pragma unroll
@@ -342,21 +365,25 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
       {
         float x[KT], y[KT], c[KT], before[KT], end[KT];
         const int at = own_i * LD + own_ch;
-        get(qs + at, x);
         get(ks + at, y);
         get(cm + at, c);
-        get(cm + max(at - LD, own_ch), before);
         get(cm + (TB - 1) * LD + own_ch, end);
+        if constexpr (!STATES) {
+          get(qs + at, x);
+          get(cm + max(at - LD, own_ch), before);
+        }
 #pragma unroll
         for (int j = 0; j < KT; ++j) {
-          x[j] *= own_i > 0 ? __expf(before[j]) : 1.f;
+          if constexpr (!STATES) x[j] *= own_i > 0 ? __expf(before[j]) : 1.f;
           y[j] *= __expf(end[j] - c[j]);
           end[j] = __expf(end[j]);
         }
-        put(qd + at, x);
+        if constexpr (!STATES) put(qd + at, x);
         put(kd + at, y);
         if (own_i == 0) put(es + own_ch, end);
+        if (STATES && tid < KP) log_decay += cm[(TB - 1) * LD + tid];
       }
+      if constexpr (!STATES) {
       // Weights of earlier tokens j for i within the block. Wave `wid` takes the
       // pairs that part at half size hs: j in the lower, i in the upper half of
       // a group of 2 hs, both measured against the group's middle.
@@ -392,7 +419,9 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         for (int off = 8; off > 0; off >>= 1) d += __shfl_xor(d, off);
         if (part == 0) am[i * (TB + 4) + i] = d;
       }
+      }
       __syncthreads();
+      if constexpr (!STATES) {
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
         const float4 x = *reinterpret_cast<const float4*>(qd + lo * LD + kt * 16 + lg * 4);
@@ -406,6 +435,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
       o = mfma4(w.y, v[1], o);
       o = mfma4(w.z, v[2], o);
       o = mfma4(w.w, v[3], o);
+      }
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
         const float4 e = *reinterpret_cast<const float4*>(es + kt * 16 + lg * 4);
@@ -413,9 +443,12 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         S[kt][1] *= e.y;
         S[kt][2] *= e.z;
         S[kt][3] *= e.w;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) S[kt] = mfma4(kd[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
       }
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+          S[kt] = mfma4(kd[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
     } else {
       float cs = decay_rate * dt;                  // log decay up to and with token lo
 #pragma unroll
@@ -424,7 +457,9 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         if (lo >= off) cs += t;
       }
       const float total = __shfl(cs, TB - 1, TB);
+      log_decay += total;
       scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+      if constexpr (!STATES) {
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
         const float4 x = *reinterpret_cast<const float4*>(qs + lo * LD + kt * 16 + lg * 4);
@@ -438,6 +473,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         g = mfma4(y.w, x.w, g);
         o = mfma4(x.w, S[kt][3], o);
       }
+      }
       float f[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
@@ -446,8 +482,10 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         o[r] *= __expf(csj);
         f[r] = __expf(total - csj) * dtj;
       }
+      if constexpr (!STATES) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
+        for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
+      }
       const float e = __expf(total);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
@@ -455,21 +493,33 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         v[r] *= f[r];
       }
 #pragma unroll
-      for (int kt = 0; kt < KT; ++kt) {
-        S[kt] *= e;
+      for (int kt = 0; kt < KT; ++kt) S[kt] *= e;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[kt] = mfma4(ks[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
-      }
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+          S[kt] = mfma4(ks[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
     }
+    if constexpr (STATES) continue;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       if (live && lg * 4 + r < nt)
         a.out[(long)(s0 + c0 + lg * 4 + r) * a.H * a.P + (long)h * a.P + col] = from_f32<T>(o[r]);
   }
-  if (a.state == nullptr || len <= 0) return;
-  const int sl = a.slot[s0];
-  if (sl < 0 || sl >= a.n_slots || !live) return;
-  float* st = a.state + ((long)sl * a.H + h) * a.K * a.P + col;
+  float* st;
+  if constexpr (STATES) {
+    if (blockIdx.x == 0) {
+      if (WKV && tid < a.K) a.seg_decay[sh * a.K + tid] = __expf(log_decay);
+      if (!WKV && tid == 0) a.seg_decay[sh] = __expf(log_decay);
+    }
+    st = a.seg_state + sh * a.K * a.P + col;
+  } else {
+    if (a.state == nullptr || !last) return;
+    const int sl = a.slot[s0];
+    if (sl < 0 || sl >= a.n_slots) return;
+    st = a.state + ((long)sl * a.H + h) * a.K * a.P + col;
+  }
+  if (!live) return;
 #pragma unroll
   for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
@@ -477,6 +527,27 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
       const int key = kt * 16 + lg * 4 + r;
       if (key < a.K) st[(long)key * a.P] = S[kt][r];
     }
+}
+
+// Segments' own states -> the states they begin with, in place. A thread has one
+// element of one head; key_decay: a decay per key, else one per head.
+__global__ __launch_bounds__(256) void scan_link_kernel(float* __restrict__ seg_state,
+                                                        const float* __restrict__ seg_decay,
+                                                        const int* __restrict__ cu, int segs,
+                                                        int seg_len, int H, int K, int P,
+                                                        bool key_decay) {
+  const long n = (long)H * K * P, i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  const int seq = blockIdx.y, len = cu[seq + 1] - cu[seq];
+  const long at = key_decay ? i / P : i / ((long)K * P), decays = key_decay ? (long)H * K : H;
+  float s = 0.f;
+  for (int g = 0; g * seg_len < len; ++g) {
+    float* p = seg_state + ((long)seq * segs + g) * n + i;
+    const bool last = (g + 1) * seg_len >= len;    // has no state of its own
+    const float own = last ? 0.f : *p;
+    *p = s;
+    if (!last) s = fmaf(seg_decay[((long)seq * segs + g) * decays + at], s, own);
+  }
 }
 
 // ---------------------------------------------------------------------------
@@ -739,20 +810,41 @@ bool aligned16(const at::Tensor& t) {
          (t.dim() < 2 || t.stride(0) * t.element_size() % 16 == 0);
 }
 constexpr int64_t MAX_KEYS = 256;
+constexpr int64_t TARGET_GROUPS = 512;  // workgroups of a prompt pass: two per CU
 
 template <typename T, bool WKV>
-void launch_scan(ScanArgs<T> a, int64_t n_seqs, hipStream_t stream) {
+void launch_scan(ScanArgs<T> a, int64_t n_seqs, int64_t max_len, const at::TensorOptions& f32,
+                 hipStream_t stream) {
   auto ok = [](const void* p, int64_t ld) {
     return reinterpret_cast<uintptr_t>(p) % 16 == 0 && ld * sizeof(T) % 16 == 0;
   };
   a.vec = (a.K == 16 || a.K == 32 || a.K == 64 || a.K == 128 || a.K == 256) && ok(a.q, a.q_ld) &&
           ok(a.k, a.k_ld) && ok(a.cum, 16);
-  const dim3 grid((a.P + 63) / 64, a.H, n_seqs);
+  // segments of at least 8 blocks, as many as fill the chip
+  const int64_t groups = (a.P + 63) / 64 * a.H * n_seqs, blocks = (max_len + TB - 1) / TB;
+  const int64_t want = std::min<int64_t>((TARGET_GROUPS + groups - 1) / groups, blocks / 8);
+  a.seg_len = (int)((blocks + std::max<int64_t>(want, 1) - 1) / std::max<int64_t>(want, 1)) * TB;
+  a.segs = (int)((max_len + a.seg_len - 1) / a.seg_len);
+  TORCH_CHECK(n_seqs * a.segs <= 65535, "recurrence: too many sequences");
+  at::Tensor seg_state, seg_decay;
+  if (a.segs > 1) {
+    seg_state = at::empty({n_seqs * a.segs, a.H, a.K, a.P}, f32);
+    seg_decay = at::empty({n_seqs * a.segs, a.H, WKV ? a.K : 1}, f32);
+    a.seg_state = seg_state.data_ptr<float>();
+    a.seg_decay = seg_decay.data_ptr<float>();
+  }
+  const dim3 grid((a.P + 63) / 64, a.H, n_seqs * a.segs);
 #define LAUNCH(KT)                                                                              \
   do {                                                                                          \
     const size_t row = TB * (KT * 16 + 4);                                                      \
     const size_t n = WKV ? 5 * row + 2 * KT * 16 + TB * (TB + 4) : 2 * row;                     \
-    scan_prompt_kernel<T, KT, WKV><<<grid, dim3(256), n * sizeof(float), stream>>>(a);          \
+    if (a.segs > 1) {                                                                           \
+      scan_prompt_kernel<T, KT, WKV, true><<<grid, dim3(256), n * sizeof(float), stream>>>(a);  \
+      scan_link_kernel<<<dim3(ceil_div_i((long)a.H * a.K * a.P, 256), n_seqs), dim3(256), 0,    \
+                         stream>>>(a.seg_state, a.seg_decay, a.cu, a.segs, a.seg_len, a.H, a.K, \
+                                   a.P, WKV);                                                   \
+    }                                                                                           \
+    scan_prompt_kernel<T, KT, WKV, false><<<grid, dim3(256), n * sizeof(float), stream>>>(a);   \
   } while (0)
   if (a.K <= 16) LAUNCH(1);
   else if (a.K <= 32) LAUNCH(2);
@@ -903,13 +995,14 @@ at::Tensor gated_group_norm(const at::Tensor& y, const at::Tensor& z, const at::
 at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
                       const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& cu,
                       const std::optional<at::Tensor>& slot,
-                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N) {
+                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N,
+                      int64_t max_len) {
   TORCH_CHECK(xbc.dim() == 2 && is_elem(xbc), "ssd_prompt: xbc [T, C]");
   const int64_t T = xbc.size(0), H = a_log.numel(), C = xbc.size(1);
   const int64_t P = H > 0 ? (C - 2 * groups * N) / H : 0;
   const auto dt = xbc.scalar_type();
   TORCH_CHECK(H >= 1 && groups >= 1 && H % groups == 0 && N >= 1 && N <= MAX_KEYS && P >= 1 &&
-                  C == H * P + 2 * groups * N && H <= 65535,
+                  C == H * P + 2 * groups * N && H <= 65535 && max_len >= 1,
               "ssd_prompt: sizes (state up to ", MAX_KEYS, ")");
   check_t(xbc, dt, T * C, "ssd_prompt xbc");
   check_rows(dt_in, dt, T, H, "ssd_prompt dt");
@@ -942,7 +1035,7 @@ at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::
     a.K = (int)N;
     a.P = (int)P;
     a.out = PTR(out);
-    launch_scan<scalar, false>(a, n, stream);
+    launch_scan<scalar, false>(a, n, max_len, xbc.options().dtype(at::kFloat), stream);
   });
   HIP_CHECK_KERNEL();
   return out;
@@ -992,7 +1085,7 @@ at::Tensor wkv_prompt(const at::Tensor& r, const at::Tensor& k, const at::Tensor
   TORCH_CHECK(r.dim() == 2 && u.dim() == 2 && is_elem(r), "wkv_prompt: r [T, H*n], u [H, n]");
   const int64_t T = r.size(0), H = u.size(0), n = u.size(1);
   const auto dt = r.scalar_type();
-  TORCH_CHECK(n >= 1 && n <= MAX_KEYS && H >= 1 && H <= 65535 && max_len >= 0,
+  TORCH_CHECK(n >= 1 && n <= MAX_KEYS && H >= 1 && H <= 65535 && max_len >= 1,
               "wkv_prompt: heads of up to ", MAX_KEYS);
   check_rows(r, dt, T, H * n, "wkv_prompt r");
   check_rows(k, dt, T, H * n, "wkv_prompt k");
@@ -1027,7 +1120,7 @@ at::Tensor wkv_prompt(const at::Tensor& r, const at::Tensor& k, const at::Tensor
     a.H = (int)H;
     a.K = a.P = (int)n;
     a.out = PTR(out);
-    launch_scan<scalar, true>(a, seqs, stream);
+    launch_scan<scalar, true>(a, seqs, max_len, low.options(), stream);
   });
   HIP_CHECK_KERNEL();
   return out;

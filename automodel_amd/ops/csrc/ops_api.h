@@ -167,7 +167,8 @@ at::Tensor gated_group_norm(const at::Tensor& y, const at::Tensor& z, const at::
 at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
                       const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& cu,
                       const std::optional<at::Tensor>& slot,
-                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N);
+                      const std::optional<at::Tensor>& state, int64_t groups, int64_t N,
+                      int64_t max_len);
 at::Tensor ssd_decode(const at::Tensor& xbc, const at::Tensor& dt_in, const at::Tensor& dt_bias,
                       const at::Tensor& a_log, const at::Tensor& d_skip, const at::Tensor& slot,
                       at::Tensor state, int64_t groups, int64_t N);

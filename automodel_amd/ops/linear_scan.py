@@ -120,7 +120,8 @@ def ssd_scan(xbc: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor, a_log: 
     if use_hip(xbc):
         if step.prompt:
             return hip_ops().ssd_prompt(xbc, dt, dt_bias, a_log, d_skip, step.cu_seqlens,
-                                        _slots(step, state), state, groups, n_state)
+                                        _slots(step, state), state, groups, n_state,
+                                        step.max_len)
         return hip_ops().ssd_decode(xbc, dt, dt_bias, a_log, d_skip, step.slots, state, groups,
                                     n_state)
     T, H = dt.shape

@@ -546,6 +546,51 @@ def test_wkv_recurrence(dev, dt, H, n, cut):
 
 
 @on_each
+@pytest.mark.parametrize("kind", ["ssd", "wkv"])
+@torch.no_grad()
+def test_long_prompts_of_few_heads(dev, dt, kind):
+    """Lengths at which the GPU works on parts of a sequence at once; the state
+    that is left behind continues the sequence."""
+    dtype, lens, H, n, N = getattr(torch, dt), [390, 1, 257, 128], 2, 16, 24
+    T = sum(lens)
+    u, w0 = randn(H, n, seed=3).to(dtype), torch.linspace(-8, 1, H * n).to(dtype)
+    x = randn(T, 3 * H * n + 2 * N + H, seed=5).to(dtype)
+    norm, w2 = torch.ones(H * n).to(dtype), torch.zeros(H * n, 8).to(dtype)
+    a_log, D = torch.tensor([-4.0, 0.5]).to(dtype), randn(H, seed=6).to(dtype)
+    state = torch.full((4, H, n if kind == "wkv" else N, n), 1e4, device=dev)
+    d = [t.to(dev) for t in (x, u, w0, norm, w2, a_log, D)]
+
+    def run(rows, step):
+        xs = d[0][rows.to(dev)]
+        if kind == "ssd":
+            return linear_scan.ssd_scan(xs[:, :H * n + 2 * N].contiguous(), xs[:, -H:], d[6], d[5],
+                                        d[6], 1, N, step, state)
+        r, k, v = xs[:, :3 * H * n].split(H * n, -1)
+        if step.prompt:
+            low = torch.zeros(xs.shape[0], H * n, device=dev)
+            o = linear_scan.wkv_scan(r, k, v, low, d[2], d[1], step, state)
+            return linear_scan.gated_group_norm(o, torch.ones_like(o), d[3], H, 1e-3, False)
+        proj = torch.cat([r, k, v, torch.ones_like(r), torch.zeros_like(r[:, :8])], -1)
+        return linear_scan.wkv_decode(proj, d[4], d[2], d[1], d[3], 1e-3, step, state)
+
+    got = in_parts(run, lens, 386, dev)
+    for g, xs in zip(got, x.double().split(lens)):
+        m = xs.shape[0]
+        if kind == "ssd":
+            v, B, C = xs[:, :H * n + 2 * N].split([H * n, N, N], -1)
+            want = oracle.ssd_recurrence(v.reshape(m, H, n), B.reshape(m, 1, N),
+                                         C.reshape(m, 1, N),
+                                         oracle.softplus(xs[:, -H:] + D.double()),
+                                         a_log.double(), D.double()).reshape(m, -1)
+        else:
+            r, k, v = (t.reshape(m, H, n) for t in xs[:, :3 * H * n].split(H * n, -1))
+            w = torch.exp(-torch.exp(w0.double())).view(1, H, n).expand(m, -1, -1)
+            o = oracle.unit_rms(oracle.wkv_recurrence(r, k, v, w, u.double()), 1e-3)
+            want = o.reshape(m, -1) * oracle.silu(torch.ones(1).double())
+        close(g, want, dt, 1.0)
+
+
+@on_each
 @torch.no_grad()
 def test_states_remember_for_long(dev, dt):
     """One early token is all there is; it is read back 300 tokens later."""
