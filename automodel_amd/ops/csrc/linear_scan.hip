@@ -13,8 +13,9 @@
 //   ssd_decode / wkv_decode   one token per sequence
 //   gated_group_norm    rms norm in equal groups, gated before or after
 //
-// The prompt kernels hold S in the accumulators of 16x16x4 f32 MFMAs: a wave
-// owns 16 columns of one head and walks its sequence. A lane (g, c) of S has
+// The prompt kernels hold S in the accumulators of 16x16 MFMAs with f32 operands
+// (or with bf16 ones where that is exact): a wave owns 16 columns of one head and
+// walks its sequence. A lane (g, c) of S has
 // keys 4g..4g+3 of a tile, which is an MFMA operand once the summed index is
 // permuted in both operands alike; so S, the values and the 16x16 matrix within
 // a block are all used where they are, and only queries and keys pass through
@@ -24,14 +25,14 @@
 #include <ATen/ATen.h>
 #include <c10/hip/HIPStream.h>
 
-#include <type_traits>
-
 #include "elem.h"
 #include "ops_api.h"
 
 namespace amd_ops {
 
 typedef float scan_f32x4 __attribute__((ext_vector_type(4)));
+typedef short scan_s16x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 scan_bf16x8 __attribute__((ext_vector_type(8)));
 
 namespace {
 
@@ -245,69 +246,78 @@ struct ScanArgs {
   T* out;                              // [T, H * P]
 };
 
-template <typename T, int KT, bool WKV, bool STATES>
-__global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
-  constexpr int KP = KT * 16, LD = KP + 4;
-  extern __shared__ __attribute__((aligned(16))) float lds[];
-  float* qs = lds;                     // [TB][LD]
-  float* ks = qs + TB * LD;
-  float* cm = ks + TB * LD;            // wkv only from here
-  float* qd = cm + TB * LD;            // r times the decay since the block's start
-  float* kd = qd + TB * LD;            // k times the decay up to the block's end
-  float* es = kd + TB * LD;            // [KP] decay over the block
-  float* us = es + KP;                 // [KP]
-  float* am = us + KP;                 // [TB][TB + 4] weights within the block
-
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, lo = lane & 15, lg = lane >> 4;
-  const int h = blockIdx.y, seq = blockIdx.z / a.segs, seg = blockIdx.z % a.segs;
-  const int left = a.cu[seq + 1] - a.cu[seq] - seg * a.seg_len;
-  const int s0 = a.cu[seq] + seg * a.seg_len, len = min(left, a.seg_len);
-  const bool last = left <= a.seg_len;
-  if (len <= 0 || (STATES && last)) return;        // uniform over the block
-  const long sh = (long)blockIdx.z * a.H + h;
-  const int col = (blockIdx.x * 4 + wid) * 16 + lo;
-  const bool live = col < a.P;
-  const int colc = live ? col : a.P - 1;
-  const T* qb = a.q + (long)(h / a.per_group) * a.q_hs;
-  const T* kb = a.k + (long)(h / a.per_group) * a.k_hs;
-  const T* vb = a.v + (long)h * a.P + colc;
-  const float* cb = WKV ? a.cum + (long)h * a.K : nullptr;
-
-  float decay_rate = 0.f, dt_bias = 0.f, d_skip = 0.f;
-  if constexpr (WKV) {
-    for (int i = tid; i < KP; i += 256) us[i] = i < a.K ? to_f32(a.u[(long)h * a.K + i]) : 0.f;
-    for (int i = tid; i < TB * (TB + 4); i += 256) am[i] = 0.f;
-  } else {
-    decay_rate = -expf(to_f32(a.a_log[h]));
-    dt_bias = to_f32(a.dt_bias[h]);
-    d_skip = to_f32(a.d_skip[h]);
-  }
-
+// What a workgroup works on, and the state in MFMA accumulators: lane (g, c) of
+// tile kt has keys 16 kt + 4 g + r of column c.
+template <typename T, int KT>
+struct ScanWork {
+  static constexpr int KP = KT * 16;
+  const ScanArgs<T>& a;
+  int tid, wid, lo, lg, h, seg, s0, len, col, colc;
+  int own_i, own_ch;                   // staging: KT neighbouring channels of one token
+  bool live, last;
+  long sh;                             // index of (sequence, segment, head)
   scan_f32x4 S[KT];
+
+  __device__ __forceinline__ explicit ScanWork(const ScanArgs<T>& args) : a(args) {
+    tid = threadIdx.x;
+    wid = tid >> 6;
+    lo = tid & 15;
+    lg = (tid & 63) >> 4;
+    own_i = tid >> 4;
+    own_ch = (tid & 15) * KT;
+    h = blockIdx.y;
+    seg = blockIdx.z % a.segs;
+    const int seq = blockIdx.z / a.segs;
+    const int left = a.cu[seq + 1] - a.cu[seq] - seg * a.seg_len;
+    s0 = a.cu[seq] + seg * a.seg_len;
+    len = min(left, a.seg_len);
+    last = left <= a.seg_len;
+    col = (blockIdx.x * 4 + wid) * 16 + lo;
+    live = col < a.P;
+    colc = live ? col : a.P - 1;
+    sh = (long)blockIdx.z * a.H + h;
+  }
+  __device__ __forceinline__ void begin(bool from_zero) {
 #pragma unroll
-  for (int i = 0; i < KT; ++i) S[i] = scan_f32x4{0.f, 0.f, 0.f, 0.f};
-  if (!STATES && seg > 0) {
+    for (int i = 0; i < KT; ++i) S[i] = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+    if (from_zero || seg == 0) return;
     const float* st = a.seg_state + sh * a.K * a.P + colc;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = kt * 16 + lg * 4 + r;
-        S[kt][r] = st[(long)min(key, a.K - 1) * a.P];
-        if (key >= a.K) S[kt][r] = 0.f;
+        const float x = st[(long)min(key, a.K - 1) * a.P];
+        S[kt][r] = key < a.K ? x : 0.f;
       }
   }
-  float log_decay = 0.f;                           // STATES: over the segment
-
-  // The next block's operands, loaded while this one is computed: as they are,
-  // and from clamped places without a branch, so that all loads are in flight
-  // at once. A thread has KT neighbouring channels of one token.
-  const int own_i = tid >> 4, own_ch = (tid & 15) * KT;
-  T qr[KT], kr[KT], vr[4], dtr = T{};
-  float cr[WKV ? KT : 1];
-  auto fetch_row = [&](const auto* row, auto (&to)[KT], bool vec) {
-    using E = std::remove_reference_t<decltype(to[0])>;
-    if (vec) {
+  __device__ __forceinline__ void store(float* st) const {
+    if (!live) return;
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = kt * 16 + lg * 4 + r;
+        if (key < a.K) st[(long)key * a.P + col] = S[kt][r];
+      }
+  }
+  __device__ __forceinline__ void store_segment() const { store(a.seg_state + sh * a.K * a.P); }
+  __device__ __forceinline__ void store_final() const {
+    if (a.state == nullptr || !last) return;
+    const int sl = a.slot[s0];
+    if (sl >= 0 && sl < a.n_slots) store(a.state + ((long)sl * a.H + h) * a.K * a.P);
+  }
+  __device__ __forceinline__ void store_out(int c0, int nt, const scan_f32x4& o) const {
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (live && lg * 4 + r < nt)
+        a.out[(long)(s0 + c0 + lg * 4 + r) * a.H * a.P + (long)h * a.P + col] = from_f32<T>(o[r]);
+  }
+  // This thread's channels of a token's row, as they are. Places are clamped
+  // rather than skipped: all loads of a block are then in flight at once.
+  template <typename E>
+  __device__ __forceinline__ void fetch_row(const E* row, E (&to)[KT]) const {
+    if (a.vec) {
       constexpr int N = KT * sizeof(E) > 16 ? 16 / sizeof(E) : KT;   // elements per load
 #pragma unroll
       for (int j = 0; j < KT; j += N) {
@@ -319,91 +329,115 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
 #pragma unroll
       for (int j = 0; j < KT; ++j) to[j] = row[min(own_ch + j, a.K - 1)];
     }
-  };
-  auto fetch = [&](int c0) {
-    const int nt = min(TB, len - c0);
-    const long t = s0 + c0 + min(own_i, nt - 1);
-    if constexpr (!STATES) fetch_row(qb + t * a.q_ld, qr, a.vec);
-    fetch_row(kb + t * a.k_ld, kr, a.vec);
-    // past the end the sum of log decays stays where it is
-    if constexpr (WKV) fetch_row(cb + t * ((long)a.H * a.K), cr, a.vec);
+  }
+  __device__ __forceinline__ void fetch_values(int c0, int nt, T (&to)[4]) const {
+    const T* vb = a.v + (long)h * a.P + colc;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) vr[r] = vb[(long)(s0 + c0 + min(lg * 4 + r, nt - 1)) * a.v_ld];
-    if constexpr (!WKV) dtr = a.dt[(long)(s0 + c0 + min(lo, nt - 1)) * a.dt_ld + h];
+    for (int r = 0; r < 4; ++r) to[r] = vb[(long)(s0 + c0 + min(lg * 4 + r, nt - 1)) * a.v_ld];
+  }
+  __device__ __forceinline__ bool own_in(int j, int nt) const {
+    return own_i < nt && own_ch + j < a.K;
+  }
+};
+
+// STATES: the segment's state from zero and its decay, without outputs.
+template <typename T, int KT, bool STATES>
+__global__ __launch_bounds__(256) void wkv_prompt_kernel(ScanArgs<T> a) {
+  constexpr int KP = KT * 16, LD = KP + 4;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float* qs = lds;                     // [TB][LD]
+  float* ks = qs + TB * LD;
+  float* cm = ks + TB * LD;            // sums of log decays
+  float* qd = cm + TB * LD;            // r times the decay since the block's start
+  float* kd = qd + TB * LD;            // k times the decay up to the block's end
+  float* es = kd + TB * LD;            // [KP] decay over the block
+  float* us = es + KP;                 // [KP]
+  float* am = us + KP;                 // [TB][TB + 4] weights within the block
+
+  ScanWork<T, KT> wk(a);
+  if (wk.len <= 0 || (STATES && wk.last)) return;  // uniform over the block
+  const int tid = wk.tid, lo = wk.lo, lg = wk.lg;
+  const T* qb = a.q + (long)wk.h * a.q_hs;
+  const T* kb = a.k + (long)wk.h * a.k_hs;
+  const float* cb = a.cum + (long)wk.h * a.K;
+  if constexpr (!STATES) {
+    for (int i = tid; i < KP; i += 256) us[i] = i < a.K ? to_f32(a.u[(long)wk.h * a.K + i]) : 0.f;
+    for (int i = tid; i < TB * (TB + 4); i += 256) am[i] = 0.f;
+  }
+  wk.begin(STATES);
+  float log_decay = 0.f;                           // STATES: of channel tid
+
+  T qr[KT], kr[KT], vr[4];                         // the next block's operands
+  float cr[KT];
+  auto fetch = [&](int c0) {
+    const int nt = min(TB, wk.len - c0);
+    const long t = wk.s0 + c0 + min(wk.own_i, nt - 1);
+    if constexpr (!STATES) wk.fetch_row(qb + t * a.q_ld, qr);
+    wk.fetch_row(kb + t * a.k_ld, kr);
+    // past the end the sum of log decays stays where it is
+    wk.fetch_row(cb + t * ((long)a.H * a.K), cr);
+    wk.fetch_values(c0, nt, vr);
   };
   fetch(0);
-
-  for (int c0 = 0; c0 < len; c0 += TB) {
-    const int nt = min(TB, len - c0);
+  for (int c0 = 0; c0 < wk.len; c0 += TB) {
+    const int nt = min(TB, wk.len - c0), at = wk.own_i * LD + wk.own_ch;
     __syncthreads();                               // the last block has been read
-    {
-      float x[KT], y[KT];
+    float x[KT], y[KT], c[KT];
 #pragma unroll
-      for (int j = 0; j < KT; ++j) {
-        const bool in = own_i < nt && own_ch + j < a.K;
-        x[j] = !STATES && in ? to_f32(qr[j]) : 0.f;
-        y[j] = in ? to_f32(kr[j]) : 0.f;
-      }
-      if constexpr (!STATES) put(qs + own_i * LD + own_ch, x);
-      put(ks + own_i * LD + own_ch, y);
-      if constexpr (WKV) {
-#pragma unroll
-        for (int j = 0; j < KT; ++j) x[j] = own_ch + j < a.K ? cr[j] : 0.f;
-        put(cm + own_i * LD + own_ch, x);
-      }
+    for (int j = 0; j < KT; ++j) {
+      x[j] = !STATES && wk.own_in(j, nt) ? to_f32(qr[j]) : 0.f;
+      y[j] = wk.own_in(j, nt) ? to_f32(kr[j]) : 0.f;
+      c[j] = wk.own_ch + j < a.K ? cr[j] : 0.f;
     }
+    if constexpr (!STATES) put(qs + at, x);
+    put(ks + at, y);
+    put(cm + at, c);
     float v[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = lg * 4 + r < nt ? to_f32(vr[r]) : 0.f;
-    float dt = 0.f;
-    if constexpr (!WKV) dt = lo < nt ? softplus_f(to_f32(dtr) + dt_bias) : 0.f;
     __syncthreads();
-    if (c0 + TB < len) fetch(c0 + TB);
+    if (c0 + TB < wk.len) fetch(c0 + TB);
 
-    scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f};
-    if constexpr (WKV) {
-      {
-        float x[KT], y[KT], c[KT], before[KT], end[KT];
-        const int at = own_i * LD + own_ch;
-        get(ks + at, y);
-        get(cm + at, c);
-        get(cm + (TB - 1) * LD + own_ch, end);
-        if constexpr (!STATES) {
-          get(qs + at, x);
-          get(cm + max(at - LD, own_ch), before);
-        }
+    float end[KT];
+    get(cm + (TB - 1) * LD + wk.own_ch, end);
+    if constexpr (!STATES) {
+      float before[KT];
+      get(cm + max(at - LD, wk.own_ch), before);
 #pragma unroll
-        for (int j = 0; j < KT; ++j) {
-          if constexpr (!STATES) x[j] *= own_i > 0 ? __expf(before[j]) : 1.f;
-          y[j] *= __expf(end[j] - c[j]);
-          end[j] = __expf(end[j]);
-        }
-        if constexpr (!STATES) put(qd + at, x);
-        put(kd + at, y);
-        if (own_i == 0) put(es + own_ch, end);
-        if (STATES && tid < KP) log_decay += cm[(TB - 1) * LD + tid];
-      }
-      if constexpr (!STATES) {
+      for (int j = 0; j < KT; ++j) x[j] *= wk.own_i > 0 ? __expf(before[j]) : 1.f;
+      put(qd + at, x);
+    } else if (tid < KP) {
+      log_decay += cm[(TB - 1) * LD + tid];
+    }
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      y[j] *= __expf(end[j] - c[j]);
+      end[j] = __expf(end[j]);
+    }
+    put(kd + at, y);
+    if (wk.own_i == 0) put(es + wk.own_ch, end);
+
+    if constexpr (!STATES) {
       // Weights of earlier tokens j for i within the block. Wave `wid` takes the
       // pairs that part at half size hs: j in the lower, i in the upper half of
       // a group of 2 hs, both measured against the group's middle.
-      const int hs = 8 >> wid;
+      const int hs = 8 >> wk.wid;
       const int mid = lo / (2 * hs) * (2 * hs) + hs - 1;
       const bool upper = (lo & hs) != 0;
       scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
         const int ch = kt * 16 + lg * 4;
-        const float4 x = *reinterpret_cast<const float4*>((upper ? qs : ks) + lo * LD + ch);
+        const float4 p = *reinterpret_cast<const float4*>((upper ? qs : ks) + lo * LD + ch);
         const float4 cmid = *reinterpret_cast<const float4*>(cm + mid * LD + ch);
         const float4 cown =
             *reinterpret_cast<const float4*>(cm + (upper ? lo - 1 : lo) * LD + ch);
-        const float xs[4] = {x.x, x.y, x.z, x.w};
+        const float ps[4] = {p.x, p.y, p.z, p.w};
         const float ds[4] = {cown.x - cmid.x, cown.y - cmid.y, cown.z - cmid.z, cown.w - cmid.w};
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float y = xs[r] * __expf(upper ? ds[r] : -ds[r]);
-          g = mfma4(upper ? 0.f : y, upper ? y : 0.f, g);   // row j, column i
+          const float w = ps[r] * __expf(upper ? ds[r] : -ds[r]);
+          g = mfma4(upper ? 0.f : w, upper ? w : 0.f, g);   // row j, column i
         }
       }
 #pragma unroll
@@ -411,122 +445,266 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanArgs<T> a) {
         const int j = lg * 4 + r, i = lo;
         if (upper && !(j & hs) && i / (2 * hs) == j / (2 * hs)) am[i * (TB + 4) + j] = g[r];
       }
-      {                                            // the token itself, with the bonus
-        const int i = tid >> 4, part = tid & 15;
-        float d = 0.f;
-        for (int ch = part; ch < KP; ch += 16) d = fmaf(qs[i * LD + ch] * us[ch], ks[i * LD + ch], d);
+      // the token itself, with the bonus: 16 threads each
+      float d = 0.f;
+      for (int ch = lo; ch < KP; ch += 16)
+        d = fmaf(qs[wk.own_i * LD + ch] * us[ch], ks[wk.own_i * LD + ch], d);
 #pragma unroll
-        for (int off = 8; off > 0; off >>= 1) d += __shfl_xor(d, off);
-        if (part == 0) am[i * (TB + 4) + i] = d;
-      }
-      }
-      __syncthreads();
-      if constexpr (!STATES) {
+      for (int off = 8; off > 0; off >>= 1) d += __shfl_xor(d, off);
+      if (lo == 0) am[wk.own_i * (TB + 4) + wk.own_i] = d;
+    }
+    __syncthreads();
+    if constexpr (!STATES) {
+      scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f}, o2 = o;
 #pragma unroll
       for (int kt = 0; kt < KT; ++kt) {
-        const float4 x = *reinterpret_cast<const float4*>(qd + lo * LD + kt * 16 + lg * 4);
-        o = mfma4(x.x, S[kt][0], o);
-        o = mfma4(x.y, S[kt][1], o);
-        o = mfma4(x.z, S[kt][2], o);
-        o = mfma4(x.w, S[kt][3], o);
+        const float4 p = *reinterpret_cast<const float4*>(qd + lo * LD + kt * 16 + lg * 4);
+        o = mfma4(p.x, wk.S[kt][0], o);
+        o2 = mfma4(p.y, wk.S[kt][1], o2);
+        o = mfma4(p.z, wk.S[kt][2], o);
+        o2 = mfma4(p.w, wk.S[kt][3], o2);
       }
       const float4 w = *reinterpret_cast<const float4*>(am + lo * (TB + 4) + lg * 4);
       o = mfma4(w.x, v[0], o);
-      o = mfma4(w.y, v[1], o);
+      o2 = mfma4(w.y, v[1], o2);
       o = mfma4(w.z, v[2], o);
-      o = mfma4(w.w, v[3], o);
-      }
-#pragma unroll
-      for (int kt = 0; kt < KT; ++kt) {
-        const float4 e = *reinterpret_cast<const float4*>(es + kt * 16 + lg * 4);
-        S[kt][0] *= e.x;
-        S[kt][1] *= e.y;
-        S[kt][2] *= e.z;
-        S[kt][3] *= e.w;
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-#pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
-          S[kt] = mfma4(kd[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
-    } else {
-      float cs = decay_rate * dt;                  // log decay up to and with token lo
-#pragma unroll
-      for (int off = 1; off < TB; off <<= 1) {
-        const float t = __shfl_up(cs, off, TB);
-        if (lo >= off) cs += t;
-      }
-      const float total = __shfl(cs, TB - 1, TB);
-      log_decay += total;
-      scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
-      if constexpr (!STATES) {
-#pragma unroll
-      for (int kt = 0; kt < KT; ++kt) {
-        const float4 x = *reinterpret_cast<const float4*>(qs + lo * LD + kt * 16 + lg * 4);
-        const float4 y = *reinterpret_cast<const float4*>(ks + lo * LD + kt * 16 + lg * 4);
-        g = mfma4(y.x, x.x, g);
-        o = mfma4(x.x, S[kt][0], o);
-        g = mfma4(y.y, x.y, g);
-        o = mfma4(x.y, S[kt][1], o);
-        g = mfma4(y.z, x.z, g);
-        o = mfma4(x.z, S[kt][2], o);
-        g = mfma4(y.w, x.w, g);
-        o = mfma4(x.w, S[kt][3], o);
-      }
-      }
-      float f[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float csj = __shfl(cs, lg * 4 + r, TB), dtj = __shfl(dt, lg * 4 + r, TB);
-        g[r] = lg * 4 + r <= lo ? g[r] * __expf(cs - csj) * dtj : 0.f;
-        o[r] *= __expf(csj);
-        f[r] = __expf(total - csj) * dtj;
-      }
-      if constexpr (!STATES) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
-      }
-      const float e = __expf(total);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        o[r] = fmaf(d_skip, v[r], o[r]);
-        v[r] *= f[r];
-      }
-#pragma unroll
-      for (int kt = 0; kt < KT; ++kt) S[kt] *= e;
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-#pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
-          S[kt] = mfma4(ks[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
+      o2 = mfma4(w.w, v[3], o2);
+      o += o2;
+      wk.store_out(c0, nt, o);
     }
-    if constexpr (STATES) continue;
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const float4 e = *reinterpret_cast<const float4*>(es + kt * 16 + lg * 4);
+      wk.S[kt][0] *= e.x;
+      wk.S[kt][1] *= e.y;
+      wk.S[kt][2] *= e.z;
+      wk.S[kt][3] *= e.w;
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      if (live && lg * 4 + r < nt)
-        a.out[(long)(s0 + c0 + lg * 4 + r) * a.H * a.P + (long)h * a.P + col] = from_f32<T>(o[r]);
-  }
-  float* st;
-  if constexpr (STATES) {
-    if (blockIdx.x == 0) {
-      if (WKV && tid < a.K) a.seg_decay[sh * a.K + tid] = __expf(log_decay);
-      if (!WKV && tid == 0) a.seg_decay[sh] = __expf(log_decay);
-    }
-    st = a.seg_state + sh * a.K * a.P + col;
-  } else {
-    if (a.state == nullptr || !last) return;
-    const int sl = a.slot[s0];
-    if (sl < 0 || sl >= a.n_slots) return;
-    st = a.state + ((long)sl * a.H + h) * a.K * a.P + col;
-  }
-  if (!live) return;
 #pragma unroll
-  for (int kt = 0; kt < KT; ++kt)
+      for (int kt = 0; kt < KT; ++kt)
+        wk.S[kt] = mfma4(kd[(lg * 4 + r) * LD + kt * 16 + lo], v[r], wk.S[kt]);
+  }
+  if constexpr (STATES) {
+    if (blockIdx.x == 0 && tid < a.K) a.seg_decay[wk.sh * a.K + tid] = __expf(log_decay);
+    wk.store_segment();
+  } else {
+    wk.store_final();
+  }
+}
+
+// Queries and keys in LDS for the state-space kernel, and the products with them.
+// f32: both as [TB][KP + 4].
+template <typename T, int KT>
+struct SsdOperands {
+  static constexpr int KP = KT * 16, LD = KP + 4;
+  static constexpr size_t BYTES = 2 * TB * LD * sizeof(float);
+  float *qs, *ks;
+  __device__ __forceinline__ explicit SsdOperands(char* lds)
+      : qs(reinterpret_cast<float*>(lds)), ks(qs + TB * LD) {}
+  template <typename W>
+  __device__ __forceinline__ void stage(const W& wk, const T (&q)[KT], const T (&k)[KT], int nt,
+                                        bool queries) {
+    float x[KT], y[KT];
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      x[j] = queries && wk.own_in(j, nt) ? to_f32(q[j]) : 0.f;
+      y[j] = wk.own_in(j, nt) ? to_f32(k[j]) : 0.f;
+    }
+    if (queries) put(qs + wk.own_i * LD + wk.own_ch, x);
+    put(ks + wk.own_i * LD + wk.own_ch, y);
+  }
+  // row j, column i: k_j . q_i
+  __device__ __forceinline__ scan_f32x4 gram(int lo, int lg) const {
+    scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f}, g2 = g;
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const float4 x = *reinterpret_cast<const float4*>(qs + lo * LD + kt * 16 + lg * 4);
+      const float4 y = *reinterpret_cast<const float4*>(ks + lo * LD + kt * 16 + lg * 4);
+      g = mfma4(y.x, x.x, g);
+      g2 = mfma4(y.y, x.y, g2);
+      g = mfma4(y.z, x.z, g);
+      g2 = mfma4(y.w, x.w, g2);
+    }
+    return g + g2;
+  }
+  __device__ __forceinline__ float4 query4(int lo, int ch) const {
+    return *reinterpret_cast<const float4*>(qs + lo * LD + ch);
+  }
+  // S += k^T v, v[r] the value of token 4 lg + r
+  __device__ __forceinline__ void add(scan_f32x4 (&S)[KT], const float (&v)[4], int lo,
+                                      int lg) const {
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt)
+        S[kt] = mfma4(ks[(lg * 4 + r) * LD + kt * 16 + lo], v[r], S[kt]);
+  }
+};
+
+// bf16: products of two bf16 operands are exact in f32, and an f32 value is the
+// sum of three bf16 parts, so the bf16 matrix cores give f32 results here at a
+// multiple of the f32 rate. Keys also transposed, [KP][TB + 4].
+template <int KT>
+struct SsdOperands<bf16, KT> {
+  static constexpr int KP = KT * 16, LD = KP + 8, TD = TB + 4;
+  static constexpr size_t BYTES = (2 * TB * LD + KP * TD) * sizeof(bf16);
+  bf16 *qs, *ks, *kt_;
+  __device__ __forceinline__ explicit SsdOperands(char* lds)
+      : qs(reinterpret_cast<bf16*>(lds)), ks(qs + TB * LD), kt_(ks + TB * LD) {}
+  template <typename W>
+  __device__ __forceinline__ void stage(const W& wk, const bf16 (&q)[KT], const bf16 (&k)[KT],
+                                        int nt, bool queries) {
+    const bf16 zero = f2bf(0.f);
+    ElemPack<bf16, KT> x, y;
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      x.v[j] = queries && wk.own_in(j, nt) ? q[j] : zero;
+      y.v[j] = wk.own_in(j, nt) ? k[j] : zero;
+      kt_[(wk.own_ch + j) * TD + wk.own_i] = y.v[j];
+    }
+    if (!queries) return;
+    *reinterpret_cast<ElemPack<bf16, KT>*>(qs + wk.own_i * LD + wk.own_ch) = x;
+    *reinterpret_cast<ElemPack<bf16, KT>*>(ks + wk.own_i * LD + wk.own_ch) = y;
+  }
+  __device__ __forceinline__ scan_f32x4 gram(int lo, int lg) const {
+    scan_f32x4 g = scan_f32x4{0.f, 0.f, 0.f, 0.f};
+    if constexpr (KT == 1) {
+      const scan_s16x4 y = *reinterpret_cast<const scan_s16x4*>(ks + lo * LD + lg * 4);
+      const scan_s16x4 x = *reinterpret_cast<const scan_s16x4*>(qs + lo * LD + lg * 4);
+      return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(y, x, g, 0, 0, 0);
+    } else {
+#pragma unroll
+      for (int c = 0; c < KP / 32; ++c) {
+        const scan_bf16x8 y = *reinterpret_cast<const scan_bf16x8*>(ks + lo * LD + c * 32 + lg * 8);
+        const scan_bf16x8 x = *reinterpret_cast<const scan_bf16x8*>(qs + lo * LD + c * 32 + lg * 8);
+        g = __builtin_amdgcn_mfma_f32_16x16x32_bf16(y, x, g, 0, 0, 0);
+      }
+      return g;
+    }
+  }
+  __device__ __forceinline__ float4 query4(int lo, int ch) const {
+    float x[4];
+    load_vec<bf16, 4>(qs + lo * LD + ch, x);
+    return float4{x[0], x[1], x[2], x[3]};
+  }
+  __device__ __forceinline__ void add(scan_f32x4 (&S)[KT], const float (&v)[4], int lo,
+                                      int lg) const {
+    // Both products are the same instruction: a chain through one accumulator of
+    // 16x16x32 and 16x16x16 steps right after one another lost results here.
+    scan_bf16x8 b;                                 // leading parts, then the middle ones
+    scan_bf16x8 b3{};                              // the rest
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int key = kt * 16 + lg * 4 + r;
-      if (key < a.K) st[(long)key * a.P] = S[kt][r];
+      const __bf16 v1 = (__bf16)v[r];
+      const float rest = v[r] - (float)v1;
+      const __bf16 v2 = (__bf16)rest;
+      b[r] = v1;
+      b[4 + r] = v2;
+      b3[r] = (__bf16)(rest - (float)v2);
     }
+    scan_bf16x8 k8[KT];                            // the tokens' keys, twice
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const scan_s16x4 k4 = *reinterpret_cast<const scan_s16x4*>(kt_ + (kt * 16 + lo) * TD + lg * 4);
+      k8[kt] = __builtin_bit_cast(scan_bf16x8,
+                                  __builtin_shufflevector(k4, k4, 0, 1, 2, 3, 4, 5, 6, 7));
+    }
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+      S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8[kt], b, S[kt], 0, 0, 0);
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+      S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8[kt], b3, S[kt], 0, 0, 0);
+  }
+};
+
+template <typename T, int KT, bool STATES>
+__global__ __launch_bounds__(256) void ssd_prompt_kernel(ScanArgs<T> a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  SsdOperands<T, KT> op(reinterpret_cast<char*>(lds));
+  ScanWork<T, KT> wk(a);
+  if (wk.len <= 0 || (STATES && wk.last)) return;  // uniform over the block
+  const int lo = wk.lo, lg = wk.lg;
+  const T* qb = a.q + (long)(wk.h / a.per_group) * a.q_hs;
+  const T* kb = a.k + (long)(wk.h / a.per_group) * a.k_hs;
+  const float rate = -expf(to_f32(a.a_log[wk.h])), dt_bias = to_f32(a.dt_bias[wk.h]);
+  const float skip = to_f32(a.d_skip[wk.h]);
+  wk.begin(STATES);
+  float log_decay = 0.f;                           // over the segment
+
+  T qr[KT], kr[KT], vr[4], dtr;                    // the next block's operands
+  auto fetch = [&](int c0) {
+    const int nt = min(TB, wk.len - c0);
+    const long t = wk.s0 + c0 + min(wk.own_i, nt - 1);
+    if constexpr (!STATES) wk.fetch_row(qb + t * a.q_ld, qr);
+    wk.fetch_row(kb + t * a.k_ld, kr);
+    wk.fetch_values(c0, nt, vr);
+    dtr = a.dt[(long)(wk.s0 + c0 + min(lo, nt - 1)) * a.dt_ld + wk.h];
+  };
+  fetch(0);
+  for (int c0 = 0; c0 < wk.len; c0 += TB) {
+    const int nt = min(TB, wk.len - c0);
+    __syncthreads();                               // the last block has been read
+    op.stage(wk, qr, kr, nt, !STATES);
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = lg * 4 + r < nt ? to_f32(vr[r]) : 0.f;
+    const float dt = lo < nt ? softplus_f(to_f32(dtr) + dt_bias) : 0.f;
+    __syncthreads();
+    if (c0 + TB < wk.len) fetch(c0 + TB);
+
+    float cs = rate * dt;                          // log decay up to and with token lo
+#pragma unroll
+    for (int off = 1; off < TB; off <<= 1) {
+      const float t = __shfl_up(cs, off, TB);
+      if (lo >= off) cs += t;
+    }
+    const float total = __shfl(cs, TB - 1, TB);
+    log_decay += total;
+    float csj[4], f[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      csj[r] = __shfl(cs, lg * 4 + r, TB);
+      f[r] = __shfl(dt, lg * 4 + r, TB);           // dt of token j
+    }
+    if constexpr (!STATES) {
+      scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f}, o2 = o;
+      scan_f32x4 g = op.gram(lo, lg);
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt) {
+        const float4 x = op.query4(lo, kt * 16 + lg * 4);
+        o = mfma4(x.x, wk.S[kt][0], o);
+        o2 = mfma4(x.y, wk.S[kt][1], o2);
+        o = mfma4(x.z, wk.S[kt][2], o);
+        o2 = mfma4(x.w, wk.S[kt][3], o2);
+      }
+      o += o2;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        g[r] = lg * 4 + r <= lo ? g[r] * __expf(cs - csj[r]) * f[r] : 0.f;
+        o[r] *= __expf(csj[r]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o = mfma4(g[r], v[r], o);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = fmaf(skip, v[r], o[r]);
+      wk.store_out(c0, nt, o);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] *= __expf(total - csj[r]) * f[r];
+    const float e = __expf(total);
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) wk.S[kt] *= e;
+    op.add(wk.S, v, lo, lg);
+  }
+  if constexpr (STATES) {
+    if (blockIdx.x == 0 && wk.tid == 0) a.seg_decay[wk.sh] = __expf(log_decay);
+    wk.store_segment();
+  } else {
+    wk.store_final();
+  }
 }
 
 // Segments' own states -> the states they begin with, in place. A thread has one
@@ -834,17 +1012,25 @@ void launch_scan(ScanArgs<T> a, int64_t n_seqs, int64_t max_len, const at::Tenso
     a.seg_decay = seg_decay.data_ptr<float>();
   }
   const dim3 grid((a.P + 63) / 64, a.H, n_seqs * a.segs);
+#define LAUNCH_PASS(KT, STATES)                                                                 \
+  do {                                                                                          \
+    if constexpr (WKV) {                                                                        \
+      const size_t n = 5 * TB * (KT * 16 + 4) + 2 * KT * 16 + TB * (TB + 4);                    \
+      wkv_prompt_kernel<T, KT, STATES><<<grid, dim3(256), n * sizeof(float), stream>>>(a);      \
+    } else {                                                                                    \
+      ssd_prompt_kernel<T, KT, STATES>                                                          \
+          <<<grid, dim3(256), SsdOperands<T, KT>::BYTES, stream>>>(a);                          \
+    }                                                                                           \
+  } while (0)
 #define LAUNCH(KT)                                                                              \
   do {                                                                                          \
-    const size_t row = TB * (KT * 16 + 4);                                                      \
-    const size_t n = WKV ? 5 * row + 2 * KT * 16 + TB * (TB + 4) : 2 * row;                     \
     if (a.segs > 1) {                                                                           \
-      scan_prompt_kernel<T, KT, WKV, true><<<grid, dim3(256), n * sizeof(float), stream>>>(a);  \
+      LAUNCH_PASS(KT, true);                                                                    \
       scan_link_kernel<<<dim3(ceil_div_i((long)a.H * a.K * a.P, 256), n_seqs), dim3(256), 0,    \
                          stream>>>(a.seg_state, a.seg_decay, a.cu, a.segs, a.seg_len, a.H, a.K, \
                                    a.P, WKV);                                                   \
     }                                                                                           \
-    scan_prompt_kernel<T, KT, WKV, false><<<grid, dim3(256), n * sizeof(float), stream>>>(a);   \
+    LAUNCH_PASS(KT, false);                                                                     \
   } while (0)
   if (a.K <= 16) LAUNCH(1);
   else if (a.K <= 32) LAUNCH(2);
@@ -852,6 +1038,7 @@ void launch_scan(ScanArgs<T> a, int64_t n_seqs, int64_t max_len, const at::Tenso
   else if (a.K <= 128) LAUNCH(8);
   else LAUNCH(16);
 #undef LAUNCH
+#undef LAUNCH_PASS
 }
 
 int64_t check_bounds(const at::Tensor& cu, int64_t T, const std::optional<at::Tensor>& slot,
