@@ -8,7 +8,7 @@
 //
 //   causal_conv_silu    short convolution per channel, with its cached inputs
 //   token_shift         h + (h' - h) * mu for several mu, h' the token before
-//   decay_cumsum        log decays summed within blocks of 16 tokens
+//   decay_cumsum / step_cumsum   log decays summed within blocks of 16 tokens
 //   ssd_prompt / wkv_prompt   blocks of 16 tokens on the f32 matrix cores
 //   ssd_decode / wkv_decode   one token per sequence
 //   gated_group_norm    rms norm in equal groups, gated before or after
@@ -191,6 +191,27 @@ __global__ __launch_bounds__(256) void decay_cumsum_kernel(float* __restrict__ l
   }
 }
 
+// dt [T, H] -> steps softplus(dt + bias) and sums of the log decays
+// -exp(A_log) * step from each block's start, both [H, T].
+template <typename T>
+__global__ __launch_bounds__(256) void step_cumsum_kernel(
+    const T* __restrict__ dt, long dt_ld, const T* __restrict__ bias, const T* __restrict__ a_log,
+    const int* __restrict__ cu, int H, int n_tok, float* __restrict__ steps,
+    float* __restrict__ sums) {
+  const int h = blockIdx.z * 64 + (threadIdx.x & 63);
+  const int t0 = cu[blockIdx.y] + (blockIdx.x * 4 + (threadIdx.x >> 6)) * TB;
+  const int t1 = min(t0 + TB, cu[blockIdx.y + 1]);
+  if (h >= H) return;
+  const float b = to_f32(bias[h]), rate = -expf(to_f32(a_log[h]));
+  float s = 0.f;
+  for (int t = t0; t < t1; ++t) {
+    const float step = softplus_f(to_f32(dt[t * dt_ld + h]) + b);
+    s += fmaxf(rate * step, MIN_LOG);
+    steps[(long)h * n_tok + t] = step;
+    sums[(long)h * n_tok + t] = s;
+  }
+}
+
 // ---------------------------------------------------------------------------
 // prompts: grid (column groups of 64, heads, sequences x segments), one wave per
 // 16 columns. Few heads and long sequences leave most of the chip idle, so a
@@ -234,8 +255,9 @@ struct ScanArgs {
   int q_hs, k_hs, per_group;           // head strides; heads per q/k group
   const float* cum;                    // wkv: [T, H * K]
   const T* u;                          // wkv: [H, K]
-  const T *dt, *dt_bias, *a_log, *d_skip;   // state space: dt row t at t * dt_ld
-  long dt_ld;
+  const T* d_skip;                     // state space: [H]
+  const float *steps, *sums;           // state space: [H, n_tok]
+  int n_tok;
   const int *cu, *slot;
   float* state;                        // [slots, H, K, P] or null
   int segs, seg_len;                   // segments per sequence, in whole blocks
@@ -629,19 +651,27 @@ __global__ __launch_bounds__(256) void ssd_prompt_kernel(ScanArgs<T> a) {
   const int lo = wk.lo, lg = wk.lg;
   const T* qb = a.q + (long)(wk.h / a.per_group) * a.q_hs;
   const T* kb = a.k + (long)(wk.h / a.per_group) * a.k_hs;
-  const float rate = -expf(to_f32(a.a_log[wk.h])), dt_bias = to_f32(a.dt_bias[wk.h]);
+  const float* steps = a.steps + (long)wk.h * a.n_tok + wk.s0;
+  const float* sums = a.sums + (long)wk.h * a.n_tok + wk.s0;
   const float skip = to_f32(a.d_skip[wk.h]);
   wk.begin(STATES);
   float log_decay = 0.f;                           // over the segment
 
-  T qr[KT], kr[KT], vr[4], dtr;                    // the next block's operands
+  T qr[KT], kr[KT], vr[4];                         // the next block's operands
+  float step_r[4], sum_r[4], own_r, total_r;
   auto fetch = [&](int c0) {
     const int nt = min(TB, wk.len - c0);
     const long t = wk.s0 + c0 + min(wk.own_i, nt - 1);
     if constexpr (!STATES) wk.fetch_row(qb + t * a.q_ld, qr);
     wk.fetch_row(kb + t * a.k_ld, kr);
     wk.fetch_values(c0, nt, vr);
-    dtr = a.dt[(long)(wk.s0 + c0 + min(lo, nt - 1)) * a.dt_ld + wk.h];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      step_r[r] = steps[c0 + min(lg * 4 + r, nt - 1)];
+      sum_r[r] = sums[c0 + min(lg * 4 + r, nt - 1)];
+    }
+    own_r = sums[c0 + min(lo, nt - 1)];
+    total_r = sums[c0 + nt - 1];
   };
   fetch(0);
   for (int c0 = 0; c0 < wk.len; c0 += TB) {
@@ -651,24 +681,18 @@ __global__ __launch_bounds__(256) void ssd_prompt_kernel(ScanArgs<T> a) {
     float v[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) v[r] = lg * 4 + r < nt ? to_f32(vr[r]) : 0.f;
-    const float dt = lo < nt ? softplus_f(to_f32(dtr) + dt_bias) : 0.f;
-    __syncthreads();
-    if (c0 + TB < wk.len) fetch(c0 + TB);
-
-    float cs = rate * dt;                          // log decay up to and with token lo
-#pragma unroll
-    for (int off = 1; off < TB; off <<= 1) {
-      const float t = __shfl_up(cs, off, TB);
-      if (lo >= off) cs += t;
-    }
-    const float total = __shfl(cs, TB - 1, TB);
-    log_decay += total;
+    // of token lo, of tokens 4 lg + r (whose value is 0 past the end), of the block
+    const float cs = own_r, total = total_r;
     float csj[4], f[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      csj[r] = __shfl(cs, lg * 4 + r, TB);
-      f[r] = __shfl(dt, lg * 4 + r, TB);           // dt of token j
+      csj[r] = sum_r[r];
+      f[r] = step_r[r];
     }
+    __syncthreads();
+    if (c0 + TB < wk.len) fetch(c0 + TB);
+
+    log_decay += total;
     if constexpr (!STATES) {
       scan_f32x4 o = scan_f32x4{0.f, 0.f, 0.f, 0.f}, o2 = o;
       scan_f32x4 g = op.gram(lo, lg);
@@ -1200,6 +1224,7 @@ at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::
   if (state) check_t(*state, at::kFloat, state->size(0) * H * N * P, "ssd_prompt state");
   auto out = at::empty({T, H * P}, xbc.options());
   if (T == 0) return out;
+  auto steps = at::empty({H, T}, xbc.options().dtype(at::kFloat)), sums = at::empty_like(steps);
   auto stream = c10::hip::getCurrentHIPStream().stream();
   AMD_DISPATCH_T(dt, {
     ScanArgs<scalar> a{};
@@ -1209,10 +1234,13 @@ at::Tensor ssd_prompt(const at::Tensor& xbc, const at::Tensor& dt_in, const at::
     a.q_ld = a.k_ld = a.v_ld = C;
     a.q_hs = a.k_hs = (int)N;
     a.per_group = (int)(H / groups);
-    a.dt = PTR(dt_in);
-    a.dt_ld = dt_in.stride(0);
-    a.dt_bias = PTR(dt_bias);
-    a.a_log = PTR(a_log);
+    step_cumsum_kernel<scalar>
+        <<<dim3(ceil_div_i(max_len, 4 * TB), n, ceil_div_i(H, 64)), dim3(256), 0, stream>>>(
+            PTR(dt_in), dt_in.stride(0), PTR(dt_bias), PTR(a_log), cu.data_ptr<int>(), (int)H,
+            (int)T, steps.data_ptr<float>(), sums.data_ptr<float>());
+    a.steps = steps.data_ptr<float>();
+    a.sums = sums.data_ptr<float>();
+    a.n_tok = (int)T;
     a.d_skip = PTR(d_skip);
     a.cu = cu.data_ptr<int>();
     a.slot = OPT_I(slot);
