@@ -13,7 +13,7 @@ mixers, hyper-connections) and decoded through
 
 from __future__ import annotations
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 from typing import Any
 
 import torch
@@ -29,6 +29,9 @@ from automodel_amd.ops.packed_step import PackedStep
 from automodel_amd.ops.rms_norm import RMSNorm
 from automodel_amd.serving.decode_linear import project
 from automodel_amd.utils.kv_cache import MixerStateCache, active_kv_cache
+
+
+MIXERS = ("parallel", "wkv")
 
 
 def _rope_scaling(scaling: dict | None) -> tuple | None:
@@ -71,17 +74,16 @@ class PapidraConfig:
     conv_kernel: int = 4
     wkv_head_dim: int = 64
     num_wkv_heads: int | None = None
-    _kinds: tuple = field(default=("parallel", "wkv"), repr=False)
 
     def __post_init__(self):
         if self.layers is None:
-            self.layers = [self._uniform_layer(self._kinds[i % 2])
+            self.layers = [self._uniform_layer(MIXERS[i % 2])
                            for i in range(self.num_hidden_layers)]
         self.num_hidden_layers = len(self.layers)
         if self.streams < 1:
             raise ValueError("at least one residual stream")
         for i, layer in enumerate(self.layers):
-            if layer.get("type") not in self._kinds:
+            if layer.get("type") not in MIXERS:
                 raise ValueError(f"layer {i}: unknown mixer type {layer.get('type')!r}")
             mlp = layer.get("mlp")
             if mlp is not None and mlp.get("kind") != "dense":

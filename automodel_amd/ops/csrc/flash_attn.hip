@@ -47,7 +47,8 @@ template <int DQK, int DV, int WAVES, bool VARLEN>
 __global__ __launch_bounds__(WAVES * WAVE_SIZE, 2) void flash_fwd_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k, const bf16* __restrict__ v,
     bf16* __restrict__ out, float* __restrict__ lse, const int* __restrict__ doc_start,
-    const bf16* __restrict__ sink, int B, int Sq, int Skv, int Hq, int Hk, int q_start, float scale, bool causal) {
+    const bf16* __restrict__ sink, int B, int Sq, int Skv, int Hq, int Hk, int q_start,
+    float scale, bool causal) {
   constexpr int KB = pad256(DQK * 2);     // K tile row stride (bytes)
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* k_lds = smem;                               // KVBLK*KB

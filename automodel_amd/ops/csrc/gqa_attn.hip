@@ -220,8 +220,8 @@ __global__ __launch_bounds__(256) void gqa_decode_attn_kernel(
   float m = -INFINITY, l = 0.f;
   const bf16* kb = reinterpret_cast<const bf16*>(cache.k) +
                    (((long)max(sl, 0) * G + g) * cache.rows + lo) * kd + lg * 8;
-  const bf16* vb = reinterpret_cast<const bf16*>(cache.v) +
-                   ((long)max(sl, 0) * G + g) * (cache.rows / 32) * (long)vd * 32 + lo * 32 + lg * 8;
+  const bf16* vb = reinterpret_cast<const bf16*>(cache.v) + lo * 32 + lg * 8 +
+                   ((long)max(sl, 0) * G + g) * (cache.rows / 32) * (long)vd * 32;
   for (int b = b0; b < b1; ++b) {
     gqa_bf16x8 kf[2][KT], vf[VT];
 #pragma unroll
@@ -229,7 +229,8 @@ __global__ __launch_bounds__(256) void gqa_decode_attn_kernel(
 #pragma unroll
       for (int c = 0; c < KT; ++c)
         if (c < kt)
-          kf[i][c] = *reinterpret_cast<const gqa_bf16x8*>(kb + (long)(b * 32 + i * 16) * kd + c * 32);
+          kf[i][c] =
+              *reinterpret_cast<const gqa_bf16x8*>(kb + (long)(b * 32 + i * 16) * kd + c * 32);
 #pragma unroll
     for (int c = 0; c < VT; ++c)
       if (c < vt)

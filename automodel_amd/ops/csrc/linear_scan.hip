@@ -629,7 +629,8 @@ struct SsdOperands<bf16, KT> {
     scan_bf16x8 k8[KT];                            // the tokens' keys, twice
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
-      const scan_s16x4 k4 = *reinterpret_cast<const scan_s16x4*>(kt_ + (kt * 16 + lo) * TD + lg * 4);
+      const scan_s16x4 k4 =
+          *reinterpret_cast<const scan_s16x4*>(kt_ + (kt * 16 + lo) * TD + lg * 4);
       k8[kt] = __builtin_bit_cast(scan_bf16x8,
                                   __builtin_shufflevector(k4, k4, 0, 1, 2, 3, 4, 5, 6, 7));
     }
