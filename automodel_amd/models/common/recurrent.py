@@ -17,7 +17,12 @@ from automodel_amd.ops.linear_scan import (
     wkv_scan,
 )
 from automodel_amd.ops.packed_step import PackedStep
-from automodel_amd.serving.decode_linear import grouped_rows, project, project_grouped
+from automodel_amd.serving.decode_linear import (
+    DecodeLinear,
+    grouped_rows,
+    project,
+    project_grouped,
+)
 
 
 @dataclass(frozen=True)
@@ -99,25 +104,21 @@ class TimeMixing(nn.Module):
         return {"shift": torch.zeros(n_slots, self.mu.shape[1], device=device, dtype=dtype),
                 "wkv": torch.zeros(n_slots, self.heads, self.dim, self.dim, device=device)}
 
-    def _project(self, xs: torch.Tensor) -> list[torch.Tensor]:
-        n = self.heads * self.dim
-        if self.rank <= n:
-            return project_grouped(self.in_proj, xs, n)
-        parts = self.in_proj.weight.split([n] * 4 + [self.rank])
-        return [nn.functional.linear(x, w) for x, w in zip(xs, parts)]
-
     def forward(self, h: torch.Tensor, step: PackedStep, state=None) -> torch.Tensor:
         shift, wkv = (state["shift"], state["wkv"]) if state else (None, None)
-        n = self.heads * self.dim
+        sizes = [self.heads * self.dim] * 4 + [self.rank]
         xs = token_shift(h, self.mu, step, shift)
         if not step.prompt:
-            proj = grouped_rows(self.in_proj, xs, n) if self.rank <= n else None
+            if type(self.decay_proj) not in (nn.Linear, DecodeLinear):
+                # the decode kernel multiplies by the raw weight
+                raise RuntimeError("merge adapters on decay_proj before decoding with a cache")
+            proj = grouped_rows(self.in_proj, xs, sizes)
             if proj is None:
-                proj = torch.cat(self._project(xs), dim=-1)
+                proj = torch.cat(project_grouped(self.in_proj, xs, sizes), dim=-1)
             o = wkv_decode(proj, self.decay_proj.weight, self.decay_bias, self.bonus,
                            self.norm_weight, self.eps, step, wkv)
             return project(self.o_proj, o)
-        r, k, v, g, low = self._project(xs)
+        r, k, v, g, low = project_grouped(self.in_proj, xs, sizes)
         low = project(self.decay_proj, torch.tanh(low), out_f32=True)
         o = wkv_scan(r, k, v, low, self.decay_bias, self.bonus, step, wkv)
         o = gated_group_norm(o, g, self.norm_weight, self.heads, self.eps, gate_first=False)

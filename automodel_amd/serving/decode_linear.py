@@ -72,28 +72,34 @@ def project(lin: nn.Module, x: torch.Tensor, relu2: bool = False,
     return rn.relu2(y) if relu2 else y
 
 
-def project_grouped(lin: nn.Module, xs: torch.Tensor, group: int) -> list[torch.Tensor]:
-    """Several inputs through one stacked projection: rows [i * group, (i+1) *
-    group) of the weight apply to xs[i], xs [n, T, K]; the last part may be
-    smaller. -> the n outputs [T, <= group].
+def project_grouped(lin: nn.Module, xs: torch.Tensor, sizes: list[int]) -> list[torch.Tensor]:
+    """Several inputs through one stacked projection: the weight's rows, split by
+    ``sizes``, apply to xs[i] each, xs [n, T, K]. -> the n outputs [T, sizes[i]].
 
     Up to 64 bf16 rows on the GPU are one launch (the outputs are slices of one
-    [T, N] tensor then, see ``grouped_rows``); more take a GEMM each."""
-    y = grouped_rows(lin, xs, group)
+    [T, N] tensor then, see ``grouped_rows``); more take a GEMM each. A wrapped
+    layer (adapters) sees every input as a whole."""
+    y = grouped_rows(lin, xs, sizes)
     if y is not None:
-        return list(y.split(group, dim=1))
-    return [F.linear(x, w) for x, w in zip(xs, lin.weight.split(group))]
+        return list(y.split(sizes, dim=1))
+    if type(lin) not in (nn.Linear, DecodeLinear):
+        return [lin(x).split(sizes, dim=-1)[i] for i, x in enumerate(xs)]
+    return [F.linear(x, w) for x, w in zip(xs, lin.weight.split(sizes))]
 
 
-def grouped_rows(lin: nn.Module, xs: torch.Tensor, group: int) -> torch.Tensor | None:
-    """The one-launch form of ``project_grouped``, [T, N], if it applies."""
+def grouped_rows(lin: nn.Module, xs: torch.Tensor, sizes: list[int]) -> torch.Tensor | None:
+    """The one-launch form of ``project_grouped``, [T, N], if it applies: equal
+    sizes, of which the last may be smaller."""
     from automodel_amd.ops import residual_norm as rn
 
     n, T, K = xs.shape
-    w = lin.weight
+    group = sizes[0]
     if not (rn.use_hip(xs) and xs.dtype == torch.bfloat16 and 1 <= T <= 64 and K % 8 == 0
-            and group % (2 if T <= 4 else 16) == 0 and -(-w.shape[0] // group) == n):
+            and type(lin) in (nn.Linear, DecodeLinear) and lin.bias is None
+            and sizes[:-1] == [group] * (n - 1) and 1 <= sizes[-1] <= group
+            and group % (2 if T <= 4 else 16) == 0):
         return None
+    w = lin.weight
     from automodel_amd.ops._backend import hip_ops
 
     x = xs.reshape(n * T, K)

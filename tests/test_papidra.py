@@ -613,15 +613,17 @@ def test_states_remember_for_long(dev, dt):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("rows", [1, 3, 4, 5, 16, 33, 64, 65])
-@pytest.mark.parametrize("group,rank,k", [(32, 16, 8), (48, 48, 72), (144, 5, 2048), (7, 3, 24)])
+@pytest.mark.parametrize("group,rank,k", [(32, 16, 8), (48, 48, 72), (144, 5, 2048), (7, 3, 24),
+                                          (16, 40, 64)])
 @torch.no_grad()
 def test_grouped_projection(rows, group, rank, k):
     from automodel_amd.serving.decode_linear import project_grouped
 
     lin = torch.nn.Linear(k, 4 * group + rank, bias=False).bfloat16()
     x = randn(5, rows, k).bfloat16()
-    got = project_grouped(lin.cuda(), x.cuda(), group)
-    for y, xi, w in zip(got, x.double(), lin.weight.detach().double().cpu().split(group)):
+    got = project_grouped(lin.cuda(), x.cuda(), [group] * 4 + [rank])
+    parts = lin.weight.detach().double().cpu().split([group] * 4 + [rank])
+    for y, xi, w in zip(got, x.double(), parts):
         assert rel(y, xi @ w.T) < 1e-2
 
 
@@ -971,3 +973,30 @@ def test_training_forward_and_gradients(model_of, dev, dt):
               "l3.mix.right.conv", "l4.mlp.gate", "embed"):
         e = (grads[k].double().cpu() - w[k].grad).norm() / w[k].grad.norm()
         assert e < (1e-4 if dt == "float32" else 0.15), (k, float(e))
+
+
+@torch.no_grad()
+def test_adapters_on_the_stacked_projection(checkpoints):
+    """A wrapped projection is used as a whole; what decoding reads as a raw
+    weight refuses a wrapper."""
+    class Wrapped(torch.nn.Module):
+        def __init__(self, lin, extra):
+            super().__init__()
+            self.lin, self.extra = lin, extra
+
+        def forward(self, x):
+            return self.lin(x) + x @ self.extra.T
+
+    m = load_pretrained(checkpoints("wkv-only"), dtype="float32", device="cpu")
+    ids = ids_of("wkv-only", 20)
+    mixer = m.model.layers[0].mixer
+    extra = 0.05 * randn(*mixer.in_proj.weight.shape)
+    mixer.in_proj = Wrapped(mixer.in_proj, extra)
+    got = by_parts(m, ids, 9)
+    mixer.in_proj = mixer.in_proj.lin
+    assert rel(by_parts(m, ids, 9), got) > 1e-3
+    mixer.in_proj.weight += extra
+    assert rel(by_parts(m, ids, 9), got) < 1e-5
+    mixer.decay_proj = Wrapped(mixer.decay_proj, torch.zeros_like(mixer.decay_proj.weight))
+    with pytest.raises(RuntimeError, match="adapters"):
+        by_parts(m, ids, 9)
